@@ -866,6 +866,261 @@ int32_t qllm_apply_presence_penalty_rows(float* logits, size_t row_stride,
 int32_t qllm_mark_presence(uint8_t* emitted, const uint32_t* tokens,
                            uint32_t token_count, uint32_t count, void* stream);
 
+/* ---- mixed-layer decoders -------------------------------------------------------
+ *
+ * Kernels of decoders whose layers differ: windowed attention with mixed heads
+ * beside recurrent layers, bf16 weights, a parallel mixer and feed-forward on
+ * one residual stream.  No counterpart in the reference.  Sizes and constants
+ * are parameters throughout; `element` says what activations and cached keys
+ * and values are stored as (F32 mode computes every product in true 32-bit).
+ * The residual stream, norms, positions and angles, scores and attention
+ * weights, decays and recurrent states are F32 in both modes.
+ *
+ * Kernels that depend on where a pass stands read it from three device words
+ * when they run - first position, request slot, rows - so a captured pass is
+ * replayed as the request advances. */
+
+enum qllm_element { QLLM_ELEMENT_BF16 = 0, QLLM_ELEMENT_F32 = 1 };
+
+enum qllm_activation {
+  QLLM_ACTIVATION_GELU_TANH = 0,
+  QLLM_ACTIVATION_SILU = 1
+};
+
+/* bf16 weights in fragment order: one fragment is 16 rows x 32 columns, 1 KiB,
+ * in the lane order of a v_mfma_f32_16x16x32_bf16 operand (lane 16g + n = row
+ * n, columns 8g .. 8g + 7); fragments of a 16-row tile follow each other along
+ * the columns.  Rows are padded to 16, columns to 64 (with zeros), so tiles of
+ * several matrices over the same columns concatenate. */
+size_t qllm_linear_packed_bytes(uint32_t rows, uint32_t columns);
+
+/* Packs row-major bf16 [rows, columns] into a packed matrix of
+ * `packed_columns` (a multiple of 64) columns: row tile t goes to tile
+ * first_tile + t * tile_stride (stride 2 interleaves two matrices, as the
+ * gated epilogue needs), its columns start at first_column (a multiple of 64:
+ * two matrices side by side take a concatenated input).  Fragments it covers
+ * only in part are zero outside the matrix. */
+int32_t qllm_linear_pack(const void* source_bf16, uint32_t rows,
+                         uint32_t columns, void* packed,
+                         uint32_t packed_columns, uint32_t first_tile,
+                         uint32_t tile_stride, uint32_t first_column,
+                         void* stream);
+
+enum qllm_linear_epilogue {
+  QLLM_LINEAR_STORE = 0,    /* output f32 [m][n] = product */
+  QLLM_LINEAR_ADD = 1,      /* output f32 [m][n] += product */
+  /* row tiles alternate between two matrices (gate, up): output element
+   * [m][n] = activation(gate product) * up product; n < rows / 2 */
+  QLLM_LINEAR_GATED = 2,
+  /* output f32 [split][m][n]: the product cut along K in `splits` parts, which
+   * the norm that follows adds (qllm_stream_norm).  At most 64 batch rows. */
+  QLLM_LINEAR_PARTIALS = 3
+};
+
+/* One matrix of a batched launch: output = input x weights^T. */
+typedef struct qllm_linear_segment {
+  const void* weights;       /* packed */
+  const void* input;         /* element [m][input_stride], 16-byte aligned rows */
+  void* output;
+  uint32_t rows;             /* packed rows, a multiple of 16 (gated: of 32) */
+  uint32_t columns;          /* packed columns, a multiple of 64 */
+  uint32_t input_stride;     /* elements; at least `columns`, a multiple of 8 */
+  uint32_t output_stride;    /* elements; a multiple of 4 */
+  uint32_t output_columns;   /* columns stored (the rest is padding) */
+  uint32_t epilogue;
+  uint32_t activation;
+  uint32_t splits;           /* PARTIALS only, 1 .. 16 */
+} qllm_linear_segment;
+
+/* Up to 8 segments in one launch, the same `batch` input rows for all of them.
+ * bf16: up to 64 rows stream the weights once with K cut over a workgroup's
+ * waves, more rows go through the tall tiles.  F32: plain 32-bit
+ * multiply-adds. */
+int32_t qllm_linear_batch(const qllm_linear_segment* segments, uint32_t count,
+                          uint32_t batch, uint32_t element, void* stream);
+
+/* x[row] = table[token] * scale; a token outside the table gives zeros. */
+int32_t qllm_embedding_bf16_batch(const void* table_bf16, uint32_t vocabulary,
+                                  const uint32_t* tokens, float* output,
+                                  uint32_t rows, uint32_t width, float scale,
+                                  void* stream);
+
+/* The head of a parallel layer: stream = input + the `partials` K-split partial
+ * sums of the projection before it (f32 [partials][rows][partial_stride],
+ * written to `stream_out` when there are any), then up to two RMS norms of it
+ * with their own weights, padded with zeros to their strides.  With `shift` the
+ * first output is `shift->count` blends of every row's first norm with that of
+ * the row before it, each to its own buffer: norm + (before - norm) * mu[s];
+ * row 0 takes `previous` of the request's slot ([slot][slot_stride] f32, all
+ * zeros at the start of a sequence) and the last row's norm is left in `last`.
+ * `gather`, when given, lists the input row of every output row. */
+typedef struct qllm_token_shift {
+  uint32_t count;              /* 1 .. 6 */
+  const float* mu[6];          /* f32 [width] */
+  void* output[6];             /* element [rows][stride] */
+  const float* previous;       /* f32, of slot 0 */
+  uint64_t slot_stride;        /* floats between slots */
+  float* last;                 /* f32 [width] */
+} qllm_token_shift;
+
+typedef struct qllm_stream_norm_launch {
+  const float* input;          /* f32 [rows][width] */
+  float* stream_out;           /* f32 [rows][width]; not `input` */
+  const float* partials;
+  uint32_t partial_count;
+  uint32_t partial_stride;
+  const float* weight[2];      /* f32 [width]; NULL = no such output */
+  void* output[2];             /* element [rows][stride] */
+  uint32_t stride[2];
+  uint32_t rows;
+  uint32_t width;
+  float epsilon;
+  uint32_t element;
+  const qllm_token_shift* shift;
+  const uint32_t* gather;      /* device, [rows] */
+  const uint32_t* step;        /* device words; needed with `shift` */
+} qllm_stream_norm_launch;
+int32_t qllm_stream_norm(const qllm_stream_norm_launch* launch, void* stream);
+
+/* ---- windowed attention with mixed heads ---------------------------------- */
+
+/* Geometry of one attention layer.  A page holds, from layer_offset on, the
+ * layer's keys [kv_heads][page_tokens / 16][key_stride / 32][16][32] and then
+ * its values [kv_heads][page_tokens / 32][value_stride][32], both in fragment
+ * order (keys: 16 tokens x 32 dimensions; values transposed: 16 dimensions x
+ * 32 tokens), elements as `element` says.
+ * Position i sees j if j <= i and (i - j < window or j < sinks); window 0 =
+ * every earlier position.  Softmax weights of all heads are mixed before they
+ * meet the values: head h uses sum_g head_mix[h][g] * weight_g. */
+typedef struct qllm_windowed_attention {
+  uint32_t query_heads, kv_heads;
+  uint32_t dim, vdim;
+  uint32_t key_stride;         /* dim padded to 32 */
+  uint32_t value_stride;       /* vdim padded to 16 */
+  uint32_t window, sinks;
+  float scale;
+  const float* head_mix;       /* device f32 [heads][heads]; NULL = none */
+  uint32_t page_tokens;        /* a multiple of 32 */
+  uint32_t pages_per_slot;
+  uint64_t layer_offset;       /* bytes */
+  void* const* page_table;     /* device [slots][pages_per_slot] */
+  const uint32_t* step;        /* device words */
+  uint32_t element;
+} qllm_windowed_attention;
+
+size_t qllm_windowed_layer_bytes(uint32_t page_tokens, uint32_t kv_heads,
+                                 uint32_t key_stride, uint32_t value_stride,
+                                 uint32_t element);
+
+/* Rotates the query and key rows of a pass (pair 2i, 2i + 1 by position *
+ * frequencies[i], i < rotary_dims / 2), blends values with those of an earlier
+ * layer (v + (first - v) * share, when `first_values` is given), stores keys
+ * and values into the pages and leaves the queries in `query_out`, element
+ * [rows][query_heads][key_stride].  projections: f32 rows of `stride` floats
+ * with query, key and value columns at the given offsets.  `values_out`, when
+ * given, keeps the unblended value rows f32 [rows][kv_heads * vdim]. */
+typedef struct qllm_rope_store_launch {
+  const float* projections;
+  uint32_t stride, query_column, key_column, value_column;
+  uint32_t rotary_dims;
+  const double* frequencies;   /* device [rotary_dims / 2] */
+  const float* first_values;
+  const float* value_share;    /* device scalar */
+  float* values_out;
+  void* query_out;
+  uint32_t rows;
+} qllm_rope_store_launch;
+int32_t qllm_windowed_rope_store(const qllm_windowed_attention* attention,
+                                 const qllm_rope_store_launch* launch,
+                                 void* stream);
+
+/* Attention of `rows` consecutive positions over the pages (their own keys and
+ * values included): output element [rows][output_stride], head h's vdim values
+ * at h * vdim, multiplied by sigmoid(gate[row][h]) when `gate` (f32, rows of
+ * gate_stride floats) is given.  bf16: one to four rows split the context over
+ * workgroups (decode), more rows take the prompt kernel; head counts or sizes
+ * outside those kernels (see qllm_windowed_attention_form) and F32 go through
+ * the general kernel. */
+typedef struct qllm_attention_launch {
+  const void* query;           /* from qllm_windowed_rope_store */
+  const float* gate;
+  uint32_t gate_stride;
+  void* output;
+  uint32_t output_stride;
+  uint32_t rows;
+  uint32_t maximum_position;   /* no row's position exceeds it (sizes grids) */
+  void* workspace;
+  size_t workspace_bytes;
+} qllm_attention_launch;
+size_t qllm_windowed_attention_workspace_bytes(
+    const qllm_windowed_attention* attention, uint32_t maximum_position);
+enum qllm_attention_form {
+  QLLM_ATTENTION_GENERAL = 0,
+  QLLM_ATTENTION_SPLIT = 1,
+  QLLM_ATTENTION_PROMPT = 2
+};
+/* Which kernel a launch of `rows` rows takes. */
+uint32_t qllm_windowed_attention_form(const qllm_windowed_attention* attention,
+                                      uint32_t rows);
+int32_t qllm_windowed_attention_rows(const qllm_windowed_attention* attention,
+                                     const qllm_attention_launch* launch,
+                                     void* stream);
+
+/* ---- recurrent layers ------------------------------------------------------ */
+
+/* A per-head matrix state [dim (key)][dim (value)], F32, carried from token to
+ * token.  r, k, v: rows of a token's projections.
+ *   DELTA: u = k / sqrt(sum k^2 + unit_epsilon), a = sigmoid(rate + bias),
+ *          w = exp(decay_scale * sigmoid(inner)), decay_scale < 0:
+ *          S <- diag(w) S - (a u) (u^T S) + k v^T;  o = S^T r
+ *   BONUS: w = exp(-exp(inner)):
+ *          o = (S + diag(bonus) k v^T)^T r;  S <- diag(w) S + k v^T
+ * inner = W2 tanh(low) + base, with low the rank-sized projection. */
+enum qllm_recurrence_kind { QLLM_RECURRENCE_DELTA = 0, QLLM_RECURRENCE_BONUS = 1 };
+enum qllm_gate_kind { QLLM_GATE_SIGMOID = 0, QLLM_GATE_SILU = 1 };
+
+typedef struct qllm_recurrence {
+  uint32_t kind;
+  uint32_t heads, dim;         /* dim <= 256 */
+  uint32_t rank;               /* of the decay's low-rank projection */
+  uint32_t gate_kind;
+  float epsilon;               /* output norm */
+  float unit_epsilon;
+  float decay_scale;
+  const void* decay_up_bf16;   /* W2 [heads * dim][rank], row-major */
+  const float* decay_base;     /* [heads * dim] */
+  const float* rate_bias;      /* DELTA: [heads * dim] */
+  const float* bonus;          /* BONUS: [heads * dim] */
+  const float* norm_weight;    /* [heads * dim] */
+  float* state;                /* [slot][heads][dim][dim], of slot 0 */
+  uint64_t slot_stride;        /* floats between slots */
+  const uint32_t* step;        /* device words */
+  uint32_t element;
+} qllm_recurrence;
+
+/* `rows` tokens: output element [rows][output_stride] = o / rms(o) * norm *
+ * gate.  projections: f32 rows of `stride` floats with the given columns.
+ * One row is a single launch; more rows go through preparation, scan and
+ * finish over `workspace`.  carry_from / carry_to (token shift): `width` floats
+ * copied to the slot's carry state at the end, when given. */
+typedef struct qllm_recurrence_launch {
+  const float* projections;
+  uint32_t stride;
+  uint32_t r_column, k_column, v_column, gate_column, rate_column, low_column;
+  void* output;
+  uint32_t output_stride;
+  uint32_t rows;
+  const float* carry_from;
+  float* carry_to;             /* of slot 0; slot_stride floats between slots */
+  uint32_t carry_width;
+  void* workspace;
+  size_t workspace_bytes;
+} qllm_recurrence_launch;
+size_t qllm_recurrence_workspace_bytes(const qllm_recurrence* recurrence,
+                                       uint32_t rows);
+int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
+                             const qllm_recurrence_launch* launch, void* stream);
+
 /* ---- synthetic data (benchmarks and tests) ------------------------------------- */
 
 /* Fill device memory from a counter-based generator (splitmix64 of seed and

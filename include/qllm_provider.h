@@ -324,6 +324,44 @@ int32_t qllm_artifact_tensor(qllm_artifact* artifact, const char* name,
                              int32_t check_header, const void** record,
                              uint64_t* record_bytes);
 
+/* ---- opened models -------------------------------------------------------------
+ *
+ * A model of any stored form (artifact directory or model folder) driven batch
+ * by batch through its compiled program: what the worker does per request, for
+ * hosts that want logits as well.  kv_cache_dtype as the worker's launch option
+ * (NULL = "artifact"); chunk_rows 0 = the provider's own batch limit. */
+typedef struct qllm_model qllm_model;
+qllm_model* qllm_model_open(const char* path, uint32_t max_context,
+                            uint32_t capacity, uint32_t kv_page_tokens,
+                            const char* kv_cache_dtype, uint32_t chunk_rows);
+void qllm_model_close(qllm_model* model);
+uint32_t qllm_model_vocabulary(const qllm_model* model);
+uint32_t qllm_model_hidden(const qllm_model* model);
+uint32_t qllm_model_batch_limit(const qllm_model* model);
+
+/* A request of its own slot; the id is positive and never reused.  Parameters
+ * as a BEGIN line's SAMPLING group; temperature 0 = greedy. */
+int32_t qllm_model_begin(qllm_model* model, uint32_t temperature_ppm,
+                         uint32_t top_p_ppm, uint32_t top_k, uint32_t min_p_ppm,
+                         int32_t presence_ppm, uint64_t seed,
+                         uint32_t first_output_position, uint64_t* request);
+int32_t qllm_model_end(qllm_model* model, uint64_t request);
+
+/* The request's next `count` tokens (any number); logits f32 [wanted_count]
+ * [vocabulary] of the wanted places among them (ascending) when wanted_count
+ * is not 0; next_token = the head's selection after the last one. */
+int32_t qllm_model_step(qllm_model* model, uint64_t request,
+                        const uint32_t* tokens, uint32_t count,
+                        const uint32_t* wanted, uint32_t wanted_count,
+                        float* logits, uint32_t* next_token);
+/* The same tokens one program operation at a time, and the residual stream
+ * after every layer: hidden f32 [layers][count][hidden].  count is at most
+ * qllm_model_batch_limit(). */
+int32_t qllm_model_trace_layers(qllm_model* model, uint64_t request,
+                                const uint32_t* tokens, uint32_t count,
+                                float* hidden, uint32_t* next_token);
+uint64_t qllm_model_telemetry(const qllm_model* model, const char* name);
+
 #ifdef __cplusplus
 }
 #endif

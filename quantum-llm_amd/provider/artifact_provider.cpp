@@ -292,6 +292,58 @@ er::CreateExecutionProviderModuleResult make_mi355_dense_fp4_callable_provider(
   }
 }
 
+er::CreateExecutionProviderModuleResult make_mi355_mixed_module(
+    const er::ModelDescriptor& model, std::shared_ptr<er::IModelTensorStore> tensors,
+    const ArtifactProviderOptions& options) {
+  try {
+    if (!tensors) return {invalid("model tensors are absent"), {}};
+    if (options.routed_vram_policy != "fixed")
+      return {invalid("a dense resident provider has no routed VRAM policy but "
+                      "\"fixed\""),
+              {}};
+    auto metadata = make_mi355_mixed_provider();
+    if (auto status = er::provider_supports_model(model, metadata.capabilities);
+        !status.ok())
+      return {status, {}};
+    MixedGeometry geometry;
+    geometry.hidden = model.hidden_size;
+    geometry.vocabulary = model.vocab_size;
+    geometry.max_context =
+        options.max_context ? options.max_context : model.max_context_tokens;
+    if (geometry.max_context > model.max_context_tokens)
+      return {invalid("requested context exceeds the model's maximum"), {}};
+    geometry.kv_page_tokens = options.kv_page_tokens;
+    geometry.capacity = std::max(1U, options.capacity);
+    geometry.chunk_rows = options.chunk_rows;
+    if (options.kv_cache_dtype == "fp32")
+      geometry.element = QLLM_ELEMENT_F32;
+    else if (options.kv_cache_dtype != "artifact" && options.kv_cache_dtype != "bf16")
+      return {invalid("unsupported KV cache dtype: " + options.kv_cache_dtype), {}};
+
+    auto implementation = std::make_shared<Mi355MixedProvider>(geometry);
+    er::ExecutionProviderModule module;
+    module.definition = {metadata.name, metadata.priority,
+                         std::move(metadata.capabilities), implementation};
+    module.tensor_store = std::move(tensors);
+    module.service = implementation->service_contract();
+    module.service.vram_cache_bytes = options.vram_cache_bytes;
+    module.service.routed_vram_policy = options.routed_vram_policy;
+    module.telemetry = [implementation] { return implementation->telemetry(); };
+    // pages, states and workspaces follow from all operations together
+    module.finalize_service =
+        [implementation](er::ExecutionProviderModule::ServiceContract& service) {
+          if (auto status = implementation->finalize(); !status.ok()) return status;
+          service.kv_page_bytes = implementation->service_contract().kv_page_bytes;
+          return er::Status::success();
+        };
+    return {er::Status::success(), std::move(module)};
+  } catch (const std::exception& error) {
+    return {{er::ErrorCode::internal,
+             std::string("mixed-layer provider creation failed: ") + error.what()},
+            {}};
+  }
+}
+
 er::Status prepare_program(const er::ModelDescriptor& model,
                            const er::ExecutionProviderModule& module,
                            PreparedProgram& prepared) {

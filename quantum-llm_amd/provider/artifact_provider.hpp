@@ -7,6 +7,7 @@
 #pragma once
 
 #include "dense_fp4_provider.hpp"
+#include "mixed_provider.hpp"
 #include "expert/runtime/model_artifact.hpp"
 #include "expert/runtime/model_tensor_store.hpp"
 
@@ -24,12 +25,14 @@ namespace qllm {
 struct ArtifactProviderOptions final {
   std::uint32_t max_context{};      // 0 = the artifact's max_context_tokens
   std::uint32_t kv_page_tokens{256};
-  // "q4-f16-per-head" (also chosen by "artifact") or "fp16"
+  // dense FP4: "q4-f16-per-head" (also chosen by "artifact") or "fp16";
+  // mixed layers: "bf16" (also chosen by "artifact") or "fp32"
   std::string kv_cache_dtype{"artifact"};
   std::uint32_t mtp_draft_depth{};  // 0 = the artifact's declared depth
   std::uint64_t vram_cache_bytes{1};  // echoed in the service contract
   std::string routed_vram_policy{"fixed"};
   std::uint32_t capacity{1};        // request slots
+  std::uint32_t chunk_rows{};       // mixed layers: rows per batch, 0 = default
   bool profile_gpu_phases{};        // provider_gpu_*_ns telemetry, uncaptured passes
 };
 
@@ -67,6 +70,13 @@ make_mi355_dense_fp4_callable_provider(
 [[nodiscard]] er::CreateExecutionProviderModuleResult
 make_mi355_dense_fp4_module(std::shared_ptr<er::ModelArtifact> artifact,
                             const ArtifactProviderOptions& options);
+
+// The module of the mixed-layer provider for a described model and its tensors
+// (a model folder).  kv_cache_dtype "fp32" runs the model in true 32-bit,
+// "bf16" (also chosen by "artifact") in bf16 with F32 accumulation.
+[[nodiscard]] er::CreateExecutionProviderModuleResult make_mi355_mixed_module(
+    const er::ModelDescriptor& model, std::shared_ptr<er::IModelTensorStore> tensors,
+    const ArtifactProviderOptions& options);
 
 // What the common VM's start-up does with a module
 // (ExecutionProviderRegistry::add / bind, then the preparation loop of

@@ -1,5 +1,7 @@
 #include "dense_fp4_provider.hpp"
 
+#include "host_support.hpp"
+
 #include <hip/hip_runtime.h>
 
 #include <algorithm>
@@ -13,62 +15,9 @@
 namespace qllm {
 namespace {
 
-constexpr std::uint32_t kMaximumGpuSamplingTopK = 64U;  // provider.cpp:8359
 constexpr std::uint32_t kMaximumDraftDepth = 7U;
 
-void hip_check(hipError_t error, const char* what) {
-  if (error != hipSuccess)
-    throw std::runtime_error(std::string(what) + ": " +
-                             hipGetErrorString(error));
-}
-
-void status_check(std::int32_t status) {
-  if (status != QLLM_OK) throw std::runtime_error(qllm_last_error());
-}
-
 std::uint32_t pad32(std::uint32_t value) { return (value + 31U) / 32U * 32U; }
-
-// A device allocation that is freed unless release() hands it on.
-class DeviceBuffer final {
- public:
-  DeviceBuffer(std::size_t bytes, const char* what) {
-    hip_check(hipMalloc(&pointer_, bytes), what);
-  }
-  ~DeviceBuffer() {
-    if (pointer_) (void)hipFree(pointer_);
-  }
-  DeviceBuffer(const DeviceBuffer&) = delete;
-  DeviceBuffer& operator=(const DeviceBuffer&) = delete;
-  [[nodiscard]] void* get() const noexcept { return pointer_; }
-  [[nodiscard]] void* release() noexcept {
-    void* pointer = pointer_;
-    pointer_ = nullptr;
-    return pointer;
-  }
-
- private:
-  void* pointer_{};
-};
-
-std::uint64_t request_parameter(const er::ProgramRequestContext& request,
-                                std::string_view name) {
-  const auto found = request.parameters.find(name);
-  if (found == request.parameters.end())
-    throw std::runtime_error("request parameter is absent: " +
-                             std::string(name));
-  return found->second;
-}
-
-// The penalty a request asks for: the parameter is biased by 2,000,000 ppm so
-// that negative penalties travel as unsigned values
-// (runtime/tools/moe_vm_runner.cpp:318-347, dense_fp4_provider.cpp:8336-8341).
-double presence_penalty_of(const er::ProgramRequestContext& request) {
-  const auto biased =
-      request_parameter(request, "sampling_presence_penalty_biased_ppm");
-  if (biased > 4'000'000U)
-    throw std::runtime_error("sampling presence penalty is invalid");
-  return (static_cast<double>(biased) - 2'000'000.0) / 1'000'000.0;
-}
 
 er::ExactDecodeExecutionHandle completed_exact(
     er::ExactDecodeExecutionResult result) {
@@ -83,20 +32,6 @@ er::ExactDecodeExecutionHandle completed_exact(
       [shared]() { shared->reset(); });
 }
 
-const er::ImmutableModelTensor& tensor_for(
-    std::span<const er::PreparedTensorBinding> tensors, std::string_view role) {
-  for (const auto& binding : tensors)
-    if (binding.role == role && binding.tensor) return *binding.tensor;
-  throw std::runtime_error("tensor role is not bound: " + std::string(role));
-}
-
-const er::ImmutableModelTensor* optional_tensor(
-    std::span<const er::PreparedTensorBinding> tensors, std::string_view role) {
-  for (const auto& binding : tensors)
-    if (binding.role == role && binding.tensor) return binding.tensor.get();
-  return nullptr;
-}
-
 // The role the artifact compiler binds (compiler/expert_pack/adapters.py:
 // 1422-1602: "weight", "input_norm", "norm"), or the longer name that hosts
 // without an artifact use for the same tensor.
@@ -106,41 +41,6 @@ const er::ImmutableModelTensor& tensor_for_either(
   if (const auto* tensor = optional_tensor(tensors, role)) return *tensor;
   if (const auto* tensor = optional_tensor(tensors, other_role)) return *tensor;
   throw std::runtime_error("tensor role is not bound: " + std::string(role));
-}
-
-// Value ABIs between operations as the artifact declares them
-// (dense_fp4_provider.cpp:59-74).  The hidden-state ABI string names F32 rows
-// in device memory; the memory domain says whose device.
-constexpr std::string_view kHiddenAbi = "batch.hidden.f32.cuda.v1";
-constexpr std::string_view kTokenAbi = "batch.token-id.u32.host.v1";
-constexpr std::string_view kPositionAbi = "batch.position.u32.host.v1";
-constexpr std::string_view kDeviceDomain = "hip.device";
-
-// :550-564
-std::span<const std::uint32_t> host_u32_batch(const er::ExecutionValue& value,
-                                              std::string_view abi,
-                                              std::string_view description) {
-  if (!value.valid() || value.abi != abi || value.memory_domain != "host" ||
-      value.bytes % sizeof(std::uint32_t) != 0U ||
-      value.bytes / sizeof(std::uint32_t) > 1024U ||
-      reinterpret_cast<std::uintptr_t>(value.data) % alignof(std::uint32_t) != 0U)
-    throw std::runtime_error(std::string(description) + " ABI mismatch");
-  return {reinterpret_cast<const std::uint32_t*>(value.data),
-          static_cast<std::size_t>(value.bytes / sizeof(std::uint32_t))};
-}
-
-// :5605-5620
-er::OperationExecutionHandle completed_operation(
-    er::OperationExecutionResult result) {
-  auto shared = std::make_shared<std::optional<er::OperationExecutionResult>>(
-      std::move(result));
-  return er::OperationExecutionHandle::from_callbacks(
-      [shared]() {
-        auto value = std::move(*shared);
-        shared->reset();
-        return value;
-      },
-      [shared]() { shared->reset(); });
 }
 
 er::Status validate_parameters(
@@ -261,9 +161,8 @@ void Mi355DenseFp4Provider::release() {
     (void)hipHostFree(staging_);
     staging_ = nullptr;
   }
-  for (auto& slot : slots_)
-    for (void* page : slot.pages)
-      if (page) (void)hipFree(page);
+  selector_.reset();
+  kv_slots_ = {};
   slots_.clear();
   for (auto& events : gpu_event_pool_) {
     (void)hipEventDestroy(static_cast<hipEvent_t>(events.start));
@@ -404,9 +303,9 @@ void Mi355DenseFp4Provider::allocate_workspaces() {
   select_workspace_bytes_ = std::max(
       std::max(head_maxima_bytes,
                qllm_argmax_workspace_bytes(g_.vocabulary, max_rows_)),
-      std::max(qllm_topk_workspace_bytes(g_.vocabulary, kMaximumGpuSamplingTopK),
+      std::max(qllm_topk_workspace_bytes(g_.vocabulary, TokenSelector::kMaximumTopK),
                qllm_topk_batch_workspace_bytes(g_.vocabulary,
-                                               kMaximumGpuSamplingTopK, max_rows_)));
+                                               TokenSelector::kMaximumTopK, max_rows_)));
   select_workspace_ = device_alloc(select_workspace_bytes_);
   argmax_tokens_ = static_cast<std::uint32_t*>(device_alloc(rows * 4U));
   presence_ = static_cast<std::uint8_t*>(device_alloc(g_.vocabulary));
@@ -414,12 +313,8 @@ void Mi355DenseFp4Provider::allocate_workspaces() {
   hip_check(hipMemset(presence_, 0, g_.vocabulary), "clear presence bytes");
   hip_check(hipMemset(proposal_presence_, 0, g_.vocabulary),
             "clear presence bytes");
-  mark_tokens_ = static_cast<std::uint32_t*>(device_alloc(8U * 4U));
-  // top-k logits of up to 8 rows, then their tokens: one buffer, one readback
-  top_logits_ = static_cast<float*>(
-      device_alloc(8U * kMaximumGpuSamplingTopK * (4U + 4U)));
-  top_tokens_ = reinterpret_cast<std::uint32_t*>(
-      top_logits_ + 8U * kMaximumGpuSamplingTopK);
+  selector_ = std::make_unique<TokenSelector>(stream_, g_.vocabulary, select_workspace_,
+                                              select_workspace_bytes_);
 
   if (g_.mtp_layers) {
     mtp_tokens_ = static_cast<std::uint32_t*>(device_alloc((8U + 4U) * 4U));
@@ -453,10 +348,9 @@ void Mi355DenseFp4Provider::allocate_workspaces() {
                      qllm_q8_layer_bytes(g_.kv_page_tokens, g_.kv_heads, g_.head_dim);
   const std::size_t page_count =
       (g_.max_context + g_.kv_page_tokens - 1U) / g_.kv_page_tokens;
-  slots_.resize(std::max(1U, g_.capacity));
+  kv_slots_ = RequestSlots(g_.capacity, page_count, kv_page_bytes_);
+  slots_.resize(kv_slots_.capacity());
   for (auto& slot : slots_) {
-    slot.leased = std::make_shared<std::atomic<bool>>(false);
-    slot.pages.assign(page_count, nullptr);
     if (slots_.size() > 1U) {
       slot.saved_presence = static_cast<std::uint8_t*>(device_alloc(g_.vocabulary));
       hip_check(hipMemset(slot.saved_presence, 0, g_.vocabulary),
@@ -498,8 +392,9 @@ void Mi355DenseFp4Provider::activate(std::uint32_t slot) {
               "load proposer state");
   }
   // a pageable source: the copy has read it when the call returns
-  hip_check(hipMemcpyAsync(device_page_table_, incoming.pages.data(),
-                           incoming.pages.size() * sizeof(void*),
+  const auto& pages = kv_slots_.pages(slot);
+  hip_check(hipMemcpyAsync(device_page_table_, pages.data(),
+                           pages.size() * sizeof(void*),
                            hipMemcpyHostToDevice, stream),
             "load request page table");
   active_slot_ = slot;
@@ -556,20 +451,12 @@ void Mi355DenseFp4Provider::collect_gpu_phases() {
 }
 
 void Mi355DenseFp4Provider::ensure_pages(std::uint32_t last_position) {
-  auto& pages = slots_[active_slot_].pages;
-  const std::size_t last_page = last_position / g_.kv_page_tokens;
-  if (last_page >= pages.size())
-    throw std::runtime_error("KV position exceeds the configured context");
-  for (std::size_t page = 0; page <= last_page; ++page) {
-    if (pages[page]) continue;
-    void* pointer{};
-    hip_check(hipMalloc(&pointer, kv_page_bytes_), "allocate KV page");
-    hip_check(hipMemset(pointer, 0, kv_page_bytes_), "clear KV page");
-    pages[page] = pointer;
-    hip_check(hipMemcpy(device_page_table_ + page, &pointer, sizeof(pointer),
-                        hipMemcpyHostToDevice),
-              "publish KV page");
-  }
+  kv_slots_.ensure(active_slot_, 0U, last_position / g_.kv_page_tokens,
+                   [this](std::size_t page, void* pointer) {
+                     hip_check(hipMemcpy(device_page_table_ + page, &pointer,
+                                         sizeof(pointer), hipMemcpyHostToDevice),
+                               "publish KV page");
+                   });
 }
 
 DeviceFp4Matrix Mi355DenseFp4Provider::upload_matrix(
@@ -942,27 +829,18 @@ Mi355DenseFp4Provider::create_request_state(
     const er::ProgramRequestContext& request) {
   try {
     std::lock_guard lock(mutex_);
-    // the sampling profile check of dense_fp4_provider.cpp:5502-5513
-    const auto temperature = request.parameters.find("sampling_temperature_ppm");
-    if (temperature != request.parameters.end() && temperature->second != 0U) {
-      const auto first = request.parameters.find("sampling_first_output_position");
-      const auto presence =
-          request.parameters.find("sampling_presence_penalty_biased_ppm");
-      if (first == request.parameters.end() || first->second >= g_.max_context ||
-          presence == request.parameters.end() || presence->second > 4'000'000U)
-        throw std::runtime_error("request has an invalid sampling profile");
-    }
+    require_sampling_profile(request, g_.max_context);
     // a free slot, or the reference's answer when every slot is taken
     // (dense_fp4_provider.cpp:5514-5518)
-    std::uint32_t slot = 0U;
-    while (slot < slots_.size() &&
-           slots_[slot].leased->load(std::memory_order_acquire))
-      ++slot;
-    if (slot == slots_.size())
+    const auto grant = kv_slots_.take();
+    if (!grant)
       return {{er::ErrorCode::backpressure,
                "dense FP4 provider has no free request slot"},
               {}};
-    activate(slot);
+    auto state = std::make_shared<DenseFp4RequestState>();
+    state->slot = grant->slot;
+    state->lease = grant->lease;
+    activate(state->slot);
     hip_check(hipMemsetAsync(presence_, 0, g_.vocabulary,
                              static_cast<hipStream_t>(stream_)),
               "zero request sampling presence");
@@ -973,29 +851,10 @@ Mi355DenseFp4Provider::create_request_state(
     if (reserved != request.parameters.end() && reserved->second != 0U)
       ensure_pages(static_cast<std::uint32_t>(
           std::min<std::uint64_t>(reserved->second, g_.max_context) - 1U));
-    auto state = std::make_shared<DenseFp4RequestState>();
-    state->slot = slot;
-    state->lease = slots_[slot].leased;
-    state->lease->store(true, std::memory_order_release);
     return {er::Status::success(), std::move(state)};
   } catch (const std::exception& error) {
     return {{er::ErrorCode::internal, error.what()}, {}};
   }
-}
-
-void Mi355DenseFp4Provider::mark_presence(
-    std::uint8_t* emitted, std::span<const std::uint32_t> tokens) {
-  if (tokens.empty()) return;
-  if (tokens.size() > 8U) throw std::runtime_error("too many presence marks");
-  const auto stream = static_cast<hipStream_t>(stream_);
-  // the pinned words are free: every pass that used them ended with a wait
-  std::copy(tokens.begin(), tokens.end(), staging_->marks);
-  hip_check(hipMemcpyAsync(mark_tokens_, staging_->marks, tokens.size() * 4U,
-                           hipMemcpyHostToDevice, stream),
-            "upload presence marks");
-  status_check(qllm_mark_presence(emitted, mark_tokens_,
-                                  static_cast<std::uint32_t>(tokens.size()),
-                                  g_.vocabulary, stream_));
 }
 
 er::Status Mi355DenseFp4Provider::rebind_request_state(
@@ -1044,93 +903,6 @@ std::uint32_t Mi355DenseFp4Provider::require_hidden_value(
   return static_cast<std::uint32_t>(value.bytes / row_bytes);
 }
 
-// The head's token for a request (run_head with a request, :8433-8517): the
-// presence penalty from the first output position on, arg-max at temperature
-// zero, otherwise top-k or whole-row candidates ordered on the host and one
-// draw from stream 0; an output token is marked as emitted.  logits_ row 0.
-std::uint32_t Mi355DenseFp4Provider::select_head_token(
-    const er::ProgramRequestContext& request, std::uint32_t sample_position) {
-  const auto stream = static_cast<hipStream_t>(stream_);
-  const auto first_output =
-      request_parameter(request, "sampling_first_output_position");
-  const bool output_sampling = sample_position >= first_output;
-  const auto penalty = presence_penalty_of(request);
-  if (output_sampling && penalty != 0.0) {
-    status_check(qllm_apply_presence_penalty(logits_, presence_, g_.vocabulary,
-                                             static_cast<float>(penalty),
-                                             stream_));
-    status_check(qllm_argmax_batch(logits_, g_.vocabulary, 1U, argmax_tokens_,
-                                   select_workspace_, select_workspace_bytes_,
-                                   stream_));
-  }
-  const auto temperature = request_parameter(request, "sampling_temperature_ppm");
-  std::uint32_t selected{};
-  if (temperature == 0U) {
-    hip_check(hipMemcpyAsync(&selected, argmax_tokens_, sizeof(selected),
-                             hipMemcpyDeviceToHost, stream),
-              "copy dense FP4 greedy token");
-    hip_check(hipStreamSynchronize(stream), "copy dense FP4 greedy token");
-    // a row without a finite logit selects nothing (0xffffffff): reported
-    // before the presence bytes or the caller's state change
-    if (selected >= g_.vocabulary)
-      throw std::runtime_error("head logits have no finite maximum");
-  } else {
-    // the penalty, if any, has been applied: the distribution is taken from
-    // the row as it stands
-    er::ProgramRequestContext unpenalised = request;
-    unpenalised.parameters["sampling_presence_penalty_biased_ppm"] = 2'000'000U;
-    const auto top_k = request_parameter(request, "sampling_top_k");
-    if (top_k > kMaximumGpuSamplingTopK) {
-      // the scalar sampler orders that many candidates on the host
-      // (sample_token, :773-799)
-      std::vector<float> row(g_.vocabulary);
-      hip_check(hipMemcpyAsync(row.data(), logits_, row.size() * 4U,
-                               hipMemcpyDeviceToHost, stream),
-                "copy dense FP4 sampling logits");
-      hip_check(hipStreamSynchronize(stream), "copy dense FP4 sampling logits");
-      if (top_k > row.size())
-        throw std::runtime_error("invalid token sampling contract");
-      std::vector<std::uint32_t> candidates(row.size());
-      std::iota(candidates.begin(), candidates.end(), 0U);
-      const auto before = [&](std::uint32_t left, std::uint32_t right) {
-        const float a = row[left];
-        const float b = row[right];
-        if (std::isnan(a)) return false;
-        if (std::isnan(b)) return true;
-        return a == b ? left < right : a > b;
-      };
-      std::partial_sort(candidates.begin(), candidates.begin() + top_k,
-                        candidates.end(), before);
-      candidates.resize(top_k);
-      std::vector<float> ordered;
-      for (const auto candidate : candidates) ordered.push_back(row[candidate]);
-      sampling_logit_transfer_bytes_ += row.size() * 4U;
-      const auto distribution = er::make_sampling_distribution(
-          ordered, candidates, static_cast<std::uint32_t>(temperature),
-          static_cast<std::uint32_t>(
-              request_parameter(request, "sampling_top_p_ppm")),
-          static_cast<std::uint32_t>(
-              request_parameter(request, "sampling_min_p_ppm")));
-      selected = er::sample_distribution(
-          distribution,
-          er::counter_uniform(request_parameter(request, "sampling_seed"),
-                              sample_position, 0U));
-    } else {
-      const auto distribution = distribution_from_logits(
-          logits_, g_.vocabulary, argmax_tokens_, unpenalised, nullptr);
-      selected = er::sample_distribution(
-          distribution,
-          er::counter_uniform(request_parameter(request, "sampling_seed"),
-                              sample_position, 0U));
-    }
-  }
-  if (output_sampling) {
-    const std::uint32_t token[1] = {selected};
-    mark_presence(presence_, token);
-  }
-  return selected;
-}
-
 // One operation of the artifact's program (execute, :10680-10992).
 er::OperationExecutionHandle Mi355DenseFp4Provider::execute(
     const er::IPreparedOperation& opaque_operation,
@@ -1173,7 +945,7 @@ er::OperationExecutionHandle Mi355DenseFp4Provider::execute(
         if (state->synchronization_rows != 0U)
           throw std::runtime_error("previous target batch was not synchronized");
         const auto tokens =
-            host_u32_batch(input("token_ids"), kTokenAbi, "embedding token batch");
+            host_u32_batch(input("token_ids"), kTokenAbi, "embedding token batch", 1024U);
         if (tokens.empty() || tokens.size() > max_rows_)
           throw std::runtime_error("invalid FP4 hidden batch size");
         for (const auto token : tokens)
@@ -1194,7 +966,7 @@ er::OperationExecutionHandle Mi355DenseFp4Provider::execute(
       case PreparedOperation::Kind::attention: {
         const auto rows = require_hidden_value(input("hidden"));
         const auto positions = host_u32_batch(input("positions"), kPositionAbi,
-                                              "attention position batch");
+                                              "attention position batch", 1024U);
         if (positions.size() != rows || rows != state->current_batch_rows)
           throw std::runtime_error("attention batch width changed in program");
         for (std::uint32_t row = 0; row < rows; ++row)
@@ -1240,7 +1012,8 @@ er::OperationExecutionHandle Mi355DenseFp4Provider::execute(
         end_gpu_phase(phase_events);
         collect_gpu_phases();
         auto owner = std::make_shared<std::vector<std::uint32_t>>(
-            1U, select_head_token(invocation.request, state->current_position));
+            1U, selector_->select(logits_, presence_, argmax_tokens_, invocation.request,
+                                  state->current_position));
         outputs.emplace(
             "token_ids",
             er::ExecutionValue{std::string(kTokenAbi), "host", owner,
@@ -2131,7 +1904,8 @@ Mi355DenseFp4Provider::PrefillResult Mi355DenseFp4Provider::prefill(
     if (request.parameters.contains("sampling_temperature_ppm")) {
       // the head under the request's sampling profile, at the position of the
       // prompt's last token (run_head with a request, :8433-8517)
-      predicted = select_head_token(request, first_position + count - 1U);
+      predicted = selector_->select(logits_, presence_, argmax_tokens_, request,
+                                    first_position + count - 1U);
     } else {
       hip_check(hipMemcpyAsync(&predicted, argmax_tokens_, sizeof(predicted),
                                hipMemcpyDeviceToHost, hip_stream),
@@ -2506,121 +2280,6 @@ er::Status Mi355DenseFp4Provider::synchronize() {
 
 // ---- sampling ---------------------------------------------------------------
 
-// distribution_from_logits, dense_fp4_provider.cpp:8331-8391.  top_k == 0
-// selects the whole-vocabulary path of the scalar sampler (sample_token,
-// :773-799): the row is copied to the host and ordered there.
-er::SamplingDistribution Mi355DenseFp4Provider::distribution_from_logits(
-    float* row_logits, std::uint32_t vocabulary, std::uint32_t* device_argmax,
-    const er::ProgramRequestContext& request, const std::uint8_t* presence) {
-  const auto stream = static_cast<hipStream_t>(stream_);
-  const auto penalty = presence_penalty_of(request);
-  const auto temperature = request_parameter(request, "sampling_temperature_ppm");
-  if (penalty != 0.0) {
-    if (!presence) throw std::runtime_error("sampling presence state is absent");
-    status_check(qllm_apply_presence_penalty(row_logits, presence, vocabulary,
-                                             static_cast<float>(penalty),
-                                             stream_));
-    // the arg-max the pass left behind was taken before the penalty
-    if (temperature == 0U)
-      status_check(qllm_argmax_batch(row_logits, vocabulary, 1U, device_argmax,
-                                     select_workspace_, select_workspace_bytes_,
-                                     stream_));
-  }
-  if (temperature == 0U) {
-    std::uint32_t token{};
-    hip_check(hipMemcpyAsync(&token, device_argmax, sizeof(token),
-                             hipMemcpyDeviceToHost, stream),
-              "copy exact greedy token");
-    hip_check(hipStreamSynchronize(stream), "copy exact greedy token");
-    return {{{token, 1.0}}};
-  }
-  const auto top_p = static_cast<std::uint32_t>(
-      request_parameter(request, "sampling_top_p_ppm"));
-  const auto min_p = static_cast<std::uint32_t>(
-      request_parameter(request, "sampling_min_p_ppm"));
-  const auto top_k = request_parameter(request, "sampling_top_k");
-  if (top_k > kMaximumGpuSamplingTopK || top_k > vocabulary)
-    throw std::runtime_error(
-        "sampled exact decode requires top-k of at most 64 (0 = whole row)");
-  std::vector<float> host_logits;
-  std::vector<std::uint32_t> host_tokens;
-  if (top_k == 0U) {
-    std::vector<float> full(vocabulary);
-    hip_check(hipMemcpyAsync(full.data(), row_logits, full.size() * 4U,
-                             hipMemcpyDeviceToHost, stream),
-              "copy logit row");
-    hip_check(hipStreamSynchronize(stream), "copy logit row");
-    host_tokens.resize(vocabulary);
-    std::iota(host_tokens.begin(), host_tokens.end(), 0U);
-    std::sort(host_tokens.begin(), host_tokens.end(),
-              [&](std::uint32_t left, std::uint32_t right) {
-                const float a = full[left];
-                const float b = full[right];
-                if (std::isnan(a)) return false;
-                if (std::isnan(b)) return true;
-                return a == b ? left < right : a > b;
-              });
-    host_logits.reserve(vocabulary);
-    for (const auto token : host_tokens) host_logits.push_back(full[token]);
-    sampling_logit_transfer_bytes_ += full.size() * 4U;
-  } else {
-    return std::move(distributions_from_top_k(row_logits, vocabulary, vocabulary,
-                                              1U, request)
-                         .front());
-  }
-  return er::make_sampling_distribution(
-      host_logits, host_tokens, static_cast<std::uint32_t>(temperature), top_p,
-      min_p);
-}
-
-// The distributions of `rows` rows of logits (row r at logits + r * stride)
-// for a sampled request with 1 <= top_k <= 64: one selection launch for all
-// rows, one readback, then make_sampling_distribution per row
-// (distribution_from_logits, dense_fp4_provider.cpp:8331-8391, which selects
-// and reads back row by row).
-std::vector<er::SamplingDistribution>
-Mi355DenseFp4Provider::distributions_from_top_k(
-    const float* logits, std::uint32_t vocabulary, std::size_t stride,
-    std::uint32_t rows, const er::ProgramRequestContext& request) {
-  const auto stream = static_cast<hipStream_t>(stream_);
-  const auto temperature = request_parameter(request, "sampling_temperature_ppm");
-  const auto top_p = static_cast<std::uint32_t>(
-      request_parameter(request, "sampling_top_p_ppm"));
-  const auto min_p = static_cast<std::uint32_t>(
-      request_parameter(request, "sampling_min_p_ppm"));
-  const auto top_k =
-      static_cast<std::uint32_t>(request_parameter(request, "sampling_top_k"));
-  if (!rows || rows > 8U || !top_k || top_k > kMaximumGpuSamplingTopK ||
-      top_k > vocabulary)
-    throw std::runtime_error(
-        "sampled exact decode requires top-k of at most 64 (0 = whole row)");
-  status_check(qllm_topk_logits_batch(logits, vocabulary, stride, top_k, rows,
-                                      top_logits_, top_tokens_, select_workspace_,
-                                      select_workspace_bytes_, stream_));
-  // logits of all rows, then tokens of all rows (the device buffers are
-  // adjacent with room for 8 rows of 64)
-  constexpr std::size_t kCapacity = 8U * kMaximumGpuSamplingTopK;
-  hip_check(hipMemcpyAsync(staging_->top_logits, top_logits_,
-                           kCapacity * 4U + std::size_t{rows} * top_k * 4U,
-                           hipMemcpyDeviceToHost, stream),
-            "copy speculative top-k");
-  hip_check(hipStreamSynchronize(stream), "copy speculative top-k");
-  ++sampling_gpu_calls_;
-  sampling_logit_transfer_bytes_ += std::size_t{rows} * top_k * 8U;
-  std::vector<er::SamplingDistribution> result;
-  result.reserve(rows);
-  for (std::uint32_t row = 0; row < rows; ++row) {
-    const std::span<const float> row_logits(
-        staging_->top_logits + std::size_t{row} * top_k, top_k);
-    const std::span<const std::uint32_t> row_tokens(
-        staging_->top_tokens + std::size_t{row} * top_k, top_k);
-    result.push_back(er::make_sampling_distribution(
-        row_logits, row_tokens, static_cast<std::uint32_t>(temperature), top_p,
-        min_p));
-  }
-  return result;
-}
-
 // ---- the proposer (run_mtp / extend_mtp_rollout, :8681-8852) -----------------
 
 // The kernels of one proposer pass over the tokens in mtp_tokens_, through the
@@ -2929,7 +2588,7 @@ std::optional<DraftPrediction> Mi355DenseFp4Provider::run_mtp(
 
   DraftPrediction result;
   if (request) {
-    result.distribution = distribution_from_logits(
+    result.distribution = selector_->distribution(
         mtp_logits_, g_.draft_vocabulary, mtp_argmax_, *request, presence);
     result.token = er::sample_distribution(
         result.distribution,
@@ -3022,7 +2681,7 @@ void Mi355DenseFp4Provider::propose_with_graphs(
       launch_mtp_graph(depth ? 1U : rows, depth != 0U);
       DraftPrediction prediction;
       // a request with a presence penalty takes the uncaptured passes
-      prediction.distribution = distribution_from_logits(
+      prediction.distribution = selector_->distribution(
           mtp_logits_, g_.draft_vocabulary, mtp_argmax_, request, nullptr);
       prediction.token = er::sample_distribution(
           prediction.distribution,
@@ -3054,7 +2713,7 @@ void Mi355DenseFp4Provider::extend_mtp_rollout(
   state.draft_predictions.push_back(std::move(first));
   // every draft is present for the drafts after it (:8822-8847)
   const std::uint32_t root[1] = {state.draft_predictions.back().token};
-  mark_presence(proposal_presence_, root);
+  selector_->mark(proposal_presence_, root);
   while (state.draft_predictions.size() < g_.draft_depth &&
          state.mtp_length + 2U < context_limit) {
     // the next pass reads the proposer's own last hidden state before it
@@ -3068,7 +2727,7 @@ void Mi355DenseFp4Provider::extend_mtp_rollout(
     if (!prediction) throw std::runtime_error("MTP rollout produced no proposal");
     state.draft_predictions.push_back(std::move(*prediction));
     const std::uint32_t drafted[1] = {state.draft_predictions.back().token};
-    mark_presence(proposal_presence_, drafted);
+    selector_->mark(proposal_presence_, drafted);
   }
   state.draft_valid = !state.draft_predictions.empty();
   // speculative rows of the proposer's cache are overwritten by the next pass
@@ -3142,14 +2801,14 @@ er::ExactDecodeExecutionHandle Mi355DenseFp4Provider::execute_exact_decode(
       for (std::uint32_t row = 0; row < rows; ++row)
         target_distributions.push_back({{{staging_->download[row], 1.0}}});
     } else if (request_parameter(invocation.request, "sampling_top_k") != 0U) {
-      target_distributions = distributions_from_top_k(
+      target_distributions = selector_->top_k_distributions(
           logits_, g_.vocabulary, g_.vocabulary, rows, invocation.request);
     } else {
       // whole-vocabulary candidates; the penalty has been applied above
       er::ProgramRequestContext unpenalised = invocation.request;
       unpenalised.parameters["sampling_presence_penalty_biased_ppm"] = 2'000'000U;
       for (std::uint32_t row = 0; row < rows; ++row)
-        target_distributions.push_back(distribution_from_logits(
+        target_distributions.push_back(selector_->distribution(
             logits_ + std::size_t{row} * g_.vocabulary, g_.vocabulary,
             argmax_tokens_ + row, unpenalised, nullptr));
     }
@@ -3192,7 +2851,7 @@ er::ExactDecodeExecutionHandle Mi355DenseFp4Provider::execute_exact_decode(
       for (std::size_t index = 0; index < accepted; ++index)
         emitted_now.push_back(state->draft_predictions[index].token);
       emitted_now.push_back(next_token);
-      mark_presence(presence_, emitted_now);
+      selector_->mark(presence_, emitted_now);
     }
     if (mtp_.ready) {
       // advance the proposer over the accepted drafts and the next token (row r
@@ -3442,7 +3101,7 @@ er::Status Mi355DenseFp4Provider::copy_mtp_state(float* host_last_hidden,
 er::Status Mi355DenseFp4Provider::copy_kv_page(std::uint32_t page_index,
                                                void* host_output) {
   std::lock_guard lock(mutex_);
-  const auto& pages_ = slots_[active_slot_].pages;
+  const auto& pages_ = kv_slots_.pages(active_slot_);
   if (!host_output || page_index >= pages_.size())
     return {er::ErrorCode::invalid_argument, "KV page index is invalid"};
   auto status = hipStreamSynchronize(static_cast<hipStream_t>(stream_));
@@ -3465,9 +3124,9 @@ Mi355DenseFp4Provider::telemetry() const {
   values["provider_exact_calls"] = exact_calls_;
   values["provider_accepted_drafts"] = accepted_drafts_;
   values["provider_program_steps"] = program_steps_;
-  values["provider_sampling_gpu_calls"] = sampling_gpu_calls_;
+  values["provider_sampling_gpu_calls"] = selector_->gpu_calls();
   values["provider_sampling_logit_transfer_bytes"] =
-      sampling_logit_transfer_bytes_;
+      selector_->logit_transfer_bytes();
   for (std::size_t depth = 0; depth < accepted_depth_calls_.size(); ++depth)
     values["provider_accepted_depth_" + std::to_string(depth)] =
         accepted_depth_calls_[depth];
@@ -3571,7 +3230,7 @@ Mi355DenseFp4Provider::service_contract() const {
   contract.kv_allocation = "paged_on_demand";
   contract.kv_page_tokens = g_.kv_page_tokens;
   contract.kv_page_bytes = kv_page_bytes_;
-  contract.kv_page_capacity = slots_.size() * slots_.front().pages.size();
+  contract.kv_page_capacity = kv_slots_.capacity() * kv_slots_.pages_per_slot();
   contract.placement_mode = "resident";
   contract.placement_profile = "resident";
   contract.ram_cache_bytes = 0U;

@@ -19,7 +19,10 @@
 #include <string>
 #include <vector>
 
+#include "decoder_provider.hpp"
 #include "qllm_kernels.h"
+#include "request_slots.hpp"
+#include "token_selector.hpp"
 #include "expert/runtime/program_executor.hpp"
 #include "expert/runtime/worker_provider.hpp"
 #include "expert/runtime/speculative_sampling.hpp"
@@ -144,7 +147,7 @@ struct MtpWeights final {
   qllm_fp4_matrix head_prefix{};   // the first draft_vocabulary rows of the head
 };
 
-class Mi355DenseFp4Provider final : public er::IOperationProvider {
+class Mi355DenseFp4Provider final : public DecoderProvider {
  public:
   explicit Mi355DenseFp4Provider(const DenseGeometry& geometry);
   ~Mi355DenseFp4Provider() override;
@@ -237,16 +240,16 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
   [[nodiscard]] const DenseGeometry& geometry() const noexcept { return g_; }
   // The tall prompt path takes bf16 activations; with Q8 activations a prompt
   // goes through the program in row batches.
-  [[nodiscard]] bool supports_tall_prefill() const noexcept {
+  [[nodiscard]] bool supports_tall_prefill() const noexcept override {
     return !g_.activation_q8;
   }
-  [[nodiscard]] bool profiles_gpu_phases() const noexcept {
+  [[nodiscard]] bool profiles_gpu_phases() const noexcept override {
     return g_.profile_gpu_phases;
   }
   [[nodiscard]] std::map<std::string, std::uint64_t, std::less<>> telemetry()
-      const;
+      const override;
   [[nodiscard]] er::ExecutionProviderModule::ServiceContract service_contract()
-      const;
+      const override;
 
   // Prompt prefill: runs `tokens` (positions first_position ..) through the
   // target in chunks of up to prefill_chunk_rows() rows - the linears on the
@@ -259,14 +262,10 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
   // (runtime/tools/moe_vm_runner.cpp:682-745), and the first drafts are rolled
   // out: the state is then ready for execute_exact_decode at
   // first_position + tokens.size() with the prediction as guaranteed token.
-  struct PrefillResult final {
-    er::Status status;
-    std::uint32_t predicted{};
-  };
   [[nodiscard]] PrefillResult prefill(
       const std::shared_ptr<er::IOperationProviderRequestState>& state,
       std::span<const std::uint32_t> tokens, std::uint32_t first_position,
-      const er::ProgramRequestContext& request);
+      const er::ProgramRequestContext& request) override;
   [[nodiscard]] std::uint32_t prefill_chunk_rows() const noexcept {
     return g_.prefill_chunk_rows ? g_.prefill_chunk_rows : 32768U;
   }
@@ -316,11 +315,6 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
                                const std::uint16_t* input, float* logits,
                                std::uint32_t rows, std::uint32_t* tokens,
                                const qllm_rollout_step* advance);
-  // run_head with a request (dense_fp4_provider.cpp:8433-8517): presence
-  // penalty, arg-max or sampling of the single head row in logits_, the
-  // emitted token marked
-  std::uint32_t select_head_token(const er::ProgramRequestContext& request,
-                                  std::uint32_t sample_position);
   [[nodiscard]] er::ExecutionValue device_hidden_value(std::uint32_t rows) const;
   [[nodiscard]] std::uint32_t require_hidden_value(
       const er::ExecutionValue& value) const;
@@ -334,8 +328,6 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
   // is saved into the outgoing slot and loaded from the incoming one - a page
   // table upload and two small device copies on the provider's stream.
   struct RequestSlot final {
-    std::shared_ptr<std::atomic<bool>> leased;
-    std::vector<void*> pages;        // this slot's page pointers (host view)
     std::uint8_t* saved_presence{};  // [vocabulary], capacity > 1 only
     float* saved_last_hidden{};      // [hidden], proposer, capacity > 1 only
   };
@@ -367,15 +359,6 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
                                    std::uint64_t seed, bool tiled);
   void enqueue_target(const std::uint32_t* device_tokens, std::uint32_t rows,
                       std::uint32_t first_position, bool deferred_positions);
-  std::vector<er::SamplingDistribution> distributions_from_top_k(
-      const float* logits, std::uint32_t vocabulary, std::size_t stride,
-      std::uint32_t rows, const er::ProgramRequestContext& request);
-  er::SamplingDistribution distribution_from_logits(
-      float* row_logits, std::uint32_t vocabulary, std::uint32_t* device_argmax,
-      const er::ProgramRequestContext& request, const std::uint8_t* presence);
-  // emitted[token] = 1 for every token (one upload, one launch)
-  void mark_presence(std::uint8_t* emitted,
-                     std::span<const std::uint32_t> tokens);
   // One proposer pass over `tokens` (run_mtp, dense_fp4_provider.cpp:8681-
   // 8792): row r embeds tokens[r], takes previous_hidden row r (device, F32),
   // is cached at position mtp_length + r and rotated at mtp_length + r + 1.
@@ -431,6 +414,7 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
   MtpWeights mtp_;
 
   // KV cache
+  RequestSlots kv_slots_;            // leases and pages
   std::vector<RequestSlot> slots_;
   std::uint32_t active_slot_{};
   void** device_page_table_{};
@@ -462,9 +446,6 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
     std::uint32_t target[12];
     std::uint32_t proposer[12];
     std::uint32_t download[8];
-    float top_logits[8 * 64];            // top-k readback: logits of all rows,
-    std::uint32_t top_tokens[8 * 64];    // then their tokens
-    std::uint32_t marks[8];              // tokens whose presence byte is set
   };
   HostStaging* staging_ = nullptr;
   float* projection_partials_ = nullptr;   // [splits][rows][hidden]
@@ -496,9 +477,7 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
   // request at a time, as the KV cache is.
   std::uint8_t* presence_{};
   std::uint8_t* proposal_presence_{};
-  std::uint32_t* mark_tokens_{};
-  float* top_logits_{};
-  std::uint32_t* top_tokens_{};
+  std::unique_ptr<TokenSelector> selector_;
 
   // proposer workspaces
   std::uint32_t* mtp_tokens_{};
@@ -540,8 +519,6 @@ class Mi355DenseFp4Provider final : public er::IOperationProvider {
   std::uint64_t accepted_drafts_{};
   std::vector<std::uint64_t> accepted_depth_calls_;
   std::uint64_t program_steps_{};
-  std::uint64_t sampling_gpu_calls_{};
-  std::uint64_t sampling_logit_transfer_bytes_{};
   std::uint64_t mtp_passes_{};
   std::uint64_t mtp_rows_{};
 };

@@ -240,6 +240,20 @@ std::uint64_t Value::u64(std::string_view where) const {
   wrong_type(where, "a non-negative integer");
 }
 
+double Value::number(std::string_view where) const {
+  if (const auto* value = std::get_if<std::uint64_t>(&data_))
+    return static_cast<double>(*value);
+  if (const auto* value = std::get_if<std::int64_t>(&data_))
+    return static_cast<double>(*value);
+  if (const auto* value = std::get_if<Real>(&data_)) {
+    double result{};
+    const char* const end = value->token.data() + value->token.size();
+    const auto [stop, error] = std::from_chars(value->token.data(), end, result);
+    if (error == std::errc{} && stop == end) return result;
+  }
+  wrong_type(where, "a number");
+}
+
 Value parse(std::string_view text) { return Reader(text).document(); }
 
 const Value& required(const Object& object, std::string_view key,

@@ -40,6 +40,11 @@ class Value final {
   [[nodiscard]] const std::string& string(std::string_view where) const;
   [[nodiscard]] bool boolean(std::string_view where) const;
   [[nodiscard]] std::uint64_t u64(std::string_view where) const;
+  // any number, rounded to double
+  [[nodiscard]] double number(std::string_view where) const;
+  [[nodiscard]] bool null() const noexcept {
+    return std::holds_alternative<std::nullptr_t>(data_);
+  }
 
  private:
   Storage data_;

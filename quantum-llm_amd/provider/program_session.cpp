@@ -53,6 +53,8 @@ ProgramSession::Outputs ProgramSession::execute(
                 {}};
       values[endpoint.value_index] = std::move(found->second);
     }
+    if (provider_->supports_program_sequence(program))
+      return execute_sequence(values);
     for (std::size_t index = 0; index < program.operations.size(); ++index) {
       const auto& compiled = program.operations[index];
       std::vector<er::ExecutionValue> operands;
@@ -101,6 +103,39 @@ ProgramSession::Outputs ProgramSession::execute(
              std::string("model execution failed: ") + error.what()},
             {}};
   }
+}
+
+// The whole program in one invocation, for providers that take it so: inputs
+// and outputs in the order the compiled program lists them.
+ProgramSession::Outputs ProgramSession::execute_sequence(
+    std::span<const er::ExecutionValue> values) {
+  const auto& program = prepared_->bound.program;
+  std::vector<const er::IPreparedOperation*> operations;
+  for (const auto& operation : prepared_->operations) operations.push_back(operation.get());
+  std::vector<er::ExecutionValue> operands;
+  for (const auto& endpoint : program.inputs)
+    operands.push_back(values[endpoint.value_index]);
+  auto handle = provider_->execute_program_sequence(
+      state_, er::ProgramSequenceInvocation{request_, program, operations, operands});
+  if (!handle.valid()) return {rejected("operation provider rejected invocation"), {}};
+  std::optional<er::OperationExecutionResult> result;
+  while (!(result = handle.poll())) {
+  }
+  if (!result->status.ok()) return {result->status, {}};
+  if (result->outputs.size() != program.outputs.size())
+    return {{er::ErrorCode::internal, "operation provider returned a partial output set"},
+            {}};
+  Outputs outputs;
+  outputs.status = er::Status::success();
+  for (std::size_t port = 0; port < program.outputs.size(); ++port) {
+    const auto& endpoint = program.outputs[port];
+    if (!result->outputs[port].valid() ||
+        result->outputs[port].abi != program.values.at(endpoint.value_index).abi)
+      return {{er::ErrorCode::internal, "operation provider returned an invalid output ABI"},
+              {}};
+    outputs.values.emplace(endpoint.role, std::move(result->outputs[port]));
+  }
+  return outputs;
 }
 
 bool ProgramSession::exact_decode_available() const noexcept {

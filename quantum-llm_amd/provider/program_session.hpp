@@ -58,6 +58,7 @@ class ProgramSession final {
 
  private:
   ProgramSession() = default;
+  [[nodiscard]] Outputs execute_sequence(std::span<const er::ExecutionValue> values);
   const er::ModelDescriptor* model_{};
   const PreparedProgram* prepared_{};
   std::shared_ptr<er::IOperationProvider> provider_;

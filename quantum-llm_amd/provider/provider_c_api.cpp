@@ -49,6 +49,12 @@ int32_t from_status(const er::Status& status) {
 
 }  // namespace
 
+namespace qllm {
+int32_t provider_fail(int32_t code, const std::string& message) {
+  return fail(code, message);
+}
+}  // namespace qllm
+
 extern "C" const char* qllm_provider_last_error(void) { return last_error; }
 
 extern "C" qllm_provider* qllm_provider_create(

@@ -1,17 +1,17 @@
-// Worker process for the MI355X dense FP4 provider: the line protocol of the
+// Worker process for the MI355X providers: the line protocol of the
 // reference's native runner (runtime/tools/moe_vm_runner.cpp, protocol 13) on
 // stdin / stdout, so that the service above it (ops/python/expert_server.py,
 // CudaWorker :489) talks to this worker unchanged.
 //
-//   usage: qllm-worker <artifact> --worker --max-context=N --ram-cache-gib=N
+//   usage: qllm-worker <artifact or model folder> --worker --max-context=N --ram-cache-gib=N
 //            --vram-cache-gib=N --capacity=N --kv-cache-mib=N --kv-page-tokens=N
 //            --placement-profile=latency|balanced|capacity
-//            [--kv-cache-dtype=artifact|q4-f16-per-head|fp16]
+//            [--kv-cache-dtype=artifact|q4-f16-per-head|fp16|bf16|fp32]
 //            [--mtp-draft-depth=N] [--routed-vram-policy=fixed]
 //            [--prefill-chunk-limit=N] [--profile-gpu-phases]
 //
-// Structure: Engine is what every request runs on (model, prepared program,
-// provider, the program's token ports); Request owns one conversation - its
+// Structure: Engine is what every request runs on (the opened model, its
+// provider, the batch limit); Request owns one conversation - its
 // program session, the token the model has predicted but not yet emitted, its
 // position and limit - and moves it forward by prompt, by speculative step,
 // by plain step or by its closing token; Service maps each command verb to a
@@ -31,10 +31,8 @@
 #include "expert/runtime/model_artifact.hpp"
 #include "expert/runtime/program_executor.hpp"
 
-#include "artifact_provider.hpp"
-#include "dense_fp4_provider.hpp"
 #include "launch_contract.hpp"
-#include "program_session.hpp"
+#include "model_host.hpp"
 #include "wire.hpp"
 
 #include <algorithm>
@@ -61,8 +59,6 @@ using wire::expect;
 using wire::FieldCursor;
 using wire::JsonLine;
 
-constexpr std::string_view kTokenAbi = "batch.token-id.u32.host.v1";
-constexpr std::string_view kPositionAbi = "batch.position.u32.host.v1";
 constexpr char kNoRetention[] = "callable provider does not support session retention";
 constexpr char kNoPersistence[] =
     "callable provider does not support session persistence";
@@ -150,31 +146,25 @@ enum class StepMode : std::uint8_t { decode = 0, finish = 1, plain = 2 };
 // requests, changed by none.
 class Engine final {
  public:
-  Engine(const er::ModelDescriptor& model, const er::ExecutionProviderModule& module,
-         const PreparedProgram& prepared, const LaunchOptions& options)
-      : model_(model), module_(module), prepared_(prepared) {
-    provider_ = std::dynamic_pointer_cast<Mi355DenseFp4Provider>(
-        module.definition.implementation);
-    expect(provider_ != nullptr, "callable provider module has no implementation");
-    find_ports();
-    chunk_ = std::max<std::uint32_t>(1U, module.service.prefill_chunk_tokens);
+  Engine(const ModelHost& host, const LaunchOptions& options) : host_(host) {
+    chunk_ = std::max<std::uint32_t>(1U, host.batch_limit());
     if (options.prefill_chunk_limit)
       chunk_ = std::min(chunk_, *options.prefill_chunk_limit);
   }
 
-  [[nodiscard]] const er::ModelDescriptor& model() const noexcept { return model_; }
+  [[nodiscard]] const er::ModelDescriptor& model() const noexcept { return host_.model(); }
   [[nodiscard]] const er::ExecutionProviderModule& module() const noexcept {
-    return module_;
+    return host_.module();
   }
-  [[nodiscard]] const PreparedProgram& prepared() const noexcept { return prepared_; }
-  [[nodiscard]] Mi355DenseFp4Provider& provider() const noexcept { return *provider_; }
+  [[nodiscard]] const ModelHost& host() const noexcept { return host_; }
+  [[nodiscard]] DecoderProvider& provider() const noexcept { return host_.provider(); }
   [[nodiscard]] std::uint32_t chunk_tokens() const noexcept { return chunk_; }
 
   // Whether a request with this profile may be decoded speculatively
   // (moe_vm_runner.cpp:670-676): greedy always, sampled only through the
   // version-2 exact-decode contract with a top-k the device selection serves.
   [[nodiscard]] bool speculative(const SamplingProfile& profile) const noexcept {
-    const auto& decode = model_.exact_decode_program;
+    const auto& decode = model().exact_decode_program;
     if (!decode) return false;
     if (profile.greedy()) return true;
     return decode->abi_version >= 2U && profile.top_k >= 1U && profile.top_k <= 64U;
@@ -185,63 +175,13 @@ class Engine final {
   [[nodiscard]] std::uint32_t run(ProgramSession& session,
                                   std::span<const std::uint32_t> tokens,
                                   std::uint32_t first_position) const {
-    std::vector<std::uint32_t> positions(tokens.size());
-    for (std::uint32_t row = 0U; row < positions.size(); ++row)
-      positions[row] = first_position + row;
-    std::map<std::string, er::ExecutionValue, std::less<>> inputs;
-    inputs.emplace(token_input_, words(tokens, kTokenAbi));
-    inputs.emplace(position_input_, words(positions, kPositionAbi));
-    auto outputs = session.execute(std::move(inputs));
-    expect_ok(outputs.status);
-    const auto found = outputs.values.find(token_output_);
-    expect(found != outputs.values.end(),
-           "model program did not publish its token output");
-    const er::ExecutionValue& value = found->second;
-    expect(value.valid() && value.abi == kTokenAbi && value.memory_domain == "host" &&
-               value.bytes != 0U && value.bytes % sizeof(std::uint32_t) == 0U,
-           "callable VM returned an invalid token value");
-    std::uint32_t last{};
-    std::memcpy(&last, value.data + (value.bytes - sizeof(last)), sizeof(last));
-    return last;
+    const auto result = host_.run(session, tokens, first_position);
+    expect_ok(result.status);
+    return result.token;
   }
 
  private:
-  static er::ExecutionValue words(std::span<const std::uint32_t> values,
-                                  std::string_view abi) {
-    auto storage =
-        std::make_shared<std::vector<std::uint32_t>>(values.begin(), values.end());
-    const auto* bytes = reinterpret_cast<const std::byte*>(storage->data());
-    return {std::string(abi), "host", storage, bytes,
-            storage->size() * sizeof(std::uint32_t)};
-  }
-
-  // The token-step service ABI (moe_vm_runner.cpp:297-316): exactly a token
-  // and a position input and one token output.
-  void find_ports() {
-    const auto claim = [](std::string& port, const std::string& role,
-                          std::string_view complaint) {
-      expect(port.empty(), complaint);
-      port = role;
-    };
-    for (const auto& [role, endpoint] : model_.program_inputs) {
-      if (endpoint.abi == kTokenAbi)
-        claim(token_input_, role, "multiple token program inputs");
-      else if (endpoint.abi == kPositionAbi)
-        claim(position_input_, role, "multiple position program inputs");
-    }
-    for (const auto& [role, endpoint] : model_.program_outputs)
-      if (endpoint.abi == kTokenAbi)
-        claim(token_output_, role, "multiple token program outputs");
-    expect(model_.program_inputs.size() == 2U && !token_input_.empty() &&
-               !position_input_.empty() && !token_output_.empty(),
-           "artifact does not implement the token-step service ABI");
-  }
-
-  const er::ModelDescriptor& model_;
-  const er::ExecutionProviderModule& module_;
-  const PreparedProgram& prepared_;
-  std::shared_ptr<Mi355DenseFp4Provider> provider_;
-  std::string token_input_, position_input_, token_output_;
+  const ModelHost& host_;
   std::uint32_t chunk_{1U};
 };
 
@@ -258,8 +198,7 @@ class Request final {
     context.parameters["sampling_first_output_position"] = prompt_tokens - 1U;
     context.parameters["exact_decode_enabled"] = speculative_ ? 1U : 0U;
     profile.publish(context.parameters);
-    expect_ok(ProgramSession::begin(engine.model(), engine.module(), engine.prepared(),
-                                    std::move(context), session_));
+    expect_ok(engine.host().begin(std::move(context), session_));
     speculative_ = speculative_ && session_->exact_decode_available();
   }
 
@@ -650,19 +589,6 @@ class Service final {
 
 int run(int argc, char** argv) {
   const auto options = parse_launch_options(argc, argv);
-  auto artifact = std::make_shared<er::ModelArtifact>();
-  expect_ok(er::ModelArtifact::load(std::filesystem::path(argv[1]), *artifact));
-  if (options.mtp_draft_depth)
-    expect_ok(artifact->configure_mtp_draft_depth(*options.mtp_draft_depth));
-  const er::ModelDescriptor& model = artifact->model();
-  require(model.schema_version >= 3U,
-          "callable VM service requires a schema v3 artifact");
-  // exactly one module must cover the program (moe_vm_runner.cpp:431-497);
-  // this worker links one
-  require(er::provider_supports_model(model,
-                                      make_mi355_dense_fp4_provider().capabilities)
-              .ok(),
-          "no callable provider implements the artifact program");
   ArtifactProviderOptions provider_options;
   provider_options.max_context = options.max_context;
   provider_options.capacity = options.capacity;
@@ -671,14 +597,12 @@ int run(int argc, char** argv) {
   provider_options.vram_cache_bytes = options.vram_cache_gib << 30U;
   provider_options.routed_vram_policy = options.routed_vram_policy;
   provider_options.profile_gpu_phases = options.profile_gpu_phases;
-  auto created = make_mi355_dense_fp4_module(artifact, provider_options);
-  expect_ok(created.status);
-  PreparedProgram prepared;
-  expect_ok(prepare_program(model, created.module, prepared));
-  if (created.module.finalize_service)
-    expect_ok(created.module.finalize_service(created.module.service));
-  check_service_contract(model, created.module, options);
-  const Engine engine(model, created.module, prepared, options);
+  if (options.mtp_draft_depth)
+    provider_options.mtp_draft_depth = *options.mtp_draft_depth;
+  std::unique_ptr<ModelHost> host;
+  expect_ok(ModelHost::open(std::filesystem::path(argv[1]), provider_options, host));
+  check_service_contract(host->model(), host->module(), options);
+  const Engine engine(*host, options);
   return Service(engine, options).serve(std::cin, std::cout);
 }
 
