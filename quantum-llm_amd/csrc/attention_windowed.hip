@@ -367,11 +367,11 @@ __global__ __launch_bounds__(256) void split_scores_kernel(AttentionArgs args) {
 
 constexpr uint32_t kMixRow = 40;   // bf16 values per LDS row of mixed weights (32 + pad)
 
-// NV = value_stride / 16.
-template <int NV>
+// NV = value_stride / 16, GROUP = query heads per key/value head at most.
+template <int NV, int GROUP>
 __global__ __launch_bounds__(256) void split_values_kernel(AttentionArgs args) {
   __shared__ float row_maximum[64], row_inverse[64];
-  __shared__ float mix[16][64];
+  __shared__ __attribute__((aligned(16))) float mix[64][GROUP];
   __shared__ __attribute__((aligned(16))) uint16_t mixed[4][16 * kMixRow];
   __shared__ f32x4 gathered[NV * kWave];
   const Attention& a = args.attention;
@@ -384,22 +384,30 @@ __global__ __launch_bounds__(256) void split_values_kernel(AttentionArgs args) {
   const uint32_t wave = threadIdx.x / kWave;
   const uint32_t lane = threadIdx.x % kWave;
 
-  for (uint32_t h = threadIdx.x; h < heads; h += blockDim.x) {
-    const float* pairs =
-        args.maxima + (size_t{row} * args.score_splits * heads + h) * 2u;
+  // a wave per head, a lane per score split (at most 64)
+#pragma unroll 4
+  for (uint32_t h = wave; h < heads; h += 4u) {
     float m = -INFINITY;
-    for (uint32_t s = 0; s < args.score_splits; ++s)
-      m = fmaxf(m, pairs[size_t{s} * heads * 2u]);
     float t = 0.0f;
-    for (uint32_t s = 0; s < args.score_splits; ++s)
-      t += pairs[size_t{s} * heads * 2u + 1u] * expf(pairs[size_t{s} * heads * 2u] - m);
-    row_maximum[h] = m;
-    row_inverse[h] = 1.0f / t;
+    if (lane < args.score_splits) {
+      const float* pair =
+          args.maxima + ((size_t{row} * args.score_splits + lane) * heads + h) * 2u;
+      m = pair[0];
+      t = pair[1];
+    }
+    const float top = wave_max(m);
+    t = wave_sum(t * expf(m - top));
+    if (lane == 0u) {
+      row_maximum[h] = top;
+      row_inverse[h] = 1.0f / t;
+    }
   }
-  for (uint32_t i = threadIdx.x; i < group * heads; i += blockDim.x) {
-    const uint32_t h = kv * group + i / heads;
-    mix[i / heads][i % heads] =
-        a.head_mix ? a.head_mix[size_t{h} * heads + i % heads] : (h == i % heads ? 1.0f : 0.0f);
+  for (uint32_t i = threadIdx.x; i < heads * GROUP; i += blockDim.x) {
+    const uint32_t g = i / GROUP;
+    const uint32_t in_group = i % GROUP;
+    const uint32_t h = kv * group + min(in_group, group - 1u);
+    const float value = a.head_mix ? a.head_mix[size_t{h} * heads + g] : (h == g ? 1.0f : 0.0f);
+    mix[g][in_group] = in_group < group ? value : 0.0f;
   }
   for (uint32_t i = threadIdx.x; i < 4u * 16u * kMixRow; i += blockDim.x)
     mixed[0][i] = 0u;
@@ -421,21 +429,28 @@ __global__ __launch_bounds__(256) void split_values_kernel(AttentionArgs args) {
     // lane: key lane % 32, heads of parity lane / 32
     const float* scores = args.scores + size_t{row} * heads * args.capacity +
                           size_t{ordinal} * kTileKeys + lane % 32u;
-    float share[16] = {};
-    for (uint32_t g = lane / 32u; g < heads; g += 2u) {
-      const float p =
-          expf(scores[size_t{g} * args.capacity] - row_maximum[g]) * row_inverse[g];
+    float share[GROUP] = {};
+    for (uint32_t g0 = lane / 32u; g0 < heads; g0 += 16u) {
+      float raw[8];
 #pragma unroll
-      for (int h = 0; h < 16; ++h)
-        if (static_cast<uint32_t>(h) < group) share[h] = fmaf(mix[h][g], p, share[h]);
+      for (uint32_t i = 0; i < 8u; ++i)
+        raw[i] = scores[size_t{min(g0 + 2u * i, heads - 1u)} * args.capacity];
+#pragma unroll
+      for (uint32_t i = 0; i < 8u; ++i) {
+        const uint32_t g = min(g0 + 2u * i, heads - 1u);
+        const float p = g0 + 2u * i < heads
+                            ? expf(raw[i] - row_maximum[g]) * row_inverse[g]
+                            : 0.0f;
+#pragma unroll
+        for (int h = 0; h < GROUP; ++h) share[h] = fmaf(mix[g][h], p, share[h]);
+      }
     }
 #pragma unroll
-    for (int h = 0; h < 16; ++h)
-      if (static_cast<uint32_t>(h) < group) {
-        const float both = share[h] + __shfl_xor(share[h], 32, kWave);
-        if (lane < 32u)
-          mixed[wave][h * kMixRow + lane] = static_cast<uint16_t>(f32_to_bf16_bits(both));
-      }
+    for (int h = 0; h < GROUP; ++h) {
+      const float both = share[h] + __shfl_xor(share[h], 32, kWave);
+      if (lane < 32u)
+        mixed[wave][h * kMixRow + lane] = static_cast<uint16_t>(f32_to_bf16_bits(both));
+    }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
     const i32x4 w = *reinterpret_cast<const i32x4*>(
@@ -473,10 +488,16 @@ __global__ void split_combine_kernel(AttentionArgs args) {
   const float gate =
       run.gate ? sigmoid_f32(run.gate[size_t{row} * run.gate_stride + head]) : 1.0f;
   for (uint32_t d = threadIdx.x; d < a.vdim; d += blockDim.x) {
+    float part[kMaximumValueSplits];
+#pragma unroll
+    for (uint32_t s = 0; s < kMaximumValueSplits; ++s)
+      part[s] = s < args.value_splits
+                    ? args.partials[((size_t{row} * args.value_splits + s) * a.query_heads +
+                                     head) * a.vdim + d]
+                    : 0.0f;
     float total = 0.0f;
-    for (uint32_t s = 0; s < args.value_splits; ++s)
-      total += args.partials[((size_t{row} * args.value_splits + s) * a.query_heads + head) *
-                                 a.vdim + d];
+#pragma unroll
+    for (uint32_t s = 0; s < kMaximumValueSplits; ++s) total += part[s];
     store_element(static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride +
                       head * a.vdim + d,
                   total * gate);
@@ -491,14 +512,38 @@ __device__ __forceinline__ uint32_t swizzled(uint32_t row, uint32_t slot) {
   return row * 64u + ((slot ^ (row >> 2 & 3u)) * 16u);
 }
 
+// The bf16 halves of two non-negative weights: the upper 16 bits of each as
+// they stand, and the rest, rounded.
+__device__ __forceinline__ void split_pair(float a, float b, uint32_t& high,
+                                           uint32_t& low) {
+  const uint32_t a_bits = __float_as_uint(a);
+  const uint32_t b_bits = __float_as_uint(b);
+  high = __builtin_amdgcn_perm(b_bits, a_bits, 0x07060302u);
+  low = pack_bf16(a - __uint_as_float(a_bits & 0xffff0000u),
+                  b - __uint_as_float(b_bits & 0xffff0000u));
+}
+
 // HPW heads per wave, NK = key_stride / 32, NV = value_stride / 16.
+//
+// The wave's keys are fetched one tile ahead: their registers are free as soon
+// as the tile's scores are out, and the fetch then has the rest of the
+// iteration to arrive.  With up to 16 heads (HPW <= 2) the high and the low
+// halves of the weights share one matrix operand - the mix matrix stands in it
+// twice - and with up to 32 they take one each.
 template <int HPW, int NK, int NV>
 __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs args) {
-  // normalised weights [key][query row][head], high and low halves
+  constexpr bool kFolded = HPW <= 2;
+  constexpr int kHeadTiles = kFolded ? 1 : 2;
+  constexpr int kMixHeads = kFolded ? 16 : 32;
+  constexpr int kPairs = (HPW + 1) / 2;
+  constexpr bool kEarlyValues = HPW <= 2;
+  // normalised weights [key][query row][64 bytes of heads]
   __shared__ __attribute__((aligned(16))) uint8_t high[512 * 64];
-  __shared__ __attribute__((aligned(16))) uint8_t low[512 * 64];
+  __shared__ __attribute__((aligned(16))) uint8_t low_plane[kFolded ? 16 : 512 * 64];
   // mixed weights [head][query row][key]
-  __shared__ __attribute__((aligned(16))) uint8_t mixed[kPromptHeads * 16 * 64];
+  __shared__ __attribute__((aligned(16))) uint8_t mixed[kMixHeads * 16 * 64];
+  uint8_t* const low = kFolded ? high : low_plane;
+  constexpr uint32_t kLowSlot = kFolded ? 2u : 0u;
   const Attention& a = args.attention;
   const auto& run = args.launch;
   const uint32_t heads = a.query_heads;
@@ -508,7 +553,13 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
   const uint32_t lane = threadIdx.x % kWave;
   const uint32_t column = lane % 16u;
   const uint32_t quarter = lane / 16u;
-  const uint32_t row0 = blockIdx.x * 16u;
+  // contiguous ranges of row blocks per XCD: neighbours share their keys
+  uint32_t block = blockIdx.x;
+  {
+    const uint32_t per_xcd = gridDim.x / 8u;
+    if (block < per_xcd * 8u) block = block % 8u * per_xcd + block / 8u;
+  }
+  const uint32_t row0 = block * 16u;
   const uint32_t first = a.step[kStepPosition] + row0;
   const uint32_t position = first + column;            // of this lane's query row
   const uint32_t last = first + min(16u, run.rows - row0) - 1u;
@@ -516,7 +567,7 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
 
   for (uint32_t i = threadIdx.x; i < sizeof(high) / 16u; i += blockDim.x) {
     reinterpret_cast<i32x4*>(high)[i] = i32x4{};
-    reinterpret_cast<i32x4*>(low)[i] = i32x4{};
+    if (!kFolded) reinterpret_cast<i32x4*>(low_plane)[i] = i32x4{};
   }
 
   uint32_t kv[HPW];
@@ -532,32 +583,30 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
     for (int c = 0; c < NK; ++c) q[i][c] = *reinterpret_cast<const i32x4*>(query + c * 32);
   }
   // rows head, columns other head of the mix matrix
-  i32x4 mix[2];
+  i32x4 mix[kHeadTiles];
 #pragma unroll
-  for (int t = 0; t < 2; ++t) {
+  for (int t = 0; t < kHeadTiles; ++t) {
     uint32_t packed[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      uint32_t bits[2];
+      float pair[2];
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const uint32_t h = t * 16u + column;
-        const uint32_t g = 8u * quarter + 2u * i + j;
-        const float value = h < heads && g < heads
-                                ? (a.head_mix ? a.head_mix[size_t{h} * heads + g]
-                                              : (h == g ? 1.0f : 0.0f))
-                                : 0.0f;
-        bits[j] = f32_to_bf16_bits(value);
+        const uint32_t g = (8u * quarter + 2u * i + j) % kMixHeads;
+        pair[j] = h < heads && g < heads ? (a.head_mix ? a.head_mix[size_t{h} * heads + g]
+                                                       : (h == g ? 1.0f : 0.0f))
+                                         : 0.0f;
       }
-      packed[i] = bits[0] | bits[1] << 16;
+      packed[i] = pack_bf16(pair[0], pair[1]);
     }
     mix[t] = i32x4{static_cast<int>(packed[0]), static_cast<int>(packed[1]),
                    static_cast<int>(packed[2]), static_cast<int>(packed[3])};
   }
 
-  i32x4 k[2][NK];
-  const auto load_keys = [&](uint32_t tile, uint32_t kv_head) {
-    const uint32_t key0 = tile * kTileKeys;
+  const auto fetch_keys = [&](i32x4 (&k)[2][NK], uint32_t ordinal, uint32_t kv_head)
+      __attribute__((always_inline)) {
+    const uint32_t key0 = range.tile(ordinal) * kTileKeys;
     const i32x4* keys = reinterpret_cast<const i32x4*>(
                             page_of<const uint16_t>(a, key0) +
                             key_block(a, kv_head, key0 % a.page_tokens)) +
@@ -567,159 +616,221 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
 #pragma unroll
       for (int c = 0; c < NK; ++c) k[half][c] = keys[(half * NK + c) * kWave];
   };
-  // scores of one head: s[half][i] = key 16 half + 4 quarter + i, query row column
-  const auto score = [&](const i32x4 (&query)[NK], f32x4 (&s)[2], uint32_t tile) {
-    const uint32_t key0 = tile * kTileKeys + 4u * quarter;
+  const auto products = [&](const i32x4 (&k)[2][NK], const i32x4 (&query)[NK],
+                            f32x4 (&s)[2]) __attribute__((always_inline)) {
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
       s[half] = f32x4{};
 #pragma unroll
       for (int c = 0; c < NK; ++c) s[half] = mfma_bf16(k[half][c], query[c], s[half]);
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        s[half][i] = visible(a, position, key0 + half * 16u + i) ? s[half][i] * a.scale
-                                                                 : -INFINITY;
     }
   };
+  // s[half][i] = key 16 half + 4 quarter + i of the tile, query row column
+  const auto hide = [&](f32x4 (&s)[2], uint32_t tile) __attribute__((always_inline)) {
+    const uint32_t key0 = tile * kTileKeys + 4u * quarter;
+#pragma unroll
+    for (int half = 0; half < 2; ++half)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (!visible(a, position, key0 + half * 16u + i)) s[half][i] = -INFINITY;
+  };
+  // every row of the block sees every key of the tile
+  const auto open = [&](uint32_t tile) {
+    const uint32_t first_key = tile * kTileKeys;
+    const uint32_t last_key = first_key + kTileKeys - 1u;
+    return last_key <= first &&
+           (!a.window || first + 15u - first_key < a.window || last_key < a.sinks);
+  };
 
+  // scores in units of the base-2 exponent; exp2(-inf) = 0 hides a key
+  const float unit = a.scale * 1.4426950408889634f;
   float maximum[HPW], total[HPW];
 #pragma unroll
   for (int i = 0; i < HPW; ++i) {
     maximum[i] = -INFINITY;
     total[i] = 0.0f;
   }
-  for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal) {
+  const auto survey = [&](i32x4 (&k)[2][NK], uint32_t ordinal, uint32_t ahead)
+      __attribute__((always_inline)) {
     const uint32_t tile = range.tile(ordinal);
+    const bool all = open(tile);
+    f32x4 s[HPW][2];
 #pragma unroll
     for (int i = 0; i < HPW; ++i) {
-      if (i == 0 || kv[i] != kv[i - 1]) load_keys(tile, kv[i]);
-      f32x4 s[2];
-      score(q[i], s, tile);
-      float top = -INFINITY;
+      if (i > 0 && kv[i] != kv[i - 1]) fetch_keys(k, ordinal, kv[i]);
+      products(k, q[i], s[i]);
+    }
+    fetch_keys(k, min(ahead, range.count - 1u), kv[0]);
+#pragma unroll
+    for (int i = 0; i < HPW; ++i) {
+#pragma unroll
+      for (int half = 0; half < 2; ++half) s[i][half] *= unit;
+      if (!all) hide(s[i], tile);
+      float top = maximum[i];
 #pragma unroll
       for (int half = 0; half < 2; ++half)
 #pragma unroll
-        for (int j = 0; j < 4; ++j) top = fmaxf(top, s[half][j]);
-      if (top > -INFINITY) {
-        const float fresh = fmaxf(maximum[i], top);
-        float sum = total[i] * __expf(maximum[i] - fresh);
+        for (int j = 0; j < 4; ++j) top = fmaxf(top, s[i][half][j]);
+      // a row that has seen nothing yet: keep the exponents' argument finite
+      const float base = top == -INFINITY ? 0.0f : top;
+      float sum = total[i] * __builtin_amdgcn_exp2f(maximum[i] - base);
 #pragma unroll
-        for (int half = 0; half < 2; ++half)
+      for (int half = 0; half < 2; ++half)
 #pragma unroll
-          for (int j = 0; j < 4; ++j) sum += __expf(s[half][j] - fresh);
-        total[i] = sum;
-        maximum[i] = fresh;
+        for (int j = 0; j < 4; ++j) sum += __builtin_amdgcn_exp2f(s[i][half][j] - base);
+      total[i] = sum;
+      maximum[i] = top;
+    }
+  };
+  {
+    i32x4 even[2][NK], odd[2][NK];
+    fetch_keys(even, 0u, kv[0]);
+    if constexpr (HPW <= 2) {
+      fetch_keys(odd, min(1u, range.count - 1u), kv[0]);
+      uint32_t ordinal = 0;
+      for (; ordinal + 2u <= range.count; ordinal += 2u) {
+        survey(even, ordinal, ordinal + 2u);
+        survey(odd, ordinal + 1u, ordinal + 3u);
       }
+      if (ordinal < range.count) survey(even, ordinal, ordinal);
+    } else {
+      for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal)
+        survey(even, ordinal, ordinal + 1u);
     }
   }
+  // from here on maximum holds maximum + log2(total): exp2(score - it) is the
+  // normalised weight
 #pragma unroll
   for (int i = 0; i < HPW; ++i) {
 #pragma unroll
     for (int offset = 16; offset <= 32; offset *= 2) {
       const float other = __shfl_xor(maximum[i], offset, kWave);
       const float other_total = __shfl_xor(total[i], offset, kWave);
-      const float fresh = fmaxf(maximum[i], other);
-      if (fresh > -INFINITY) {
-        total[i] = total[i] * __expf(maximum[i] - fresh) + other_total * __expf(other - fresh);
-        maximum[i] = fresh;
-      }
+      const float top = fmaxf(maximum[i], other);
+      const float base = top == -INFINITY ? 0.0f : top;
+      total[i] = total[i] * __builtin_amdgcn_exp2f(maximum[i] - base) +
+                 other_total * __builtin_amdgcn_exp2f(other - base);
+      maximum[i] = top;
     }
-    total[i] = 1.0f / total[i];
+    maximum[i] += log2f(total[i]);
   }
   __syncthreads();   // the weight buffers are clear
 
   f32x4 out[HPW][NV] = {};
+  i32x4 k[2][NK];
+  fetch_keys(k, 0u, kv[0]);
+  const auto fetch_values = [&](uint32_t ordinal, uint32_t kv_head)
+      __attribute__((always_inline)) {
+    const uint32_t key0 = range.tile(ordinal) * kTileKeys;
+    return reinterpret_cast<const i32x4*>(page_of<const uint16_t>(a, key0) +
+                                          value_block(a, kv_head, key0 % a.page_tokens)) +
+           column * 4u + quarter;
+  };
   for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal) {
     const uint32_t tile = range.tile(ordinal);
-    uint32_t high_bits[8][(HPW + 1) / 2];
-    uint32_t low_bits[8][(HPW + 1) / 2];
+    const bool all = open(tile);
+    i32x4 v[kEarlyValues ? NV : 1];
+    if constexpr (kEarlyValues) {
+      const i32x4* values = fetch_values(ordinal, kv[0]);
 #pragma unroll
-    for (int i = 0; i < HPW; ++i) {
-      if (i == 0 || kv[i] != kv[i - 1]) load_keys(tile, kv[i]);
-      f32x4 s[2];
-      score(q[i], s, tile);
+      for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
+    }
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const float p = __expf(s[e / 4][e % 4] - maximum[i]) * total[i];
-        const uint32_t upper = f32_to_bf16_bits(p);
-        const uint32_t lower = f32_to_bf16_bits(p - bf16_bits_to_f32(upper));
-        if (i % 2 == 0) {
-          high_bits[e][i / 2] = upper;
-          low_bits[e][i / 2] = lower;
-        } else {
-          high_bits[e][i / 2] |= upper << 16;
-          low_bits[e][i / 2] |= lower << 16;
+    for (int pair = 0; pair < kPairs; ++pair) {
+      f32x4 s[2][2];
+#pragma unroll
+      for (int j = 0; j < 2 && 2 * pair + j < HPW; ++j) {
+        const int i = 2 * pair + j;
+        if (i > 0 && kv[i] != kv[i - 1]) fetch_keys(k, ordinal, kv[i]);
+        products(k, q[i], s[j]);
+      }
+      if (pair + 1 == kPairs) fetch_keys(k, min(ordinal + 1u, range.count - 1u), kv[0]);
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        if (2 * pair + j >= HPW) {
+          s[j][0] = s[j][1] = f32x4{};
+          continue;
+        }
+        if (!all) hide(s[j], tile);
+        const float offset = maximum[2 * pair + j];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          // a hidden key stays at minus infinity whatever the unit's sign
+          const float raw = s[j][e / 4][e % 4];
+          const float exponent = !all && raw == -INFINITY ? raw : fmaf(raw, unit, -offset);
+          s[j][e / 4][e % 4] = __builtin_amdgcn_exp2f(exponent);
         }
       }
-    }
-    if (wave * HPW < heads) {
-      const uint32_t g = wave * HPW;
+      const uint32_t g = wave * HPW + 2u * pair;
+      if (g < heads) {
+        const bool second = HPW > 1 && g + 1u < heads;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const uint32_t key = e / 4 * 16u + 4u * quarter + e % 4;
-        const uint32_t at = swizzled(key * 16u + column, g / 8u) + g % 8u * 2u;
-        if constexpr (HPW == 4) {
-          *reinterpret_cast<i32x2*>(high + at) = i32x2{static_cast<int>(high_bits[e][0]),
-                                                       static_cast<int>(high_bits[e][1])};
-          *reinterpret_cast<i32x2*>(low + at) =
-              i32x2{static_cast<int>(low_bits[e][0]), static_cast<int>(low_bits[e][1])};
-        } else if constexpr (HPW == 2) {
-          *reinterpret_cast<uint32_t*>(high + at) = high_bits[e][0];
-          *reinterpret_cast<uint32_t*>(low + at) = low_bits[e][0];
-        } else {
-          *reinterpret_cast<uint16_t*>(high + at) = static_cast<uint16_t>(high_bits[e][0]);
-          *reinterpret_cast<uint16_t*>(low + at) = static_cast<uint16_t>(low_bits[e][0]);
+        for (int e = 0; e < 8; ++e) {
+          const uint32_t row = (e / 4 * 16u + 4u * quarter + e % 4) * 16u + column;
+          uint32_t upper, lower;
+          split_pair(s[0][e / 4][e % 4], second ? s[1][e / 4][e % 4] : 0.0f, upper, lower);
+          uint8_t* const upper_at = high + swizzled(row, g / 8u) + g % 8u * 2u;
+          uint8_t* const lower_at = low + swizzled(row, kLowSlot + g / 8u) + g % 8u * 2u;
+          if constexpr (HPW == 1) {
+            *reinterpret_cast<uint16_t*>(upper_at) = static_cast<uint16_t>(upper);
+            *reinterpret_cast<uint16_t*>(lower_at) = static_cast<uint16_t>(lower);
+          } else {
+            *reinterpret_cast<uint32_t*>(upper_at) = upper;
+            *reinterpret_cast<uint32_t*>(lower_at) = lower;
+          }
         }
       }
     }
     __syncthreads();
     // mix: four keys at a time, all query rows and heads
     for (uint32_t four = wave; four < 8u; four += waves) {
-      f32x4 m[4][2] = {};
+      f32x4 m[4][kHeadTiles] = {};
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const uint32_t at = swizzled((four * 4u + j) * 16u + column, quarter);
         const i32x4 upper = *reinterpret_cast<const i32x4*>(high + at);
-        const i32x4 lower = *reinterpret_cast<const i32x4*>(low + at);
+        if constexpr (kFolded) {
+          m[j][0] = mfma_bf16(mix[0], upper, m[j][0]);
+        } else {
+          const i32x4 lower = *reinterpret_cast<const i32x4*>(low + at);
 #pragma unroll
-        for (int t = 0; t < 2; ++t) {
-          if (t * 16u >= heads) continue;
-          m[j][t] = mfma_bf16(mix[t], lower, m[j][t]);
-          m[j][t] = mfma_bf16(mix[t], upper, m[j][t]);
+          for (int t = 0; t < kHeadTiles; ++t) {
+            m[j][t] = mfma_bf16(mix[t], lower, m[j][t]);
+            m[j][t] = mfma_bf16(mix[t], upper, m[j][t]);
+          }
         }
       }
 #pragma unroll
-      for (int t = 0; t < 2; ++t)
+      for (int t = 0; t < kHeadTiles; ++t)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const uint32_t h = t * 16u + 4u * quarter + i;
-          if (h >= heads) continue;
-          const uint32_t pair0 = f32_to_bf16_bits(m[0][t][i]) | f32_to_bf16_bits(m[1][t][i]) << 16;
-          const uint32_t pair1 = f32_to_bf16_bits(m[2][t][i]) | f32_to_bf16_bits(m[3][t][i]) << 16;
           *reinterpret_cast<i32x2*>(mixed + h * 1024u + swizzled(column, four / 2u) +
                                     four % 2u * 8u) =
-              i32x2{static_cast<int>(pair0), static_cast<int>(pair1)};
+              i32x2{static_cast<int>(pack_bf16(m[0][t][i], m[1][t][i])),
+                    static_cast<int>(pack_bf16(m[2][t][i], m[3][t][i]))};
         }
     }
     __syncthreads();
-    const uint32_t key0 = tile * kTileKeys;
-    const uint16_t* page = page_of<const uint16_t>(a, key0);
-    i32x4 v[NV];
 #pragma unroll
     for (int i = 0; i < HPW; ++i) {
       const uint32_t head = wave * HPW + i;
       if (head >= heads) continue;
-      if (i == 0 || kv[i] != kv[i - 1]) {
-        const i32x4* values = reinterpret_cast<const i32x4*>(
-                                  page + value_block(a, kv[i], key0 % a.page_tokens)) +
-                              column * 4u + quarter;
-#pragma unroll
-        for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
-      }
       const i32x4 w = *reinterpret_cast<const i32x4*>(mixed + head * 1024u +
                                                       swizzled(column, quarter));
+      if constexpr (kEarlyValues) {
+        if (i > 0 && kv[i] != kv[i - 1]) {
+          const i32x4* values = fetch_values(ordinal, kv[i]);
 #pragma unroll
-      for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, v[t], out[i][t]);
+          for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
+        }
+#pragma unroll
+        for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, v[t], out[i][t]);
+      } else {
+        const i32x4* values = fetch_values(ordinal, kv[i]);
+#pragma unroll
+        for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, values[t * kWave], out[i][t]);
+      }
     }
   }
 
@@ -911,12 +1022,20 @@ extern "C" int32_t qllm_windowed_attention_rows(const qllm_windowed_attention* a
   else
     split_scores_kernel<8><<<score_grid, 256, 0, hip_stream>>>(args);
   const dim3 value_grid(args.value_splits, a.kv_heads, launch->rows);
+  const bool narrow = a.query_heads / a.kv_heads <= 4u;
+  const auto values = [&](auto nv) {
+    constexpr int NV = decltype(nv)::value;
+    if (narrow)
+      split_values_kernel<NV, 4><<<value_grid, 256, 0, hip_stream>>>(args);
+    else
+      split_values_kernel<NV, 16><<<value_grid, 256, 0, hip_stream>>>(args);
+  };
   if (a.value_stride == 64u)
-    split_values_kernel<4><<<value_grid, 256, 0, hip_stream>>>(args);
+    values(std::integral_constant<int, 4>{});
   else if (a.value_stride == 128u)
-    split_values_kernel<8><<<value_grid, 256, 0, hip_stream>>>(args);
+    values(std::integral_constant<int, 8>{});
   else
-    split_values_kernel<16><<<value_grid, 256, 0, hip_stream>>>(args);
+    values(std::integral_constant<int, 16>{});
   split_combine_kernel<<<dim3(a.query_heads, launch->rows), 64, 0, hip_stream>>>(args);
   return launched("windowed split attention");
 }

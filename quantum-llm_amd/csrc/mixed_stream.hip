@@ -19,9 +19,19 @@ struct NormArgs {
 __device__ __forceinline__ f32x4 stream_value4(const qllm_stream_norm_launch& l,
                                                uint32_t row, uint32_t piece) {
   f32x4 value = reinterpret_cast<const f32x4*>(l.input + size_t{row} * l.width)[piece];
-  for (uint32_t p = 0; p < l.partial_count; ++p)
-    value += reinterpret_cast<const f32x4*>(
-        l.partials + (size_t{p} * l.rows + row) * l.partial_stride)[piece];
+  // eight loads in flight at a time
+  for (uint32_t first = 0; first < l.partial_count; first += 8u) {
+    f32x4 part[8];
+#pragma unroll
+    for (uint32_t i = 0; i < 8u; ++i)
+      part[i] = first + i < l.partial_count
+                    ? reinterpret_cast<const f32x4*>(
+                          l.partials +
+                          (size_t{first + i} * l.rows + row) * l.partial_stride)[piece]
+                    : f32x4{};
+#pragma unroll
+    for (uint32_t i = 0; i < 8u; ++i) value += part[i];
+  }
   return value;
 }
 

@@ -71,6 +71,35 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(RecurrenceArgs ar
   const bool delta = l.kind == QLLM_RECURRENCE_DELTA;
   const float* p = run.projections;
 
+  // everything that depends on nothing is on its way before the first barrier
+  const uint32_t groups = 1024u / dim;
+  const uint32_t group = threadIdx.x / dim;
+  const uint32_t column = threadIdx.x - group * dim;
+  const bool active = group < groups;
+  const uint32_t per_group = (dim + groups - 1u) / groups;
+  const uint32_t row0 = group * per_group;
+  const uint32_t rows = active && row0 < dim ? min(per_group, dim - row0) : 0u;
+  float* state = l.state + l.step[kStepSlot] * l.slot_stride +
+                 (size_t{head} * dim + row0) * dim + column;
+  float s[KPT];
+#pragma unroll
+  for (int i = 0; i < KPT; ++i)
+    s[i] = static_cast<uint32_t>(i) < rows ? state[size_t{static_cast<uint32_t>(i)} * dim] : 0.0f;
+  const float value = active ? p[run.v_column + first + column] : 0.0f;
+
+  const bool owner = threadIdx.x < dim;
+  float base = 0.0f;
+  float rate = 0.0f;
+  float gate = 0.0f;
+  float weight = 0.0f;
+  if (owner) {
+    const uint32_t c = first + threadIdx.x;
+    base = l.decay_base[c];
+    gate = p[run.gate_column + c];
+    weight = l.norm_weight[c];
+    if (delta) rate = p[run.rate_column + c] + l.rate_bias[c];
+  }
+
   for (uint32_t j = threadIdx.x; j < l.rank; j += blockDim.x)
     low[j] = tanhf(p[run.low_column + j]);
   float key = 0.0f;
@@ -91,36 +120,22 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(RecurrenceArgs ar
     if (channel < dim) {
       const uint16_t* up = static_cast<const uint16_t*>(l.decay_up_bf16) +
                            size_t{first + channel} * l.rank;
+#pragma unroll 8
       for (uint32_t j = threadIdx.x % 4u; j < l.rank; j += 4u)
         inner = fmaf(bf16_bits_to_f32(up[j]), low[j], inner);
     }
     inner += __shfl_xor(inner, 1, kWave);
     inner += __shfl_xor(inner, 2, kWave);
-    if (channel < dim && threadIdx.x % 4u == 0u)
-      w[channel] = decay_of(l, inner + l.decay_base[first + channel]);
+    if (channel < dim && threadIdx.x % 4u == 0u) w[channel] = inner;
   }
-  if (delta && threadIdx.x < dim) {
-    const uint32_t c = first + threadIdx.x;
+  if (delta && owner) {
     const float unit = key / sqrtf(total + l.unit_epsilon);
     u[threadIdx.x] = unit;
-    au[threadIdx.x] = unit * sigmoid_f32(p[run.rate_column + c] + l.rate_bias[c]);
+    au[threadIdx.x] = unit * sigmoid_f32(rate);
   }
   __syncthreads();
-
-  const uint32_t groups = 1024u / dim;
-  const uint32_t group = threadIdx.x / dim;
-  const uint32_t column = threadIdx.x - group * dim;
-  const bool active = group < groups;
-  const uint32_t per_group = (dim + groups - 1u) / groups;
-  const uint32_t row0 = group * per_group;
-  const uint32_t rows = active && row0 < dim ? min(per_group, dim - row0) : 0u;
-  float* state = l.state + l.step[kStepSlot] * l.slot_stride +
-                 (size_t{head} * dim + row0) * dim + column;
-  float s[KPT];
-#pragma unroll
-  for (int i = 0; i < KPT; ++i)
-    s[i] = static_cast<uint32_t>(i) < rows ? state[size_t{static_cast<uint32_t>(i)} * dim] : 0.0f;
-  const float value = active ? p[run.v_column + first + column] : 0.0f;
+  if (owner) w[threadIdx.x] = decay_of(l, w[threadIdx.x] + base);
+  __syncthreads();
 
   const auto column_sum = [&](float mine) {
     part[threadIdx.x] = mine;
@@ -160,96 +175,124 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(RecurrenceArgs ar
   for (int i = 0; i < KPT; ++i)
     if (static_cast<uint32_t>(i) < rows) state[size_t{static_cast<uint32_t>(i)} * dim] = s[i];
 
-  const bool owner = threadIdx.x < dim;
   const float squares = block_sum(owner ? out * out : 0.0f, scratch);
   if (owner) {
-    const uint32_t c = first + threadIdx.x;
     const float unit = out / sqrtf(squares / static_cast<float>(dim) + l.epsilon);
-    store_element(static_cast<T*>(run.output) + c,
-                  unit * l.norm_weight[c] * gate_value(l.gate_kind, p[run.gate_column + c]));
+    store_element(static_cast<T*>(run.output) + first + threadIdx.x,
+                  unit * weight * gate_value(l.gate_kind, gate));
   }
   copy_carry(args);
 }
 
 // ---- prompts ---------------------------------------------------------------------
 
-constexpr uint32_t kPrepareRows = 8;
+constexpr uint32_t kRowsPerThread = 8;    // tokens a thread prepares
+constexpr uint32_t kRankChunk = 32;
 
-// Token vectors of kPrepareRows tokens of one head.
+// Token vectors of one head.  Threads lie side by side on channels, in groups
+// of kRowsPerThread tokens each; the low-rank product runs over LDS tiles of
+// kRankChunk columns.
 __global__ __launch_bounds__(256) void recurrence_prepare_kernel(RecurrenceArgs args) {
-  __shared__ float low[kPrepareRows][256];
-  __shared__ float products[kPrepareRows][256];
-  __shared__ float sums[kPrepareRows];
+  constexpr uint32_t kMostRows = 256u / 16u * kRowsPerThread;
+  __shared__ float up_tile[kRankChunk][257];
+  __shared__ __attribute__((aligned(16))) float low_tile[kMostRows][kRankChunk];
+  __shared__ float sums[kMostRows][4];
   const qllm_recurrence& l = args.layer;
   const auto& run = args.launch;
   const uint32_t head = blockIdx.y;
   const uint32_t dim = l.dim;
   const uint32_t first = head * dim;
-  const uint32_t row0 = blockIdx.x * kPrepareRows;
-  const uint32_t rows = min(kPrepareRows, run.rows - row0);
-  const bool delta = l.kind == QLLM_RECURRENCE_DELTA;
-
-  for (uint32_t i = threadIdx.x; i < rows * l.rank; i += blockDim.x) {
-    const uint32_t row = i / l.rank;
-    const uint32_t j = i % l.rank;
-    low[row][j] = tanhf(run.projections[size_t{row0 + row} * run.stride + run.low_column + j]);
-  }
-  for (uint32_t i = threadIdx.x; i < rows * dim; i += blockDim.x) {
-    const uint32_t row = i / dim;
-    const uint32_t c = i % dim;
-    const float* p = run.projections + size_t{row0 + row} * run.stride;
-    const float key = p[run.k_column + first + c];
-    products[row][c] =
-        delta ? key * key : p[run.r_column + first + c] * l.bonus[first + c] * key;
-  }
-  __syncthreads();
-  for (uint32_t row = threadIdx.x / kWave; row < rows; row += blockDim.x / kWave) {
-    float sum = 0.0f;
-    for (uint32_t c = threadIdx.x % kWave; c < dim; c += kWave) sum += products[row][c];
-    sum = wave_sum(sum);
-    if (threadIdx.x % kWave == 0u) {
-      sums[row] = sum;
-      if (!delta) args.scalars[size_t{head} * run.rows + row0 + row] = sum;
-    }
-  }
-  __syncthreads();
-
   const uint32_t padded = args.padded;
-  const uint32_t vectors = vectors_of(l.kind);
-  const uint32_t lanes = min(blockDim.x, padded);   // threads side by side on channels
-  const uint32_t groups = blockDim.x / lanes;
-  const uint32_t c = threadIdx.x % lanes;
-  const uint32_t group = threadIdx.x / lanes;
-  float inner[kPrepareRows] = {};
-  if (c < dim) {
-    const uint16_t* up =
-        static_cast<const uint16_t*>(l.decay_up_bf16) + size_t{first + c} * l.rank;
-    for (uint32_t j = 0; j < l.rank; ++j) {
-      const float weight = bf16_bits_to_f32(up[j]);
+  const uint32_t groups = 256u / padded;
+  const uint32_t block_rows = groups * kRowsPerThread;
+  const uint32_t row0 = blockIdx.x * block_rows;
+  const uint32_t rows = min(block_rows, run.rows - row0);
+  const bool delta = l.kind == QLLM_RECURRENCE_DELTA;
+  const float* block_projections = run.projections + size_t{row0} * run.stride;
+  const uint32_t c = threadIdx.x % padded;
+  const uint32_t group = threadIdx.x / padded;
+  const bool real = c < dim;
+  const uint32_t channel = first + min(c, dim - 1u);
+
+  // this thread's tokens: all loads in flight together
+  float key[kRowsPerThread], read[kRowsPerThread], rate[kRowsPerThread];
 #pragma unroll
-      for (uint32_t i = 0; i < kPrepareRows; ++i)
-        if (i * groups + group < rows)
-          inner[i] = fmaf(weight, low[i * groups + group][j], inner[i]);
+  for (uint32_t i = 0; i < kRowsPerThread; ++i) {
+    const float* p = block_projections +
+                     size_t{min(group * kRowsPerThread + i, rows - 1u)} * run.stride + channel;
+    key[i] = p[run.k_column];
+    read[i] = p[run.r_column];
+    rate[i] = delta ? p[run.rate_column] : 0.0f;
+  }
+  // per token: sum of k^2, or of r * bonus * k
+  const float bonus = delta || !real ? 0.0f : l.bonus[channel];
+#pragma unroll
+  for (uint32_t i = 0; i < kRowsPerThread; ++i) {
+    key[i] = real ? key[i] : 0.0f;
+    read[i] = real ? read[i] : 0.0f;
+    float sum = delta ? key[i] * key[i] : read[i] * bonus * key[i];
+    sum = row16_sum(sum);
+    for (uint32_t offset = 16u; offset < min(padded, 64u); offset *= 2u)
+      sum += __shfl_xor(sum, static_cast<int>(offset), kWave);
+    if (c % 64u == 0u) sums[group * kRowsPerThread + i][c / 64u] = sum;
+  }
+
+  float inner[kRowsPerThread] = {};
+  for (uint32_t j0 = 0; j0 < l.rank; j0 += kRankChunk) {
+    __syncthreads();
+#pragma unroll 8
+    for (uint32_t i = threadIdx.x; i < padded * kRankChunk; i += 256u) {
+      const uint32_t at = i / kRankChunk;
+      const uint32_t j = i % kRankChunk;
+      const float weight = bf16_bits_to_f32(static_cast<const uint16_t*>(
+          l.decay_up_bf16)[size_t{first + min(at, dim - 1u)} * l.rank +
+                           min(j0 + j, l.rank - 1u)]);
+      up_tile[j][at] = j0 + j < l.rank ? weight : 0.0f;
+    }
+#pragma unroll 4
+    for (uint32_t i = threadIdx.x; i < block_rows * kRankChunk; i += 256u) {
+      const uint32_t row = i / kRankChunk;
+      const uint32_t j = i % kRankChunk;
+      const float value =
+          tanhf(block_projections[size_t{min(row, rows - 1u)} * run.stride +
+                                  run.low_column + min(j0 + j, l.rank - 1u)]);
+      low_tile[row][j] = j0 + j < l.rank ? value : 0.0f;
+    }
+    __syncthreads();
+#pragma unroll 2
+    for (uint32_t j = 0; j < kRankChunk; j += 4u) {
+      float weight[4];
+#pragma unroll
+      for (uint32_t e = 0; e < 4u; ++e) weight[e] = up_tile[j + e][c];
+#pragma unroll
+      for (uint32_t i = 0; i < kRowsPerThread; ++i) {
+        const f32x4 low =
+            *reinterpret_cast<const f32x4*>(&low_tile[group * kRowsPerThread + i][j]);
+#pragma unroll
+        for (uint32_t e = 0; e < 4u; ++e) inner[i] = fmaf(weight[e], low[e], inner[i]);
+      }
     }
   }
+
+  const uint32_t vectors = vectors_of(l.kind);
+  const float base = real ? l.decay_base[channel] : 0.0f;
+  const float bias = real && delta ? l.rate_bias[channel] : 0.0f;
 #pragma unroll
-  for (uint32_t i = 0; i < kPrepareRows; ++i) {
-    const uint32_t row = i * groups + group;
+  for (uint32_t i = 0; i < kRowsPerThread; ++i) {
+    const uint32_t row = group * kRowsPerThread + i;
     if (row >= rows) break;
+    float sum = sums[row][0];
+    for (uint32_t wave = 1; wave < padded / 64u; ++wave) sum += sums[row][wave];
+    if (!delta && c == 0u) args.scalars[size_t{head} * run.rows + row0 + row] = sum;
     float* out = args.prepared +
                  (size_t{head} * run.rows + row0 + row) * vectors * padded + c;
-    const float* p = run.projections + size_t{row0 + row} * run.stride + first + c;
-    const bool real = c < dim;
-    const float key = real ? p[run.k_column] : 0.0f;
-    out[0] = real ? p[run.r_column] : 0.0f;
-    out[padded] = key;
-    out[2u * padded] =
-        real ? decay_of(l, inner[i] + l.decay_base[first + c]) : 0.0f;
+    out[0] = read[i];
+    out[padded] = key[i];
+    out[2u * padded] = real ? decay_of(l, inner[i] + base) : 0.0f;
     if (delta) {
-      const float unit = key / sqrtf(sums[row] + l.unit_epsilon);
+      const float unit = key[i] / sqrtf(sum + l.unit_epsilon);
       out[3u * padded] = unit;
-      out[4u * padded] =
-          real ? unit * sigmoid_f32(p[run.rate_column] + l.rate_bias[first + c]) : 0.0f;
+      out[4u * padded] = real ? unit * sigmoid_f32(rate[i] + bias) : 0.0f;
     }
   }
 }
@@ -261,7 +304,7 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
   constexpr uint32_t kVectors = DELTA ? 5u : 3u;
   constexpr uint32_t kTokens = 1024u / kPadded;
   constexpr uint32_t kChunk = 1024u * kVectors;        // floats
-  __shared__ float4 chunk[2][kChunk / 4u];
+  __shared__ f32x4 chunk[2][kChunk / 4u];
   __shared__ float values[2][kTokens][16];
   __shared__ float bonus[2][kTokens];
   const qllm_recurrence& l = args.layer;
@@ -280,19 +323,21 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
     s[i] = real && row < dim ? state[size_t{row} * dim + column] : 0.0f;
   }
 
-  const float4* source = reinterpret_cast<const float4*>(
+  const f32x4* source = reinterpret_cast<const f32x4*>(
       args.prepared + size_t{head} * run.rows * kVectors * kPadded);
   const uint32_t all_pieces = run.rows * kVectors * kPadded / 4u;
   const uint32_t chunks = (run.rows + kTokens - 1u) / kTokens;
-  float4 next[kVectors];
-  float next_values[(kTokens * 16u + 255u) / 256u];
+  constexpr uint32_t kValueLoads = (kTokens * 16u + 255u) / 256u;
+  f32x4 next[kVectors];
+  float next_values[kValueLoads];
   float next_bonus = 0.0f;
-  const auto fetch = [&](uint32_t which) {
+  // Loads of a chunk, and their way into LDS.
+  const auto fetch = [&](uint32_t which) __attribute__((always_inline)) {
 #pragma unroll
     for (uint32_t i = 0; i < kVectors; ++i)
       next[i] = source[min(which * (kChunk / 4u) + i * 256u + threadIdx.x, all_pieces - 1u)];
 #pragma unroll
-    for (uint32_t i = 0; i < sizeof(next_values) / 4u; ++i) {
+    for (uint32_t i = 0; i < kValueLoads; ++i) {
       const uint32_t index = i * 256u + threadIdx.x;
       const uint32_t row = min(which * kTokens + index / 16u, run.rows - 1u);
       const uint32_t c = min(blockIdx.x * 16u + index % 16u, dim - 1u);
@@ -303,76 +348,105 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
       next_bonus = args.scalars[size_t{head} * run.rows +
                                 min(which * kTokens + threadIdx.x % kTokens, run.rows - 1u)];
   };
-  const auto publish = [&](uint32_t slot) {
+  const auto publish = [&](uint32_t slot, uint32_t which) __attribute__((always_inline)) {
 #pragma unroll
-    for (uint32_t i = 0; i < kVectors; ++i) chunk[slot][i * 256u + threadIdx.x] = next[i];
+    for (uint32_t i = 0; i < kVectors; ++i) {
+      // tokens past the last one: decays of 1 and zeros, which change nothing
+      const uint32_t in_chunk = i * 256u + threadIdx.x;
+      const float idle = in_chunk / (kPadded / 4u) % kVectors == 2u ? 1.0f : 0.0f;
+      const bool there = which * (kChunk / 4u) + in_chunk < all_pieces;
+      f32x4 piece;
 #pragma unroll
-    for (uint32_t i = 0; i < sizeof(next_values) / 4u; ++i) {
+      for (int e = 0; e < 4; ++e) piece[e] = there ? next[i][e] : idle;
+      chunk[slot][in_chunk] = piece;
+    }
+#pragma unroll
+    for (uint32_t i = 0; i < kValueLoads; ++i) {
       const uint32_t index = i * 256u + threadIdx.x;
       if (index < kTokens * 16u) values[slot][index / 16u][index % 16u] = next_values[i];
     }
     if (!DELTA && threadIdx.x < kTokens) bonus[slot][threadIdx.x] = next_bonus;
   };
 
+  // What a token brings to this lane, read from LDS one token ahead of its use.
+  struct Token {
+    float vector[kVectors][KPL];
+    float value;
+  };
+  const auto read = [&](Token& token, uint32_t slot, uint32_t t)
+      __attribute__((always_inline)) {
+    constexpr int kAlignment = KPL >= 4 ? 16 : KPL * 4;
+    const float* at = static_cast<const float*>(__builtin_assume_aligned(
+        reinterpret_cast<const float*>(chunk[slot]) + t * kVectors * kPadded + part * KPL,
+        kAlignment));
+#pragma unroll
+    for (uint32_t v = 0; v < kVectors; ++v)
+#pragma unroll
+      for (int i = 0; i < KPL; ++i) token.vector[v][i] = at[v * kPadded + i];
+    token.value = values[slot][t][threadIdx.x / 16u];
+  };
+  const auto dot_with = [&](const float (&vector)[KPL]) __attribute__((always_inline)) {
+    float even = vector[0] * s[0];
+    float odd = 0.0f;
+#pragma unroll
+    for (int i = 1; i < KPL; ++i)
+      if (i % 2 == 1)
+        odd = i == 1 ? vector[i] * s[i] : fmaf(vector[i], s[i], odd);
+      else
+        even = fmaf(vector[i], s[i], even);
+    return even + odd;
+  };
+  // Moves the state past a token; returns this lane's part of the output.
+  const auto advance = [&](const Token& token) __attribute__((always_inline)) {
+    const auto& r = token.vector[0];
+    const auto& k = token.vector[1];
+    const auto& w = token.vector[2];
+    if constexpr (DELTA) {
+      const auto& u = token.vector[3];
+      const auto& au = token.vector[4];
+      float dot = dot_with(u);
+      // while the dot product travels: the part that does not need it
+#pragma unroll
+      for (int i = 0; i < KPL; ++i) s[i] = fmaf(k[i], token.value, w[i] * s[i]);
+      dot = row16_sum(dot);
+#pragma unroll
+      for (int i = 0; i < KPL; ++i) s[i] = fmaf(-au[i], dot, s[i]);
+      return dot_with(r);
+    } else {
+      const float out = dot_with(r);
+#pragma unroll
+      for (int i = 0; i < KPL; ++i) s[i] = fmaf(k[i], token.value, w[i] * s[i]);
+      return out;
+    }
+  };
+
   fetch(0u);
-  publish(0u);
+  publish(0u, 0u);
   __syncthreads();
+  // a block of tokens' outputs is summed over the lanes at once: lane t of a
+  // column ends with token t's
+  constexpr uint32_t kBlock = kTokens < 16u ? kTokens : 16u;
   for (uint32_t which = 0; which < chunks; ++which) {
     const uint32_t slot = which & 1u;
-    if (which + 1u < chunks) fetch(which + 1u);
-    const uint32_t first_row = which * kTokens;
-    const uint32_t tokens = min(kTokens, run.rows - first_row);
-    const float* base = reinterpret_cast<const float*>(chunk[slot]) + part * KPL;
-    float kept = 0.0f;
-    for (uint32_t t = 0; t < tokens; ++t) {
-      const float* at = base + t * kVectors * kPadded;
-      float r[KPL], k[KPL], w[KPL];
+    fetch(min(which + 1u, chunks - 1u));
+    for (uint32_t first = 0; first < kTokens; first += kBlock) {
+      float parts[16] = {};
+      Token token[2];
+      read(token[0], slot, first);
 #pragma unroll
-      for (int i = 0; i < KPL; ++i) {
-        r[i] = at[i];
-        k[i] = at[kPadded + i];
-        w[i] = at[2u * kPadded + i];
+      for (uint32_t t = 0; t < kBlock; ++t) {
+        if (t + 1u < kBlock) read(token[(t + 1u) % 2u], slot, first + t + 1u);
+        parts[t] = advance(token[t % 2u]);
       }
-      const float value = values[slot][t][threadIdx.x / 16u];
-      float out;
-      if constexpr (DELTA) {
-        float u[KPL], au[KPL];
-#pragma unroll
-        for (int i = 0; i < KPL; ++i) {
-          u[i] = at[3u * kPadded + i];
-          au[i] = at[4u * kPadded + i];
-        }
-        float dot = u[0] * s[0];
-#pragma unroll
-        for (int i = 1; i < KPL; ++i) dot = fmaf(u[i], s[i], dot);
-        // while the dot product travels: the part that does not need it
-#pragma unroll
-        for (int i = 0; i < KPL; ++i) s[i] = fmaf(k[i], value, w[i] * s[i]);
-        dot = row16_sum(dot);
-#pragma unroll
-        for (int i = 0; i < KPL; ++i) s[i] = fmaf(-au[i], dot, s[i]);
-        out = r[0] * s[0];
-#pragma unroll
-        for (int i = 1; i < KPL; ++i) out = fmaf(r[i], s[i], out);
-        out = row16_sum(out);
-      } else {
-        out = r[0] * s[0];
-#pragma unroll
-        for (int i = 1; i < KPL; ++i) out = fmaf(r[i], s[i], out);
-#pragma unroll
-        for (int i = 0; i < KPL; ++i) s[i] = fmaf(k[i], value, w[i] * s[i]);
-        out = fmaf(bonus[slot][t], value, row16_sum(out));
-      }
-      // every lane of the sixteen has the sum: lane t keeps token t's until
-      // sixteen tokens are stored at once
-      kept = t % 16u == part ? out : kept;
-      if (t % 16u == 15u || t + 1u == tokens) {
-        const uint32_t token = first_row + t / 16u * 16u + part;
-        if (real && token < first_row + tokens)
-          args.outputs[size_t{token} * l.heads * dim + head * dim + column] = kept;
-      }
+      float out = row16_transposed_sum(parts);
+      const uint32_t mine = first + part;
+      if (!DELTA && part < kBlock)
+        out = fmaf(bonus[slot][mine], values[slot][mine][threadIdx.x / 16u], out);
+      const uint32_t row = which * kTokens + mine;
+      if (real && part < kBlock && row < run.rows)
+        args.outputs[size_t{row} * l.heads * dim + head * dim + column] = out;
     }
-    if (which + 1u < chunks) publish(1u - slot);
+    publish(1u - slot, which + 1u);
     __syncthreads();
   }
 #pragma unroll
@@ -497,7 +571,8 @@ extern "C" int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
   args.scalars = reinterpret_cast<float*>(bytes + prepared_bytes(l, launch->rows));
   args.outputs = reinterpret_cast<float*>(bytes + prepared_bytes(l, launch->rows) +
                                           scalar_bytes(l, launch->rows));
-  recurrence_prepare_kernel<<<dim3((launch->rows + kPrepareRows - 1u) / kPrepareRows,
+  const uint32_t prepare_rows = 256u / args.padded * kRowsPerThread;
+  recurrence_prepare_kernel<<<dim3((launch->rows + prepare_rows - 1u) / prepare_rows,
                                    l.heads),
                               256, 0, hip_stream>>>(args);
   if (delta)

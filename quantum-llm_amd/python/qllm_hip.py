@@ -92,6 +92,77 @@ class Q8AttentionLaunch(Structure):
 
 
 # name -> (restype, argtypes); every symbol include/qllm_kernels.h declares.
+ELEMENT_BF16 = 0
+ELEMENT_F32 = 1
+LINEAR_STORE, LINEAR_ADD, LINEAR_GATED, LINEAR_PARTIALS = range(4)
+RECURRENCE_DELTA, RECURRENCE_BONUS = range(2)
+
+
+class LinearSegment(Structure):
+    _fields_ = [("weights", c_void_p), ("input", c_void_p), ("output", c_void_p),
+                ("rows", c_uint32), ("columns", c_uint32), ("input_stride", c_uint32),
+                ("output_stride", c_uint32), ("output_columns", c_uint32),
+                ("epilogue", c_uint32), ("activation", c_uint32), ("splits", c_uint32)]
+
+
+class TokenShift(Structure):
+    _fields_ = [("count", c_uint32), ("mu", c_void_p * 6), ("output", c_void_p * 6),
+                ("previous", c_void_p), ("slot_stride", c_uint64), ("last", c_void_p)]
+
+
+class StreamNormLaunch(Structure):
+    _fields_ = [("input", c_void_p), ("stream_out", c_void_p), ("partials", c_void_p),
+                ("partial_count", c_uint32), ("partial_stride", c_uint32),
+                ("weight", c_void_p * 2), ("output", c_void_p * 2),
+                ("stride", c_uint32 * 2), ("rows", c_uint32), ("width", c_uint32),
+                ("epsilon", c_float), ("element", c_uint32),
+                ("shift", POINTER(TokenShift)), ("gather", c_void_p), ("step", c_void_p)]
+
+
+class WindowedAttention(Structure):
+    _fields_ = [("query_heads", c_uint32), ("kv_heads", c_uint32), ("dim", c_uint32),
+                ("vdim", c_uint32), ("key_stride", c_uint32), ("value_stride", c_uint32),
+                ("window", c_uint32), ("sinks", c_uint32), ("scale", c_float),
+                ("head_mix", c_void_p), ("page_tokens", c_uint32),
+                ("pages_per_slot", c_uint32), ("layer_offset", c_uint64),
+                ("page_table", c_void_p), ("step", c_void_p), ("element", c_uint32)]
+
+
+class RopeStoreLaunch(Structure):
+    _fields_ = [("projections", c_void_p), ("stride", c_uint32),
+                ("query_column", c_uint32), ("key_column", c_uint32),
+                ("value_column", c_uint32), ("rotary_dims", c_uint32),
+                ("frequencies", c_void_p), ("first_values", c_void_p),
+                ("value_share", c_void_p), ("values_out", c_void_p),
+                ("query_out", c_void_p), ("rows", c_uint32)]
+
+
+class AttentionLaunch(Structure):
+    _fields_ = [("query", c_void_p), ("gate", c_void_p), ("gate_stride", c_uint32),
+                ("output", c_void_p), ("output_stride", c_uint32), ("rows", c_uint32),
+                ("maximum_position", c_uint32), ("workspace", c_void_p),
+                ("workspace_bytes", c_size_t)]
+
+
+class Recurrence(Structure):
+    _fields_ = [("kind", c_uint32), ("heads", c_uint32), ("dim", c_uint32),
+                ("rank", c_uint32), ("gate_kind", c_uint32), ("epsilon", c_float),
+                ("unit_epsilon", c_float), ("decay_scale", c_float),
+                ("decay_up_bf16", c_void_p), ("decay_base", c_void_p),
+                ("rate_bias", c_void_p), ("bonus", c_void_p), ("norm_weight", c_void_p),
+                ("state", c_void_p), ("slot_stride", c_uint64), ("step", c_void_p),
+                ("element", c_uint32)]
+
+
+class RecurrenceLaunch(Structure):
+    _fields_ = [("projections", c_void_p), ("stride", c_uint32), ("r_column", c_uint32),
+                ("k_column", c_uint32), ("v_column", c_uint32), ("gate_column", c_uint32),
+                ("rate_column", c_uint32), ("low_column", c_uint32), ("output", c_void_p),
+                ("output_stride", c_uint32), ("rows", c_uint32), ("carry_from", c_void_p),
+                ("carry_to", c_void_p), ("carry_width", c_uint32), ("workspace", c_void_p),
+                ("workspace_bytes", c_size_t)]
+
+
 SIGNATURES = {
     "qllm_last_error": (c_char_p, []),
     "qllm_version": (c_char_p, []),
@@ -164,6 +235,18 @@ SIGNATURES = {
     "qllm_apply_presence_penalty": (c_int32, [c_void_p, c_void_p, c_uint32, c_float, c_void_p]),
     "qllm_apply_presence_penalty_rows": (c_int32, [c_void_p, c_size_t, c_void_p, c_void_p, c_uint32, c_uint32, c_float, c_void_p]),
     "qllm_mark_presence": (c_int32, [c_void_p, c_void_p, c_uint32, c_uint32, c_void_p]),
+    "qllm_linear_packed_bytes": (c_size_t, [c_uint32, c_uint32]),
+    "qllm_linear_pack": (c_int32, [c_void_p, c_uint32, c_uint32, c_void_p, c_uint32, c_uint32, c_uint32, c_uint32, c_void_p]),
+    "qllm_linear_batch": (c_int32, [POINTER(LinearSegment), c_uint32, c_uint32, c_uint32, c_void_p]),
+    "qllm_embedding_bf16_batch": (c_int32, [c_void_p, c_uint32, c_void_p, c_void_p, c_uint32, c_uint32, c_float, c_void_p]),
+    "qllm_stream_norm": (c_int32, [POINTER(StreamNormLaunch), c_void_p]),
+    "qllm_windowed_layer_bytes": (c_size_t, [c_uint32, c_uint32, c_uint32, c_uint32, c_uint32]),
+    "qllm_windowed_rope_store": (c_int32, [POINTER(WindowedAttention), POINTER(RopeStoreLaunch), c_void_p]),
+    "qllm_windowed_attention_workspace_bytes": (c_size_t, [POINTER(WindowedAttention), c_uint32]),
+    "qllm_windowed_attention_form": (c_uint32, [POINTER(WindowedAttention), c_uint32]),
+    "qllm_windowed_attention_rows": (c_int32, [POINTER(WindowedAttention), POINTER(AttentionLaunch), c_void_p]),
+    "qllm_recurrence_workspace_bytes": (c_size_t, [POINTER(Recurrence), c_uint32]),
+    "qllm_recurrence_rows": (c_int32, [POINTER(Recurrence), POINTER(RecurrenceLaunch), c_void_p]),
     "qllm_fill_random": (c_int32, [c_void_p, c_size_t, c_uint32, c_uint64, c_void_p]),
 }
 

@@ -73,6 +73,16 @@ SIGNATURES = {
     "qllm_sampling_counter_uniform": (c_double, [c_uint64, c_uint32, c_uint32, c_uint32]),
     "qllm_provider_create_from_artifact": (c_void_p, [c_char_p, c_uint32, c_uint32, c_char_p, c_uint32]),
     "qllm_provider_prefill": (c_int32, [c_void_p, c_void_p, c_uint32, c_uint32, POINTER(c_uint32)]),
+    "qllm_model_open": (c_void_p, [c_char_p, c_uint32, c_uint32, c_uint32, c_char_p, c_uint32]),
+    "qllm_model_close": (None, [c_void_p]),
+    "qllm_model_vocabulary": (c_uint32, [c_void_p]),
+    "qllm_model_hidden": (c_uint32, [c_void_p]),
+    "qllm_model_batch_limit": (c_uint32, [c_void_p]),
+    "qllm_model_begin": (c_int32, [c_void_p, c_uint32, c_uint32, c_uint32, c_uint32, c_int32, c_uint64, c_uint32, POINTER(c_uint64)]),
+    "qllm_model_end": (c_int32, [c_void_p, c_uint64]),
+    "qllm_model_step": (c_int32, [c_void_p, c_uint64, c_void_p, c_uint32, c_void_p, c_uint32, c_void_p, POINTER(c_uint32)]),
+    "qllm_model_trace_layers": (c_int32, [c_void_p, c_uint64, c_void_p, c_uint32, c_void_p, POINTER(c_uint32)]),
+    "qllm_model_telemetry": (c_uint64, [c_void_p, c_char_p]),
     "qllm_sha256": (c_int32, [c_void_p, c_size_t, c_void_p]),
     "qllm_sha256_portable": (c_int32, [c_void_p, c_size_t, c_void_p]),
     "qllm_artifact_open": (c_int32, [c_char_p, c_uint32, c_int32, POINTER(c_void_p)]),
@@ -384,3 +394,61 @@ def rejection_sample(proposal, target, draft, acceptance_uniform,
 
 def counter_uniform(seed, position, stream, index=0):
     return load().qllm_sampling_counter_uniform(seed, position, stream, index)
+
+
+class Model:
+    """An opened model (artifact directory or model folder), driven batch by
+    batch through its compiled program."""
+
+    def __init__(self, path, max_context, capacity=1, kv_page_tokens=64,
+                 kv_cache_dtype="artifact", chunk_rows=0):
+        self._handle = load().qllm_model_open(os.fsencode(path), max_context, capacity,
+                                              kv_page_tokens, kv_cache_dtype.encode(),
+                                              chunk_rows)
+        if not self._handle:
+            raise ProviderError(-1, load().qllm_provider_last_error().decode())
+        self.vocabulary = load().qllm_model_vocabulary(self._handle)
+        self.hidden = load().qllm_model_hidden(self._handle)
+        self.batch_limit = load().qllm_model_batch_limit(self._handle)
+
+    def begin(self, temperature_ppm=0, top_p_ppm=1000000, top_k=0, min_p_ppm=0,
+              presence_ppm=0, seed=0, first_output_position=0):
+        request = c_uint64()
+        _check(load().qllm_model_begin(self._handle, temperature_ppm, top_p_ppm, top_k,
+                                       min_p_ppm, presence_ppm, seed,
+                                       first_output_position, ctypes.byref(request)))
+        return request.value
+
+    def end(self, request):
+        _check(load().qllm_model_end(self._handle, request))
+
+    def step(self, request, tokens, want=()):
+        """(logits [len(want), vocabulary], token selected after the last one)."""
+        import numpy as np
+        tokens = np.ascontiguousarray(tokens, dtype=np.uint32)
+        want = np.ascontiguousarray(want, dtype=np.uint32)
+        logits = np.zeros((want.size, self.vocabulary), dtype=np.float32)
+        token = c_uint32()
+        _check(load().qllm_model_step(self._handle, request, tokens.ctypes.data,
+                                      tokens.size, want.ctypes.data, want.size,
+                                      logits.ctypes.data, ctypes.byref(token)))
+        return logits, token.value
+
+    def trace_layers(self, request, tokens, layers):
+        """(residual stream after every layer [layers, tokens, hidden], token)."""
+        import numpy as np
+        tokens = np.ascontiguousarray(tokens, dtype=np.uint32)
+        hidden = np.zeros((layers, tokens.size, self.hidden), dtype=np.float32)
+        token = c_uint32()
+        _check(load().qllm_model_trace_layers(self._handle, request, tokens.ctypes.data,
+                                              tokens.size, hidden.ctypes.data,
+                                              ctypes.byref(token)))
+        return hidden, token.value
+
+    def telemetry(self, name):
+        return load().qllm_model_telemetry(self._handle, name.encode())
+
+    def close(self):
+        if self._handle:
+            load().qllm_model_close(self._handle)
+            self._handle = None
