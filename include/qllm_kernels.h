@@ -999,7 +999,7 @@ typedef struct qllm_windowed_attention {
   uint32_t value_stride;       /* vdim padded to 16 */
   uint32_t window, sinks;
   float scale;
-  const float* head_mix;       /* device f32 [heads][heads]; NULL = none */
+  const float* head_mix;       /* device f32 [heads][heads], bf16 values; NULL = none */
   uint32_t page_tokens;        /* a multiple of 32 */
   uint32_t pages_per_slot;
   uint64_t layer_offset;       /* bytes */
@@ -1053,7 +1053,8 @@ typedef struct qllm_attention_launch {
   size_t workspace_bytes;
 } qllm_attention_launch;
 size_t qllm_windowed_attention_workspace_bytes(
-    const qllm_windowed_attention* attention, uint32_t maximum_position);
+    const qllm_windowed_attention* attention, uint32_t rows,
+    uint32_t maximum_position);
 enum qllm_attention_form {
   QLLM_ATTENTION_GENERAL = 0,
   QLLM_ATTENTION_SPLIT = 1,

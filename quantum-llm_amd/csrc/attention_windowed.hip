@@ -9,13 +9,12 @@
 //    per wave, with each workgroup's maximum and sum; then, per key/value head,
 //    normalise, mix (F32) and multiply with the values, the visible tiles dealt
 //    over workgroups; then the partial outputs are added and gated.
-//  * prompt: a workgroup owns 16 query rows and all heads, a wave up to four
-//    heads.  A first walk over the visible keys takes every row's maximum and
-//    sum, a second recomputes the scores, leaves the normalised weights in LDS
-//    as bf16 high and low halves (together 16 bits of mantissa), lets the
-//    matrix cores mix them over heads - the mix matrix is bf16 as stored, so
-//    both products are exact and added in F32 - and multiplies the mixed
-//    weights with the values.
+//  * prompt: a first walk over the visible keys takes every row's softmax
+//    denominator.  In a second, a workgroup owns 16 query rows and all heads: it
+//    recomputes the scores, leaves the normalised weights in LDS as bf16 high
+//    and low halves (together 16 bits of mantissa), lets the matrix cores mix
+//    them over heads - the mix matrix is bf16 as stored, so both products are
+//    exact and added in F32 - and multiplies the mixed weights with the values.
 //  * general: one workgroup per row, any size, bf16 or F32 arithmetic.
 //
 // Keys lie in fragments of 16 tokens x 32 dimensions and values, transposed, in
@@ -66,11 +65,19 @@ __device__ __forceinline__ bool visible(const Attention& a, uint32_t position,
   return key <= position && (!a.window || position - key < a.window || key < a.sinks);
 }
 
+// The request's row of the page table, and the layer's part of a page.
+__device__ __forceinline__ void* const* pages_of(const Attention& a) {
+  return a.page_table + size_t{a.step[kStepSlot]} * a.pages_per_slot;
+}
+template <typename T>
+__device__ __forceinline__ T* page_of(const Attention& a, void* const* pages,
+                                      uint32_t position) {
+  return reinterpret_cast<T*>(static_cast<uint8_t*>(pages[position / a.page_tokens]) +
+                              a.layer_offset);
+}
 template <typename T>
 __device__ __forceinline__ T* page_of(const Attention& a, uint32_t position) {
-  void* const* table = a.page_table + size_t{a.step[kStepSlot]} * a.pages_per_slot;
-  return reinterpret_cast<T*>(static_cast<uint8_t*>(table[position / a.page_tokens]) +
-                              a.layer_offset);
+  return page_of<T>(a, pages_of(a), position);
 }
 
 // Element offsets of fragment rows inside a layer of a page.
@@ -523,149 +530,121 @@ __device__ __forceinline__ void split_pair(float a, float b, uint32_t& high,
                   b - __uint_as_float(b_bits & 0xffff0000u));
 }
 
-// HPW heads per wave, NK = key_stride / 32, NV = value_stride / 16.
-//
-// The wave's keys are fetched one tile ahead: their registers are free as soon
-// as the tile's scores are out, and the fetch then has the rest of the
-// iteration to arrive.  With up to 16 heads (HPW <= 2) the high and the low
-// halves of the weights share one matrix operand - the mix matrix stands in it
-// twice - and with up to 32 they take one each.
-template <int HPW, int NK, int NV>
-__global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs args) {
-  constexpr bool kFolded = HPW <= 2;
-  constexpr int kHeadTiles = kFolded ? 1 : 2;
-  constexpr int kMixHeads = kFolded ? 16 : 32;
-  constexpr int kPairs = (HPW + 1) / 2;
-  constexpr bool kEarlyValues = HPW <= 2;
-  // normalised weights [key][query row][64 bytes of heads]
-  __shared__ __attribute__((aligned(16))) uint8_t high[512 * 64];
-  __shared__ __attribute__((aligned(16))) uint8_t low_plane[kFolded ? 16 : 512 * 64];
-  // mixed weights [head][query row][key]
-  __shared__ __attribute__((aligned(16))) uint8_t mixed[kMixHeads * 16 * 64];
-  uint8_t* const low = kFolded ? high : low_plane;
-  constexpr uint32_t kLowSlot = kFolded ? 2u : 0u;
+// Row blocks of the prompt kernels: contiguous ranges per XCD (consecutive
+// workgroups go round the XCDs), since neighbours share their keys.
+__device__ __forceinline__ uint32_t xcd_range(uint32_t block, uint32_t blocks) {
+  const uint32_t per_xcd = blocks / 8u;
+  return block < per_xcd * 8u ? block % 8u * per_xcd + block / 8u : block;
+}
+
+// Keys of one tile as matrix operands: 16 tokens x 32 dimensions each.
+template <int NK>
+__device__ __forceinline__ void fetch_tile_keys(i32x4 (&k)[2][NK], const Attention& a,
+                                                void* const* pages, uint32_t tile,
+                                                uint32_t kv_head) {
+  const uint32_t lane = threadIdx.x % kWave;
+  const uint32_t key0 = tile * kTileKeys;
+  const i32x4* keys = reinterpret_cast<const i32x4*>(
+                          page_of<const uint16_t>(a, pages, key0) +
+                          key_block(a, kv_head, key0 % a.page_tokens)) +
+                      lane % 16u * 4u + lane / 16u;
+#pragma unroll
+  for (int half = 0; half < 2; ++half)
+#pragma unroll
+    for (int c = 0; c < NK; ++c) k[half][c] = keys[(half * NK + c) * kWave];
+}
+
+// s[half][i] = product of key 16 half + 4 quarter + i with query row column.
+template <int NK>
+__device__ __forceinline__ void tile_products(const i32x4 (&k)[2][NK],
+                                              const i32x4 (&query)[NK], f32x4 (&s)[2]) {
+#pragma unroll
+  for (int half = 0; half < 2; ++half) {
+    s[half] = f32x4{};
+#pragma unroll
+    for (int c = 0; c < NK; ++c) s[half] = mfma_bf16(k[half][c], query[c], s[half]);
+  }
+}
+
+__device__ __forceinline__ void hide_keys(const Attention& a, uint32_t position,
+                                          uint32_t tile, f32x4 (&s)[2]) {
+  const uint32_t key0 = tile * kTileKeys + 4u * (threadIdx.x % kWave / 16u);
+#pragma unroll
+  for (int half = 0; half < 2; ++half)
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (!visible(a, position, key0 + half * 16u + i)) s[half][i] = -INFINITY;
+}
+
+// Rows first .. first + 15 all see every key of the tile.
+__device__ __forceinline__ bool tile_open(const Attention& a, uint32_t first,
+                                          uint32_t tile) {
+  const uint32_t first_key = tile * kTileKeys;
+  const uint32_t last_key = first_key + kTileKeys - 1u;
+  return last_key <= first &&
+         (!a.window || first + 15u - first_key < a.window || last_key < a.sinks);
+}
+
+template <int NK>
+__device__ __forceinline__ void load_query(i32x4 (&q)[NK], const AttentionArgs& args,
+                                           uint32_t row, uint32_t head) {
+  const Attention& a = args.attention;
+  const uint16_t* query = static_cast<const uint16_t*>(args.launch.query) +
+                          (size_t{row} * a.query_heads + head) * a.key_stride +
+                          8u * (threadIdx.x % kWave / 16u);
+#pragma unroll
+  for (int c = 0; c < NK; ++c) q[c] = *reinterpret_cast<const i32x4*>(query + c * 32);
+}
+
+// First walk: for every row and head the logarithm of the softmax denominator,
+// in units of the base-2 exponent (maximum + log2 of the sum), so that
+// exp2(score - it) is the normalised weight.  A workgroup owns 16 rows and up
+// to HP heads of one key/value head; its waves deal the tiles among them.
+template <int HP, int NK>
+__global__ __launch_bounds__(256, 2) void prompt_denominators_kernel(AttentionArgs args) {
+  __shared__ float wave_maximum[4][HP][16];
+  __shared__ float wave_total[4][HP][16];
   const Attention& a = args.attention;
   const auto& run = args.launch;
   const uint32_t heads = a.query_heads;
   const uint32_t group = heads / a.kv_heads;
   const uint32_t wave = threadIdx.x / kWave;
-  const uint32_t waves = blockDim.x / kWave;
   const uint32_t lane = threadIdx.x % kWave;
   const uint32_t column = lane % 16u;
-  const uint32_t quarter = lane / 16u;
-  // contiguous ranges of row blocks per XCD: neighbours share their keys
-  uint32_t block = blockIdx.x;
-  {
-    const uint32_t per_xcd = gridDim.x / 8u;
-    if (block < per_xcd * 8u) block = block % 8u * per_xcd + block / 8u;
-  }
-  const uint32_t row0 = block * 16u;
+  const uint32_t row0 = xcd_range(blockIdx.x, gridDim.x) * 16u;
+  const uint32_t kv = blockIdx.y;
+  const uint32_t head0 = kv * group + blockIdx.z * HP;
+  const uint32_t count = min(uint32_t{HP}, group - blockIdx.z * HP);
   const uint32_t first = a.step[kStepPosition] + row0;
-  const uint32_t position = first + column;            // of this lane's query row
+  const uint32_t position = first + column;
   const uint32_t last = first + min(16u, run.rows - row0) - 1u;
   const TileRange range = tiles_for(a, first, last);
-
-  for (uint32_t i = threadIdx.x; i < sizeof(high) / 16u; i += blockDim.x) {
-    reinterpret_cast<i32x4*>(high)[i] = i32x4{};
-    if (!kFolded) reinterpret_cast<i32x4*>(low_plane)[i] = i32x4{};
-  }
-
-  uint32_t kv[HPW];
-  i32x4 q[HPW][NK];
-  const uint32_t query_row = min(row0 + column, run.rows - 1u);
-#pragma unroll
-  for (int i = 0; i < HPW; ++i) {
-    const uint32_t head = min(wave * HPW + i, heads - 1u);
-    kv[i] = head / group;
-    const uint16_t* query = static_cast<const uint16_t*>(run.query) +
-                            (size_t{query_row} * heads + head) * a.key_stride + 8u * quarter;
-#pragma unroll
-    for (int c = 0; c < NK; ++c) q[i][c] = *reinterpret_cast<const i32x4*>(query + c * 32);
-  }
-  // rows head, columns other head of the mix matrix
-  i32x4 mix[kHeadTiles];
-#pragma unroll
-  for (int t = 0; t < kHeadTiles; ++t) {
-    uint32_t packed[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      float pair[2];
-#pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        const uint32_t h = t * 16u + column;
-        const uint32_t g = (8u * quarter + 2u * i + j) % kMixHeads;
-        pair[j] = h < heads && g < heads ? (a.head_mix ? a.head_mix[size_t{h} * heads + g]
-                                                       : (h == g ? 1.0f : 0.0f))
-                                         : 0.0f;
-      }
-      packed[i] = pack_bf16(pair[0], pair[1]);
-    }
-    mix[t] = i32x4{static_cast<int>(packed[0]), static_cast<int>(packed[1]),
-                   static_cast<int>(packed[2]), static_cast<int>(packed[3])};
-  }
-
-  const auto fetch_keys = [&](i32x4 (&k)[2][NK], uint32_t ordinal, uint32_t kv_head)
-      __attribute__((always_inline)) {
-    const uint32_t key0 = range.tile(ordinal) * kTileKeys;
-    const i32x4* keys = reinterpret_cast<const i32x4*>(
-                            page_of<const uint16_t>(a, key0) +
-                            key_block(a, kv_head, key0 % a.page_tokens)) +
-                        column * 4u + quarter;
-#pragma unroll
-    for (int half = 0; half < 2; ++half)
-#pragma unroll
-      for (int c = 0; c < NK; ++c) k[half][c] = keys[(half * NK + c) * kWave];
-  };
-  const auto products = [&](const i32x4 (&k)[2][NK], const i32x4 (&query)[NK],
-                            f32x4 (&s)[2]) __attribute__((always_inline)) {
-#pragma unroll
-    for (int half = 0; half < 2; ++half) {
-      s[half] = f32x4{};
-#pragma unroll
-      for (int c = 0; c < NK; ++c) s[half] = mfma_bf16(k[half][c], query[c], s[half]);
-    }
-  };
-  // s[half][i] = key 16 half + 4 quarter + i of the tile, query row column
-  const auto hide = [&](f32x4 (&s)[2], uint32_t tile) __attribute__((always_inline)) {
-    const uint32_t key0 = tile * kTileKeys + 4u * quarter;
-#pragma unroll
-    for (int half = 0; half < 2; ++half)
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (!visible(a, position, key0 + half * 16u + i)) s[half][i] = -INFINITY;
-  };
-  // every row of the block sees every key of the tile
-  const auto open = [&](uint32_t tile) {
-    const uint32_t first_key = tile * kTileKeys;
-    const uint32_t last_key = first_key + kTileKeys - 1u;
-    return last_key <= first &&
-           (!a.window || first + 15u - first_key < a.window || last_key < a.sinks);
-  };
-
-  // scores in units of the base-2 exponent; exp2(-inf) = 0 hides a key
+  void* const* const pages = pages_of(a);
   const float unit = a.scale * 1.4426950408889634f;
-  float maximum[HPW], total[HPW];
+
+  i32x4 q[HP][NK];
 #pragma unroll
-  for (int i = 0; i < HPW; ++i) {
+  for (int i = 0; i < HP; ++i)
+    load_query<NK>(q[i], args, min(row0 + column, run.rows - 1u),
+                   head0 + min(static_cast<uint32_t>(i), count - 1u));
+  float maximum[HP], total[HP];
+#pragma unroll
+  for (int i = 0; i < HP; ++i) {
     maximum[i] = -INFINITY;
     total[i] = 0.0f;
   }
-  const auto survey = [&](i32x4 (&k)[2][NK], uint32_t ordinal, uint32_t ahead)
-      __attribute__((always_inline)) {
+  const auto survey = [&](i32x4 (&k)[2][NK], uint32_t ordinal) __attribute__((always_inline)) {
     const uint32_t tile = range.tile(ordinal);
-    const bool all = open(tile);
-    f32x4 s[HPW][2];
+    const bool all = tile_open(a, first, tile);
+    f32x4 s[HP][2];
 #pragma unroll
-    for (int i = 0; i < HPW; ++i) {
-      if (i > 0 && kv[i] != kv[i - 1]) fetch_keys(k, ordinal, kv[i]);
-      products(k, q[i], s[i]);
-    }
-    fetch_keys(k, min(ahead, range.count - 1u), kv[0]);
+    for (int i = 0; i < HP; ++i) tile_products<NK>(k, q[i], s[i]);
+    fetch_tile_keys<NK>(k, a, pages, range.tile(min(ordinal + 8u, range.count - 1u)), kv);
 #pragma unroll
-    for (int i = 0; i < HPW; ++i) {
+    for (int i = 0; i < HP; ++i) {
 #pragma unroll
       for (int half = 0; half < 2; ++half) s[i][half] *= unit;
-      if (!all) hide(s[i], tile);
+      if (!all) hide_keys(a, position, tile, s[i]);
       float top = maximum[i];
 #pragma unroll
       for (int half = 0; half < 2; ++half)
@@ -682,56 +661,146 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
       maximum[i] = top;
     }
   };
-  {
+  if (wave < range.count) {
     i32x4 even[2][NK], odd[2][NK];
-    fetch_keys(even, 0u, kv[0]);
-    if constexpr (HPW <= 2) {
-      fetch_keys(odd, min(1u, range.count - 1u), kv[0]);
-      uint32_t ordinal = 0;
-      for (; ordinal + 2u <= range.count; ordinal += 2u) {
-        survey(even, ordinal, ordinal + 2u);
-        survey(odd, ordinal + 1u, ordinal + 3u);
-      }
-      if (ordinal < range.count) survey(even, ordinal, ordinal);
-    } else {
-      for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal)
-        survey(even, ordinal, ordinal + 1u);
+    fetch_tile_keys<NK>(even, a, pages, range.tile(wave), kv);
+    fetch_tile_keys<NK>(odd, a, pages, range.tile(min(wave + 4u, range.count - 1u)), kv);
+    uint32_t ordinal = wave;
+    for (; ordinal + 4u < range.count; ordinal += 8u) {
+      survey(even, ordinal);
+      survey(odd, ordinal + 4u);
+    }
+    if (ordinal < range.count) survey(even, ordinal);
+  }
+  const auto merge = [](float& m, float& t, float other, float other_total) {
+    const float top = fmaxf(m, other);
+    const float base = top == -INFINITY ? 0.0f : top;
+    t = t * __builtin_amdgcn_exp2f(m - base) +
+        other_total * __builtin_amdgcn_exp2f(other - base);
+    m = top;
+  };
+#pragma unroll
+  for (int i = 0; i < HP; ++i) {
+#pragma unroll
+    for (int offset = 16; offset <= 32; offset *= 2)
+      merge(maximum[i], total[i], __shfl_xor(maximum[i], offset, kWave),
+            __shfl_xor(total[i], offset, kWave));
+    if (lane < 16u) {
+      wave_maximum[wave][i][lane] = maximum[i];
+      wave_total[wave][i][lane] = total[i];
     }
   }
-  // from here on maximum holds maximum + log2(total): exp2(score - it) is the
-  // normalised weight
+  __syncthreads();
+  for (uint32_t i = threadIdx.x; i < 16u * count; i += blockDim.x) {
+    const uint32_t row = row0 + i % 16u;
+    if (row >= run.rows) continue;
+    float m = wave_maximum[0][i / 16u][i % 16u];
+    float t = wave_total[0][i / 16u][i % 16u];
+    for (uint32_t other = 1; other < 4u; ++other)
+      merge(m, t, wave_maximum[other][i / 16u][i % 16u], wave_total[other][i / 16u][i % 16u]);
+    args.maxima[size_t{row} * heads + head0 + i / 16u] = m + log2f(t);
+  }
+}
+
+// Second walk: HPW score heads and OPW output heads per wave (OPW <= HPW),
+// NK = key_stride / 32, NV = value_stride / 16.
+//
+// Every wave leaves its heads' normalised weights of a tile in LDS, the waves
+// mix them (four keys each) on the matrix cores, and every wave multiplies its
+// output heads' mixed weights with their values.  With up to 16 heads the high
+// and the low halves of the weights share one matrix operand - the mix matrix
+// stands in it twice; with up to 32 they take one each, and two workgroups
+// share the output heads of a row block (their accumulators would not fit the
+// registers of one).  The wave's keys are fetched one tile ahead: their
+// registers are free as soon as the tile's scores are out, and the fetch then
+// has the rest of the iteration to arrive.
+template <int HPW, int OPW, int NK, int NV, bool SHARED>
+__global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs args) {
+  constexpr bool kFolded = HPW <= 2;
+  constexpr int kMixHeads = kFolded ? 16 : 32;
+  constexpr int kPairs = (HPW + 1) / 2;
+  // normalised weights [key][query row][64 bytes of heads]
+  __shared__ __attribute__((aligned(16))) uint8_t high[512 * 64];
+  __shared__ __attribute__((aligned(16))) uint8_t low_plane[kFolded ? 16 : 512 * 64];
+  // mixed weights [output head][query row][key]
+  __shared__ __attribute__((aligned(16))) uint8_t mixed[16 * 16 * 64];
+  uint8_t* const low = kFolded ? high : low_plane;
+  constexpr uint32_t kLowSlot = kFolded ? 2u : 0u;
+  const Attention& a = args.attention;
+  const auto& run = args.launch;
+  const uint32_t heads = a.query_heads;
+  const uint32_t group = heads / a.kv_heads;
+  const uint32_t wave = threadIdx.x / kWave;
+  const uint32_t waves = blockDim.x / kWave;
+  const uint32_t lane = threadIdx.x % kWave;
+  const uint32_t column = lane % 16u;
+  const uint32_t quarter = lane / 16u;
+  const uint32_t row0 = xcd_range(blockIdx.x, gridDim.x) * 16u;
+  const uint32_t first_output = blockIdx.y * 16u;      // of this workgroup's heads
+  const uint32_t first = a.step[kStepPosition] + row0;
+  const uint32_t position = first + column;            // of this lane's query row
+  const uint32_t last = first + min(16u, run.rows - row0) - 1u;
+  const TileRange range = tiles_for(a, first, last);
+  void* const* const pages = pages_of(a);
+  const float unit = a.scale * 1.4426950408889634f;
+
+  for (uint32_t i = threadIdx.x; i < sizeof(high) / 16u; i += blockDim.x) {
+    reinterpret_cast<i32x4*>(high)[i] = i32x4{};
+    if (!kFolded) reinterpret_cast<i32x4*>(low_plane)[i] = i32x4{};
+  }
+
+  uint32_t kv[HPW], value_kv[OPW];
+  i32x4 q[HPW][NK];
+  float denominator[HPW];
+  const uint32_t query_row = min(row0 + column, run.rows - 1u);
 #pragma unroll
   for (int i = 0; i < HPW; ++i) {
+    const uint32_t head = min(wave * HPW + i, heads - 1u);
+    kv[i] = head / group;
+    load_query<NK>(q[i], args, query_row, head);
+    denominator[i] = args.maxima[size_t{query_row} * heads + head];
+  }
 #pragma unroll
-    for (int offset = 16; offset <= 32; offset *= 2) {
-      const float other = __shfl_xor(maximum[i], offset, kWave);
-      const float other_total = __shfl_xor(total[i], offset, kWave);
-      const float top = fmaxf(maximum[i], other);
-      const float base = top == -INFINITY ? 0.0f : top;
-      total[i] = total[i] * __builtin_amdgcn_exp2f(maximum[i] - base) +
-                 other_total * __builtin_amdgcn_exp2f(other - base);
-      maximum[i] = top;
+  for (int i = 0; i < OPW; ++i)
+    value_kv[i] = min(first_output + wave * OPW + i, heads - 1u) / group;
+  // rows output head, columns head of the mix matrix
+  i32x4 mix;
+  {
+    uint32_t packed[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float pair[2];
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const uint32_t h = first_output + column;
+        const uint32_t g = (8u * quarter + 2u * i + j) % kMixHeads;
+        const float stored =
+            a.head_mix ? a.head_mix[size_t{min(h, heads - 1u)} * heads + min(g, heads - 1u)]
+                       : (h == g ? 1.0f : 0.0f);
+        pair[j] = h < heads && g < heads ? stored : 0.0f;
+      }
+      packed[i] = pack_bf16(pair[0], pair[1]);
     }
-    maximum[i] += log2f(total[i]);
+    mix = i32x4{static_cast<int>(packed[0]), static_cast<int>(packed[1]),
+                static_cast<int>(packed[2]), static_cast<int>(packed[3])};
   }
   __syncthreads();   // the weight buffers are clear
 
-  f32x4 out[HPW][NV] = {};
+  f32x4 out[OPW][NV] = {};
   i32x4 k[2][NK];
-  fetch_keys(k, 0u, kv[0]);
-  const auto fetch_values = [&](uint32_t ordinal, uint32_t kv_head)
-      __attribute__((always_inline)) {
-    const uint32_t key0 = range.tile(ordinal) * kTileKeys;
-    return reinterpret_cast<const i32x4*>(page_of<const uint16_t>(a, key0) +
+  fetch_tile_keys<NK>(k, a, pages, range.tile(0u), kv[0]);
+  const auto values_at = [&](uint32_t tile, uint32_t kv_head) __attribute__((always_inline)) {
+    const uint32_t key0 = tile * kTileKeys;
+    return reinterpret_cast<const i32x4*>(page_of<const uint16_t>(a, pages, key0) +
                                           value_block(a, kv_head, key0 % a.page_tokens)) +
            column * 4u + quarter;
   };
   for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal) {
     const uint32_t tile = range.tile(ordinal);
-    const bool all = open(tile);
-    i32x4 v[kEarlyValues ? NV : 1];
-    if constexpr (kEarlyValues) {
-      const i32x4* values = fetch_values(ordinal, kv[0]);
+    const bool all = tile_open(a, first, tile);
+    i32x4 v[NV];
+    {
+      const i32x4* values = values_at(tile, value_kv[0]);
 #pragma unroll
       for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
     }
@@ -741,25 +810,27 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
 #pragma unroll
       for (int j = 0; j < 2 && 2 * pair + j < HPW; ++j) {
         const int i = 2 * pair + j;
-        if (i > 0 && kv[i] != kv[i - 1]) fetch_keys(k, ordinal, kv[i]);
-        products(k, q[i], s[j]);
+        if (!SHARED && i > 0 && kv[i] != kv[i - 1])
+          fetch_tile_keys<NK>(k, a, pages, tile, kv[i]);
+        tile_products<NK>(k, q[i], s[j]);
       }
-      if (pair + 1 == kPairs) fetch_keys(k, min(ordinal + 1u, range.count - 1u), kv[0]);
+      if (pair + 1 == kPairs)
+        fetch_tile_keys<NK>(k, a, pages, range.tile(min(ordinal + 1u, range.count - 1u)),
+                            kv[0]);
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         if (2 * pair + j >= HPW) {
           s[j][0] = s[j][1] = f32x4{};
           continue;
         }
-        if (!all) hide(s[j], tile);
-        const float offset = maximum[2 * pair + j];
+        const float offset = denominator[2 * pair + j];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          // a hidden key stays at minus infinity whatever the unit's sign
-          const float raw = s[j][e / 4][e % 4];
-          const float exponent = !all && raw == -INFINITY ? raw : fmaf(raw, unit, -offset);
-          s[j][e / 4][e % 4] = __builtin_amdgcn_exp2f(exponent);
-        }
+        for (int e = 0; e < 8; ++e)
+          s[j][e / 4][e % 4] = fmaf(s[j][e / 4][e % 4], unit, -offset);
+        if (!all) hide_keys(a, position, tile, s[j]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          s[j][e / 4][e % 4] = __builtin_amdgcn_exp2f(s[j][e / 4][e % 4]);
       }
       const uint32_t g = wave * HPW + 2u * pair;
       if (g < heads) {
@@ -782,97 +853,113 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
       }
     }
     __syncthreads();
-    // mix: four keys at a time, all query rows and heads
+    // mix: four keys at a time, all query rows, this workgroup's output heads
     for (uint32_t four = wave; four < 8u; four += waves) {
-      f32x4 m[4][kHeadTiles] = {};
+      f32x4 m[4] = {};
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const uint32_t at = swizzled((four * 4u + j) * 16u + column, quarter);
-        const i32x4 upper = *reinterpret_cast<const i32x4*>(high + at);
-        if constexpr (kFolded) {
-          m[j][0] = mfma_bf16(mix[0], upper, m[j][0]);
-        } else {
-          const i32x4 lower = *reinterpret_cast<const i32x4*>(low + at);
-#pragma unroll
-          for (int t = 0; t < kHeadTiles; ++t) {
-            m[j][t] = mfma_bf16(mix[t], lower, m[j][t]);
-            m[j][t] = mfma_bf16(mix[t], upper, m[j][t]);
-          }
-        }
+        if constexpr (!kFolded)
+          m[j] = mfma_bf16(mix, *reinterpret_cast<const i32x4*>(low + at), m[j]);
+        m[j] = mfma_bf16(mix, *reinterpret_cast<const i32x4*>(high + at), m[j]);
       }
 #pragma unroll
-      for (int t = 0; t < kHeadTiles; ++t)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const uint32_t h = t * 16u + 4u * quarter + i;
-          *reinterpret_cast<i32x2*>(mixed + h * 1024u + swizzled(column, four / 2u) +
-                                    four % 2u * 8u) =
-              i32x2{static_cast<int>(pack_bf16(m[0][t][i], m[1][t][i])),
-                    static_cast<int>(pack_bf16(m[2][t][i], m[3][t][i]))};
-        }
+      for (int i = 0; i < 4; ++i)
+        *reinterpret_cast<i32x2*>(mixed + (4u * quarter + i) * 1024u +
+                                  swizzled(column, four / 2u) + four % 2u * 8u) =
+            i32x2{static_cast<int>(pack_bf16(m[0][i], m[1][i])),
+                  static_cast<int>(pack_bf16(m[2][i], m[3][i]))};
     }
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < HPW; ++i) {
-      const uint32_t head = wave * HPW + i;
-      if (head >= heads) continue;
-      const i32x4 w = *reinterpret_cast<const i32x4*>(mixed + head * 1024u +
+    for (int i = 0; i < OPW; ++i) {
+      const uint32_t at = wave * OPW + i;
+      const i32x4 w = *reinterpret_cast<const i32x4*>(mixed + min(at, 15u) * 1024u +
                                                       swizzled(column, quarter));
-      if constexpr (kEarlyValues) {
-        if (i > 0 && kv[i] != kv[i - 1]) {
-          const i32x4* values = fetch_values(ordinal, kv[i]);
+      if (!SHARED && i > 0 && value_kv[i] != value_kv[i - 1]) {
+        const i32x4* values = values_at(tile, value_kv[i]);
 #pragma unroll
-          for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
-        }
-#pragma unroll
-        for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, v[t], out[i][t]);
-      } else {
-        const i32x4* values = fetch_values(ordinal, kv[i]);
-#pragma unroll
-        for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, values[t * kWave], out[i][t]);
+        for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
       }
+#pragma unroll
+      for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, v[t], out[i][t]);
     }
   }
 
+  float gate[OPW][4];
 #pragma unroll
-  for (int i = 0; i < HPW; ++i) {
-    const uint32_t head = wave * HPW + i;
-    if (head >= heads) continue;
+  for (int i = 0; i < OPW; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const uint32_t row = min(row0 + 4u * quarter + j, run.rows - 1u);
+      const uint32_t head = min(first_output + wave * OPW + i, heads - 1u);
+      gate[i][j] = run.gate ? run.gate[size_t{row} * run.gate_stride + head] : 0.0f;
+    }
+#pragma unroll
+  for (int i = 0; i < OPW; ++i) {
+    const uint32_t head = first_output + wave * OPW + i;
+    if (wave * OPW + i >= 16u || head >= heads) continue;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const uint32_t row = row0 + 4u * quarter + j;
       if (row >= run.rows) continue;
-      const float gate =
-          run.gate ? sigmoid_f32(run.gate[size_t{row} * run.gate_stride + head]) : 1.0f;
+      const float open_gate = run.gate ? sigmoid_f32(gate[i][j]) : 1.0f;
+      uint16_t* const output = static_cast<uint16_t*>(run.output) +
+                               size_t{row} * run.output_stride + head * a.vdim;
 #pragma unroll
       for (int t = 0; t < NV; ++t) {
         const uint32_t d = t * 16u + column;
-        if (d < a.vdim)
-          store_element(static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride +
-                            head * a.vdim + d,
-                        out[i][t][j] * gate);
+        if (d < a.vdim) store_element(output + d, out[i][t][j] * open_gate);
       }
     }
   }
 }
 
-template <int HPW, int NK>
-void launch_prompt_values(const AttentionArgs& args, dim3 grid, uint32_t threads,
-                          hipStream_t stream) {
-  if (args.attention.value_stride == 64u)
-    prompt_attention_kernel<HPW, NK, 4><<<grid, threads, 0, stream>>>(args);
+template <int NK>
+void launch_denominators(const AttentionArgs& args, hipStream_t stream) {
+  const Attention& a = args.attention;
+  const uint32_t group = a.query_heads / a.kv_heads;
+  const uint32_t blocks = (args.launch.rows + 15u) / 16u;
+  if (group == 1u)
+    prompt_denominators_kernel<1, NK><<<dim3(blocks, a.kv_heads), 256, 0, stream>>>(args);
+  else if (group == 2u)
+    prompt_denominators_kernel<2, NK><<<dim3(blocks, a.kv_heads), 256, 0, stream>>>(args);
   else
-    prompt_attention_kernel<HPW, NK, 8><<<grid, threads, 0, stream>>>(args);
+    prompt_denominators_kernel<4, NK>
+        <<<dim3(blocks, a.kv_heads, (group + 3u) / 4u), 256, 0, stream>>>(args);
 }
 
-template <int HPW>
-void launch_prompt(const AttentionArgs& args, hipStream_t stream) {
-  const uint32_t threads = (args.attention.query_heads + HPW - 1u) / HPW * kWave;
-  const dim3 grid((args.launch.rows + 15u) / 16u);
-  if (args.attention.key_stride == 64u)
-    launch_prompt_values<HPW, 2>(args, grid, threads, stream);
+template <int HPW, int OPW, int NK, int NV>
+void launch_prompt_form(const AttentionArgs& args, hipStream_t stream) {
+  const uint32_t heads = args.attention.query_heads;
+  const uint32_t group = heads / args.attention.kv_heads;
+  const uint32_t waves = HPW == 4 ? 8u : (heads + HPW - 1u) / HPW;
+  const dim3 grid((args.launch.rows + 15u) / 16u, HPW == 4 ? 2u : 1u);
+  // a wave's heads read one key/value head unless the groups are cut unevenly
+  if (HPW == 1 || group % HPW == 0u)
+    prompt_attention_kernel<HPW, OPW, NK, NV, true>
+        <<<grid, waves * kWave, 0, stream>>>(args);
   else
-    launch_prompt_values<HPW, 4>(args, grid, threads, stream);
+    prompt_attention_kernel<HPW, OPW, NK, NV, HPW == 1>
+        <<<grid, waves * kWave, 0, stream>>>(args);
+}
+
+template <int HPW, int OPW>
+void launch_prompt(const AttentionArgs& args, hipStream_t stream) {
+  const bool narrow_keys = args.attention.key_stride == 64u;
+  const bool narrow_values = args.attention.value_stride == 64u;
+  if (narrow_keys)
+    launch_denominators<2>(args, stream);
+  else
+    launch_denominators<4>(args, stream);
+  if (narrow_keys && narrow_values)
+    launch_prompt_form<HPW, OPW, 2, 4>(args, stream);
+  else if (narrow_keys)
+    launch_prompt_form<HPW, OPW, 2, 8>(args, stream);
+  else if (narrow_values)
+    launch_prompt_form<HPW, OPW, 4, 4>(args, stream);
+  else
+    launch_prompt_form<HPW, OPW, 4, 8>(args, stream);
 }
 
 bool valid_geometry(const Attention& a) {
@@ -962,13 +1049,15 @@ extern "C" uint32_t qllm_windowed_attention_form(const qllm_windowed_attention* 
 }
 
 extern "C" size_t qllm_windowed_attention_workspace_bytes(
-    const qllm_windowed_attention* attention, uint32_t maximum_position) {
+    const qllm_windowed_attention* attention, uint32_t rows, uint32_t maximum_position) {
   if (!attention || !attention->kv_heads || !attention->query_heads) return 0u;
   const uint32_t tiles = maximum_tiles(*attention, maximum_position);
   const size_t heads = attention->query_heads;
-  return kSplitRows * heads * 4u *
-         (size_t{tiles} * kTileKeys + size_t{score_splits_for(tiles)} * 2u +
-          size_t{value_splits_for(tiles)} * attention->vdim);
+  const size_t split = kSplitRows * heads * 4u *
+                       (size_t{tiles} * kTileKeys + size_t{score_splits_for(tiles)} * 2u +
+                        size_t{value_splits_for(tiles)} * attention->vdim);
+  const size_t prompt = size_t{rows} * heads * 4u;   // denominators
+  return split > prompt ? split : prompt;
 }
 
 extern "C" int32_t qllm_windowed_attention_rows(const qllm_windowed_attention* attention,
@@ -995,17 +1084,22 @@ extern "C" int32_t qllm_windowed_attention_rows(const qllm_windowed_attention* a
     return launched("windowed attention");
   }
   if (form == QLLM_ATTENTION_PROMPT) {
+    if (!launch->workspace ||
+        launch->workspace_bytes < size_t{launch->rows} * a.query_heads * 4u)
+      return fail(QLLM_INVALID_ARGUMENT, "windowed attention workspace is too small");
+    args.maxima = static_cast<float*>(launch->workspace);
     if (a.query_heads > 16u)
-      launch_prompt<4>(args, hip_stream);
+      launch_prompt<4, 2>(args, hip_stream);
     else if (a.query_heads > 8u)
-      launch_prompt<2>(args, hip_stream);
+      launch_prompt<2, 2>(args, hip_stream);
     else
-      launch_prompt<1>(args, hip_stream);
+      launch_prompt<1, 1>(args, hip_stream);
     return launched("windowed prompt attention");
   }
   if (!launch->workspace || (reinterpret_cast<uintptr_t>(launch->workspace) & 15u) != 0u ||
       launch->workspace_bytes <
-          qllm_windowed_attention_workspace_bytes(attention, launch->maximum_position))
+          qllm_windowed_attention_workspace_bytes(attention, launch->rows,
+                                                  launch->maximum_position))
     return fail(QLLM_INVALID_ARGUMENT, "windowed attention workspace is too small");
   const uint32_t tiles = maximum_tiles(a, launch->maximum_position);
   args.capacity = tiles * kTileKeys;

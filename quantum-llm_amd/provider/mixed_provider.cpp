@@ -561,7 +561,7 @@ void Mi355MixedProvider::ensure_workspace(std::uint32_t rows) {
       query = std::max(query, std::size_t{a.query_heads} * a.key_stride);
       kept = std::max(kept, std::size_t{a.kv_heads} * a.vdim);
       scratch = std::max(scratch, qllm_windowed_attention_workspace_bytes(
-                                      &a, g_.max_context - 1U));
+                                      &a, size, g_.max_context - 1U));
     } else {
       scratch = std::max(scratch, qllm_recurrence_workspace_bytes(&block.recurrence, size));
     }

@@ -242,7 +242,7 @@ SIGNATURES = {
     "qllm_stream_norm": (c_int32, [POINTER(StreamNormLaunch), c_void_p]),
     "qllm_windowed_layer_bytes": (c_size_t, [c_uint32, c_uint32, c_uint32, c_uint32, c_uint32]),
     "qllm_windowed_rope_store": (c_int32, [POINTER(WindowedAttention), POINTER(RopeStoreLaunch), c_void_p]),
-    "qllm_windowed_attention_workspace_bytes": (c_size_t, [POINTER(WindowedAttention), c_uint32]),
+    "qllm_windowed_attention_workspace_bytes": (c_size_t, [POINTER(WindowedAttention), c_uint32, c_uint32]),
     "qllm_windowed_attention_form": (c_uint32, [POINTER(WindowedAttention), c_uint32]),
     "qllm_windowed_attention_rows": (c_int32, [POINTER(WindowedAttention), POINTER(AttentionLaunch), c_void_p]),
     "qllm_recurrence_workspace_bytes": (c_size_t, [POINTER(Recurrence), c_uint32]),
