@@ -48,7 +48,7 @@ __device__ __forceinline__ void store_four(const qllm_linear_segment& s, float* 
                                            bool add) {
   if (n >= s.output_columns) return;
   float* out = base + size_t{m} * s.output_stride + n;
-  if (n + 4u <= s.output_columns) {
+  if (n + 4u <= s.output_columns && s.output_stride % 4u == 0u) {
     f32x4* vector = reinterpret_cast<f32x4*>(out);
     *vector = add ? *vector + value : value;
   } else {
@@ -281,7 +281,7 @@ __global__ __launch_bounds__(256, 2) void linear_tall_kernel(LinearArgs args) {
           const uint32_t at = first_tile + t;
           if (at >= weight_tiles) continue;
           const uint32_t n = at / 2u * 16u + 4u * (lane / 16u);
-          if (n + 4u <= s.output_columns) {
+          if (n + 4u <= s.output_columns && s.output_stride % 4u == 0u) {
             const f32x4 gate = sum[t][mt];
             const f32x4 up = sum[t + 1][mt];
             uint32_t bits[4];
@@ -475,7 +475,7 @@ extern "C" int32_t qllm_linear_batch(const qllm_linear_segment* segments, uint32
     const uint32_t outputs = gated ? s.rows / 2u : s.rows;
     if (!s.weights || !s.input || !s.output || !s.rows || !s.columns ||
         s.rows % (gated ? 32u : 16u) || s.columns % 64u || s.input_stride < s.columns ||
-        s.input_stride % 8u || s.output_stride % 4u || !s.output_columns ||
+        s.input_stride % 8u || !s.output_columns ||
         s.output_columns > outputs || s.output_stride < s.output_columns ||
         s.epilogue > QLLM_LINEAR_PARTIALS || s.activation > QLLM_ACTIVATION_SILU ||
         (partials && (!s.splits || s.splits > 16u || batch > 64u)) ||
