@@ -280,6 +280,94 @@ def measure_long_contexts(qp, np, rows):
     return report
 
 
+# Layers of about the size of a 1B and of a 7B model, four of them: attention,
+# generalised delta rule, bonus recurrence, attention.
+MIXED_SIZES = {
+    "width-2048": dict(width=2048, ff=5632, heads=16, kv_heads=4, recurrent_heads=32),
+    "width-4096": dict(width=4096, ff=14336, heads=32, kv_heads=8, recurrent_heads=64),
+}
+MIXED_WINDOW, MIXED_KEPT, MIXED_VOCABULARY = 1024, 4, 32000
+
+
+def measure_mixed(qp, np, prompt_tokens, steps, warmup):
+    """Prefill and greedy decode of the mixed-layer decoder (bf16, random
+    weights) beside the dense FP4 decoder with as many layers of the same width,
+    feed-forward, heads and vocabulary.  Prefill: from the call to the token
+    after the prompt.  Decode: one token after the other through the program,
+    each read back by the host; the dense decoder's one-row target pass is
+    replayed back to back (its decode step is speculative).  Bytes are those of
+    the weights a token reads."""
+    import shutil
+    import tempfile
+
+    import mixed_model as mm
+
+    report = {}
+    for name, size in MIXED_SIZES.items():
+        attention = mm.attention(size["heads"], size["kv_heads"], 128, 128, MIXED_WINDOW,
+                                 MIXED_KEPT)
+        layers = [attention, mm.general_delta(size["recurrent_heads"], 64),
+                  mm.wkv(size["recurrent_heads"], 64), attention]
+        config = mm.configuration(MIXED_VOCABULARY, size["width"], layers, [size["ff"]] * 4)
+        folder = tempfile.mkdtemp()
+        try:
+            mm.write_folder(folder, config, mm.TiledWeights(config, 1))
+            model = qp.Model(folder, prompt_tokens + warmup + steps + 8, kv_page_tokens=256)
+        finally:
+            shutil.rmtree(folder, ignore_errors=True)
+        tokens = np.random.default_rng(0).integers(0, MIXED_VOCABULARY, prompt_tokens)
+        prefill = []
+        for _ in range(4):               # the first one allocates and is not counted
+            request = model.begin()
+            begin = time.perf_counter()
+            _, token = model.step(request, tokens)
+            prefill.append(time.perf_counter() - begin)
+            if len(prefill) < 4:
+                model.end(request)
+        for index in range(warmup + steps):
+            if index == warmup:
+                begin = time.perf_counter()
+            _, token = model.step(request, [token])
+        decode = (time.perf_counter() - begin) / steps
+        read = model.telemetry("provider_weight_bytes") - 2 * MIXED_VOCABULARY * size["width"]
+        model.close()
+
+        geometry = dict(MODEL)
+        geometry.update(hidden=size["width"], intermediate=size["ff"], layers=4,
+                        query_heads=size["heads"], kv_heads=size["kv_heads"],
+                        vocabulary=MIXED_VOCABULARY, max_context=prompt_tokens + 256)
+        dense = qp.Provider(**geometry)
+        dense.load_synthetic_weights(3)
+        dense.prepare_exact_decode(
+            "decode.mtp.dense-full-attention.fp4-f16-block16.exact.v2")
+        dense.begin_request(temperature_ppm=0)
+        dense_prefill = []
+        for _ in range(4):
+            begin = time.perf_counter()
+            dense.prefill(tokens.astype(np.uint32), 0)
+            dense_prefill.append(time.perf_counter() - begin)
+        dense.capture_target(np.array([5], np.uint32), MIXED_WINDOW)
+        for index in range(warmup + steps):
+            if index == warmup:
+                dense.synchronize_stream()
+                begin = time.perf_counter()
+            dense.replay_target()
+        dense.synchronize_stream()
+        dense_decode = (time.perf_counter() - begin) / steps
+        dense.close()
+        report[name] = {
+            "prefill_tok_s": round(prompt_tokens / min(prefill[1:]), 1),
+            "prefill_ms": round(1e3 * min(prefill[1:]), 3),
+            "decode_tok_s": round(1.0 / decode, 1),
+            "decode_us_per_token": round(1e6 * decode, 1),
+            "decode_weight_GBps": round(read / decode / 1e9, 1),
+            "dense_fp4_prefill_tok_s": round(prompt_tokens / min(dense_prefill[1:]), 1),
+            "dense_fp4_prefill_ms": round(1e3 * min(dense_prefill[1:]), 3),
+            "dense_fp4_one_row_pass_us": round(1e6 * dense_decode, 1),
+        }
+    return report
+
+
 def main():
     parser = argparse.ArgumentParser()
     parser.add_argument("--gpus", type=int, default=1)
@@ -301,6 +389,11 @@ def main():
                         help="prompt length of the prefill leg (0 skips it; the "
                              "default is the context of the headline metric, for "
                              "which the reference publishes its time to first token)")
+    parser.add_argument("--mixed", action="store_true",
+                        help="measure the mixed-layer decoder (prefill and decode at "
+                             "two sizes, beside the dense decoder) instead of the "
+                             "verify step")
+    parser.add_argument("--mixed-prompt-tokens", type=int, default=4096)
     parser.add_argument("--calibration-copy", action="store_true",
                         help="also run one 256 MiB device copy (a kernel of known "
                              "traffic to scale hardware counters by)")
@@ -321,6 +414,19 @@ def main():
         return 1
     rows = MODEL["draft_depth"] + 1
     steps, warmup = arguments.steps, arguments.warmup
+    if arguments.mixed:
+        report = measure_mixed(qp, np, arguments.mixed_prompt_tokens, steps, warmup)
+        first = report["width-2048"]
+        print(json.dumps({
+            "metric": "mixed-layer decoder decode tok/s", "value": first["decode_tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
+            "ms_per_step": round(first["decode_us_per_token"] / 1e3, 4),
+            "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+            "dtype": "bf16", "data": "synthetic", "sizes": report,
+            "config": {"model": "Zatupel-shaped, 4 layers, random weights",
+                       "global_batch": 1, "seq_len": arguments.mixed_prompt_tokens,
+                       "parallelism": "none"}}))
+        return 0
     geometry = dict(MODEL)
     geometry["layers"] = arguments.layers
     # room for every step to advance by up to 5 positions

@@ -32,6 +32,7 @@ constexpr uint32_t kMaximumScoreSplits = 64;
 constexpr uint32_t kMaximumValueSplits = 16;
 constexpr uint32_t kSplitRows = 4;        // rows of the split form
 constexpr uint32_t kPromptHeads = 32;
+constexpr uint32_t kMaximumLds = 160u * 1024u;
 
 using Attention = qllm_windowed_attention;
 
@@ -1072,9 +1073,18 @@ extern "C" int32_t qllm_windowed_attention_rows(const qllm_windowed_attention* a
   AttentionArgs args{a, *launch, nullptr, nullptr, nullptr, 0u, 0u, 0u};
   const uint32_t form = qllm_windowed_attention_form(attention, launch->rows);
   if (form == QLLM_ATTENTION_GENERAL) {
-    if (general_bytes(a) > 65536u)
+    if (general_bytes(a) > kMaximumLds)
       return fail(QLLM_INVALID_ARGUMENT,
                   "windowed attention: heads and dimensions exceed the general kernel");
+    if (general_bytes(a) > 65536u) {
+      const void* kernel = a.element == QLLM_ELEMENT_F32
+                               ? reinterpret_cast<const void*>(general_attention_kernel<float>)
+                               : reinterpret_cast<const void*>(
+                                     general_attention_kernel<uint16_t>);
+      const auto raised = hipFuncSetAttribute(
+          kernel, hipFuncAttributeMaxDynamicSharedMemorySize, kMaximumLds);
+      if (raised != hipSuccess) return checked(raised, "windowed attention LDS");
+    }
     if (a.element == QLLM_ELEMENT_F32)
       general_attention_kernel<float>
           <<<launch->rows, 256, general_bytes(a), hip_stream>>>(args);

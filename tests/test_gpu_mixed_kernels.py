@@ -329,6 +329,7 @@ SHAPES = [
     (6, 6, 160, 72, 48, 3, 20, 64),
     (36, 12, 40, 40, 45, 8, 40, 64),
     (40, 2, 32, 32, 45, 7, 20, 64),
+    (64, 8, 128, 120, 35, 3, 64, 64),
 ]
 
 
