@@ -37,7 +37,8 @@ class DecoderProvider : public er::IOperationProvider {
             0U};
   }
   // Rows of the next batch whose logits the program's logits output shall hold
-  // (ascending); without a call the output holds the last row's.
+  // (ascending); without a call none are copied (the output is a
+  // placeholder).
   [[nodiscard]] virtual er::Status set_logit_rows(
       const std::shared_ptr<er::IOperationProviderRequestState>&,
       std::vector<std::uint32_t>) {

@@ -643,7 +643,6 @@ er::Status Mi355MixedProvider::set_logit_rows(
   if (!state || !std::is_sorted(rows.begin(), rows.end()))
     return {er::ErrorCode::invalid_argument, "logit rows are invalid"};
   state->logit_rows = std::move(rows);
-  state->logit_rows_set = true;
   return er::Status::success();
 }
 
@@ -933,10 +932,8 @@ Mi355MixedProvider::HeadResult Mi355MixedProvider::finish_batch(
   const std::uint32_t stride = round_up(g_.vocabulary, 4U);
   HeadResult result;
   result.logits = std::make_shared<std::vector<float>>();
-  if (!state.logit_rows_set) state.logit_rows.assign(1U, rows - 1U);
   const auto wanted = std::move(state.logit_rows);
   state.logit_rows.clear();
-  state.logit_rows_set = false;
   result.logits->resize(std::max<std::size_t>(wanted.size() * g_.vocabulary, 1U));
   const auto copy_rows = [&](std::size_t first, std::size_t count) {
     if (!count) return;

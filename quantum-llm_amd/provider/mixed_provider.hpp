@@ -64,7 +64,6 @@ class MixedRequestState final : public er::IOperationProviderRequestState {
   std::shared_ptr<std::atomic<bool>> lease;
   std::uint32_t position{};                 // of the next token
   std::vector<std::uint32_t> logit_rows;    // asked for in the next batch
-  bool logit_rows_set{};
 };
 
 class Mi355MixedProvider final : public DecoderProvider {
