@@ -721,11 +721,10 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
   constexpr int kMixHeads = kFolded ? 16 : 32;
   constexpr int kPairs = (HPW + 1) / 2;
   // normalised weights [key][query row][64 bytes of heads]
-  __shared__ __attribute__((aligned(16))) uint8_t high[512 * 64];
-  __shared__ __attribute__((aligned(16))) uint8_t low_plane[kFolded ? 16 : 512 * 64];
+  __shared__ __attribute__((aligned(16))) uint8_t high[2][512 * 64];
+  __shared__ __attribute__((aligned(16))) uint8_t low[kFolded ? 1 : 2][kFolded ? 16 : 512 * 64];
   // mixed weights [output head][query row][key]
-  __shared__ __attribute__((aligned(16))) uint8_t mixed[16 * 16 * 64];
-  uint8_t* const low = kFolded ? high : low_plane;
+  __shared__ __attribute__((aligned(16))) uint8_t mixed[2][16 * 16 * 64];
   constexpr uint32_t kLowSlot = kFolded ? 2u : 0u;
   const Attention& a = args.attention;
   const auto& run = args.launch;
@@ -747,7 +746,7 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
 
   for (uint32_t i = threadIdx.x; i < sizeof(high) / 16u; i += blockDim.x) {
     reinterpret_cast<i32x4*>(high)[i] = i32x4{};
-    if (!kFolded) reinterpret_cast<i32x4*>(low_plane)[i] = i32x4{};
+    if (!kFolded) reinterpret_cast<i32x4*>(low)[i] = i32x4{};
   }
 
   uint32_t kv[HPW], value_kv[OPW];
@@ -790,21 +789,13 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
   f32x4 out[OPW][NV] = {};
   i32x4 k[2][NK];
   fetch_tile_keys<NK>(k, a, pages, range.tile(0u), kv[0]);
-  const auto values_at = [&](uint32_t tile, uint32_t kv_head) __attribute__((always_inline)) {
-    const uint32_t key0 = tile * kTileKeys;
-    return reinterpret_cast<const i32x4*>(page_of<const uint16_t>(a, pages, key0) +
-                                          value_block(a, kv_head, key0 % a.page_tokens)) +
-           column * 4u + quarter;
-  };
-  for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal) {
+
+  // weights of a tile into its buffer; the keys of the next one on their way
+  const auto weigh = [&](uint32_t ordinal) __attribute__((always_inline)) {
     const uint32_t tile = range.tile(ordinal);
     const bool all = tile_open(a, first, tile);
-    i32x4 v[NV];
-    {
-      const i32x4* values = values_at(tile, value_kv[0]);
-#pragma unroll
-      for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
-    }
+    uint8_t* const upper_plane = high[ordinal & 1u];
+    uint8_t* const lower_plane = kFolded ? upper_plane : low[kFolded ? 0u : ordinal & 1u];
 #pragma unroll
     for (int pair = 0; pair < kPairs; ++pair) {
       f32x4 s[2][2];
@@ -841,8 +832,8 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
           const uint32_t row = (e / 4 * 16u + 4u * quarter + e % 4) * 16u + column;
           uint32_t upper, lower;
           split_pair(s[0][e / 4][e % 4], second ? s[1][e / 4][e % 4] : 0.0f, upper, lower);
-          uint8_t* const upper_at = high + swizzled(row, g / 8u) + g % 8u * 2u;
-          uint8_t* const lower_at = low + swizzled(row, kLowSlot + g / 8u) + g % 8u * 2u;
+          uint8_t* const upper_at = upper_plane + swizzled(row, g / 8u) + g % 8u * 2u;
+          uint8_t* const lower_at = lower_plane + swizzled(row, kLowSlot + g / 8u) + g % 8u * 2u;
           if constexpr (HPW == 1) {
             *reinterpret_cast<uint16_t*>(upper_at) = static_cast<uint16_t>(upper);
             *reinterpret_cast<uint16_t*>(lower_at) = static_cast<uint16_t>(lower);
@@ -853,38 +844,76 @@ __global__ __launch_bounds__(512, 2) void prompt_attention_kernel(AttentionArgs 
         }
       }
     }
-    __syncthreads();
-    // mix: four keys at a time, all query rows, this workgroup's output heads
+  };
+  // mix: four keys at a time, all query rows, this workgroup's output heads
+  const auto blend = [&](uint32_t ordinal) __attribute__((always_inline)) {
+    const uint8_t* const upper_plane = high[ordinal & 1u];
+    const uint8_t* const lower_plane = low[kFolded ? 0u : ordinal & 1u];
+    uint8_t* const target = mixed[ordinal & 1u];
     for (uint32_t four = wave; four < 8u; four += waves) {
       f32x4 m[4] = {};
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const uint32_t at = swizzled((four * 4u + j) * 16u + column, quarter);
         if constexpr (!kFolded)
-          m[j] = mfma_bf16(mix, *reinterpret_cast<const i32x4*>(low + at), m[j]);
-        m[j] = mfma_bf16(mix, *reinterpret_cast<const i32x4*>(high + at), m[j]);
+          m[j] = mfma_bf16(mix, *reinterpret_cast<const i32x4*>(lower_plane + at), m[j]);
+        m[j] = mfma_bf16(mix, *reinterpret_cast<const i32x4*>(upper_plane + at), m[j]);
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        *reinterpret_cast<i32x2*>(mixed + (4u * quarter + i) * 1024u +
+        *reinterpret_cast<i32x2*>(target + (4u * quarter + i) * 1024u +
                                   swizzled(column, four / 2u) + four % 2u * 8u) =
             i32x2{static_cast<int>(pack_bf16(m[0][i], m[1][i])),
                   static_cast<int>(pack_bf16(m[2][i], m[3][i]))};
     }
-    __syncthreads();
+  };
+  const auto values_at = [&](uint32_t tile, uint32_t kv_head) __attribute__((always_inline)) {
+    const uint32_t key0 = tile * kTileKeys;
+    return reinterpret_cast<const i32x4*>(page_of<const uint16_t>(a, pages, key0) +
+                                          value_block(a, kv_head, key0 % a.page_tokens)) +
+           column * 4u + quarter;
+  };
+
+  // Three tiles are under way between two barriers: the weights of one, the
+  // mix of the one before, the values of the one before that.
+  weigh(0u);
+  __syncthreads();
+  blend(0u);
+  if (range.count > 1u) weigh(1u);
+  __syncthreads();
+  for (uint32_t ordinal = 0; ordinal < range.count; ++ordinal) {
+    const uint32_t tile = range.tile(ordinal);
+    i32x4 v[NV];
+    const i32x4* const values = values_at(tile, value_kv[0]);
+    const auto load_values = [&]() __attribute__((always_inline)) {
+#pragma unroll
+      for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
+    };
+    // the values early, where registers hold them across the other two stages
+    if constexpr (kFolded) {
+      load_values();
+      if (ordinal + 1u < range.count) blend(ordinal + 1u);
+      if (ordinal + 2u < range.count) weigh(ordinal + 2u);
+    } else {
+      if (ordinal + 2u < range.count) weigh(ordinal + 2u);
+      __builtin_amdgcn_sched_barrier(0);
+      load_values();
+      if (ordinal + 1u < range.count) blend(ordinal + 1u);
+    }
 #pragma unroll
     for (int i = 0; i < OPW; ++i) {
       const uint32_t at = wave * OPW + i;
-      const i32x4 w = *reinterpret_cast<const i32x4*>(mixed + min(at, 15u) * 1024u +
-                                                      swizzled(column, quarter));
+      const i32x4 w = *reinterpret_cast<const i32x4*>(
+          mixed[ordinal & 1u] + min(at, 15u) * 1024u + swizzled(column, quarter));
       if (!SHARED && i > 0 && value_kv[i] != value_kv[i - 1]) {
-        const i32x4* values = values_at(tile, value_kv[i]);
+        const i32x4* const other = values_at(tile, value_kv[i]);
 #pragma unroll
-        for (int t = 0; t < NV; ++t) v[t] = values[t * kWave];
+        for (int t = 0; t < NV; ++t) v[t] = other[t * kWave];
       }
 #pragma unroll
       for (int t = 0; t < NV; ++t) out[i][t] = mfma_bf16(w, v[t], out[i][t]);
     }
+    __syncthreads();
   }
 
   float gate[OPW][4];
