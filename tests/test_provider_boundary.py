@@ -168,7 +168,9 @@ def test_bind_reports_equal_the_references():
                     reason="the reference tree is not present")
 @pytest.mark.parametrize("source", ["dense_fp4_provider.cpp", "artifact_provider.cpp",
                                     "execution_provider.cpp", "operation_handles.cpp",
-                                    "speculative_sampling.cpp"])
+                                    "speculative_sampling.cpp", "mixed_provider.cpp",
+                                    "host_support.cpp", "request_slots.cpp",
+                                    "token_selector.cpp"])
 def test_provider_sources_compile_against_the_reference_headers(source):
     """Swapping the include path: the reference's runtime/include in place of
     quantum-llm_amd/provider/include.  The provider object, the module factory
