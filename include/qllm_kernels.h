@@ -869,8 +869,8 @@ int32_t qllm_mark_presence(uint8_t* emitted, const uint32_t* tokens,
 /* ---- mixed-layer decoders -------------------------------------------------------
  *
  * Kernels of decoders whose layers differ: windowed attention with mixed heads
- * beside recurrent layers, bf16 weights, a parallel mixer and feed-forward on
- * one residual stream.  No counterpart in the reference.  Sizes and constants
+ * or attention over a cached latent beside recurrent layers, bf16 weights, mixer
+ * and feed-forward parallel or one after the other on one residual stream.  No counterpart in the reference.  Sizes and constants
  * are parameters throughout; `element` says what activations and cached keys
  * and values are stored as (F32 mode computes every product in true 32-bit).
  * The residual stream, norms, positions and angles, scores and attention
@@ -905,6 +905,16 @@ int32_t qllm_linear_pack(const void* source_bf16, uint32_t rows,
                          uint32_t packed_columns, uint32_t first_tile,
                          uint32_t tile_stride, uint32_t first_column,
                          void* stream);
+
+/* The same for a matrix whose element (row, column) lies at row * row_stride +
+ * column * column_stride of `source_bf16`: part of a larger matrix, or one read
+ * transposed. */
+int32_t qllm_linear_pack_strided(const void* source_bf16, uint32_t rows,
+                                 uint32_t columns, uint64_t row_stride,
+                                 uint64_t column_stride, void* packed,
+                                 uint32_t packed_columns, uint32_t first_tile,
+                                 uint32_t tile_stride, uint32_t first_column,
+                                 void* stream);
 
 enum qllm_linear_epilogue {
   QLLM_LINEAR_STORE = 0,    /* output f32 [m][n] = product */
@@ -953,7 +963,11 @@ int32_t qllm_embedding_bf16_batch(const void* table_bf16, uint32_t vocabulary,
  * the row before it, each to its own buffer: norm + (before - norm) * mu[s];
  * row 0 takes `previous` of the request's slot ([slot][slot_stride] f32, all
  * zeros at the start of a sequence) and the last row's norm is left in `last`.
- * `gather`, when given, lists the input row of every output row. */
+ * `gather`, when given, lists the input row of every output row.
+ * With `branch_weight` the partial sums are a sublayer's output that passes an
+ * RMS norm of its own on its way into the stream: stream = input +
+ * branch_scale * rms_norm(sum of partials, branch_epsilon) * branch_weight (not
+ * together with `shift`). */
 typedef struct qllm_token_shift {
   uint32_t count;              /* 1 .. 6 */
   const float* mu[6];          /* f32 [width] */
@@ -979,6 +993,9 @@ typedef struct qllm_stream_norm_launch {
   const qllm_token_shift* shift;
   const uint32_t* gather;      /* device, [rows] */
   const uint32_t* step;        /* device words; needed with `shift` */
+  const float* branch_weight;  /* f32 [width] */
+  float branch_scale;
+  float branch_epsilon;
 } qllm_stream_norm_launch;
 int32_t qllm_stream_norm(const qllm_stream_norm_launch* launch, void* stream);
 
@@ -1067,17 +1084,115 @@ int32_t qllm_windowed_attention_rows(const qllm_windowed_attention* attention,
                                      const qllm_attention_launch* launch,
                                      void* stream);
 
+/* ---- latent attention ------------------------------------------------------- */
+
+/* Geometry and weights of one layer.  A token's cache row is its latent c
+ * (`rank` values, RMS-normed with latent_norm) and one key part of rot_dim
+ * values that all heads share, the first rotary_dims of them rotated: dimension
+ * i with i + rotary_dims / 2 by position * frequencies[i], cosine and sine times
+ * rotary_magnitude.  Head h has the keys [key_up[h] c | shared part], the values
+ * value_up[h] c and the scores (query . key) * scale.  Position i sees j if
+ * j <= i and, with a window, i - j < window.
+ *
+ * A page holds, from layer_offset on, [page_tokens / 16][chunks] fragments of 16
+ * tokens x 32 dimensions in the lane order of a matrix operand (token n,
+ * dimension k at ((k / 8) * 16 + n) * 8 + k % 8); latent and shared part are
+ * each padded to 32 with zeros.
+ *
+ * Packed weights (qllm_linear_pack_strided), tiles of every head one after the
+ * other: key_up, `dim` padded to 32 rows over `rank` columns; key_up_transposed,
+ * `rank` padded to 32 rows over `dim` columns; value_up, `vdim` padded to 16
+ * rows over `rank` columns. */
+typedef struct qllm_latent_attention {
+  uint32_t heads, dim, vdim, rank;
+  uint32_t rot_dim, rotary_dims;   /* 0 = no such part */
+  uint32_t window;                 /* 0 = every earlier position */
+  float scale;
+  float epsilon;                   /* of the latent's norm */
+  float rotary_magnitude;
+  const double* frequencies;       /* device [rotary_dims / 2] */
+  const float* latent_norm;        /* device f32 [rank] */
+  const void* key_up;
+  const void* key_up_transposed;
+  const void* value_up;
+  uint32_t page_tokens;            /* a multiple of 32 */
+  uint32_t pages_per_slot;
+  uint64_t layer_offset;           /* bytes */
+  void* const* page_table;         /* device [slots][pages_per_slot] */
+  const uint32_t* step;            /* device words */
+  uint32_t element;
+} qllm_latent_attention;
+
+size_t qllm_latent_layer_bytes(uint32_t page_tokens, uint32_t rank,
+                               uint32_t rot_dim, uint32_t element);
+
+/* Norms the latent rows, rotates the shared key parts and stores both into the
+ * pages.  projections: f32 rows of `stride` floats, `rank` latent values and
+ * rot_dim key values from latent_column on.  With query_rank the rows' query
+ * latents (at query_column) are normed as well and left in query_out, element
+ * [rows][query_stride], zeros from query_rank on. */
+typedef struct qllm_latent_store_launch {
+  const float* projections;
+  uint32_t stride, latent_column;
+  uint32_t query_column, query_rank;
+  const float* query_norm;     /* device f32 [query_rank] */
+  void* query_out;
+  uint32_t query_stride;
+  uint32_t rows;
+} qllm_latent_store_launch;
+int32_t qllm_latent_store(const qllm_latent_attention* attention,
+                          const qllm_latent_store_launch* launch, void* stream);
+
+/* Attention of `rows` consecutive positions over the pages (their own rows
+ * included).  query: f32 rows of query_stride floats, head h's dim + rot_dim
+ * values (unrotated, then to be rotated) at h * (dim + rot_dim).  Output element
+ * [rows][output_stride], head h's values at h * vdim, multiplied by
+ * sigmoid(gate) element by element when `gate` (f32 rows of gate_stride floats)
+ * is given.
+ *   SPLIT: queries taken into the latent space, scores and sums over cached
+ *          latents, the context dealt over workgroups, sums taken back to the
+ *          value space.  Few rows.
+ *   PROMPT: keys and values of the visible context expanded once, then ordinary
+ *          attention per head.  Row r is position maximum_position - rows + 1 + r.
+ *   GENERAL: a workgroup per row and head; any size, bf16 or F32. */
+typedef struct qllm_latent_launch {
+  const float* query;
+  uint32_t query_stride;
+  const float* gate;
+  uint32_t gate_stride;
+  void* output;
+  uint32_t output_stride;
+  uint32_t rows;
+  uint32_t maximum_position;   /* no row's position exceeds it */
+  void* workspace;
+  size_t workspace_bytes;
+} qllm_latent_launch;
+uint32_t qllm_latent_attention_form(const qllm_latent_attention* attention,
+                                    uint32_t rows);   /* enum qllm_attention_form */
+size_t qllm_latent_attention_workspace_bytes(const qllm_latent_attention* attention,
+                                             uint32_t rows,
+                                             uint32_t maximum_position);
+int32_t qllm_latent_attention_rows(const qllm_latent_attention* attention,
+                                   const qllm_latent_launch* launch, void* stream);
+
 /* ---- recurrent layers ------------------------------------------------------ */
 
-/* A per-head matrix state [dim (key)][dim (value)], F32, carried from token to
- * token.  r, k, v: rows of a token's projections.
+/* A per-head matrix state [dim (key)][vdim (value)], F32, carried from token to
+ * token.  DELTA and BONUS have vdim = dim.  r, k, v: rows of a token's projections.
  *   DELTA: u = k / sqrt(sum k^2 + unit_epsilon), a = sigmoid(rate + bias),
  *          w = exp(decay_scale * sigmoid(inner)), decay_scale < 0:
  *          S <- diag(w) S - (a u) (u^T S) + k v^T;  o = S^T r
  *   BONUS: w = exp(-exp(inner)):
  *          o = (S + diag(bonus) k v^T)^T r;  S <- diag(w) S + k v^T
- * inner = W2 tanh(low) + base, with low the rank-sized projection. */
-enum qllm_recurrence_kind { QLLM_RECURRENCE_DELTA = 0, QLLM_RECURRENCE_BONUS = 1 };
+ *   GATED: w = sigmoid(inner)^decay_scale:
+ *          S <- diag(w) S + k v^T;  o = S^T (read_scale r)
+ * inner = W2 tanh(low) + base (GATED: W2 low + base), with low the rank-sized
+ * projection. */
+enum qllm_recurrence_kind {
+  QLLM_RECURRENCE_DELTA = 0,
+  QLLM_RECURRENCE_BONUS = 1,
+  QLLM_RECURRENCE_GATED = 2
+};
 enum qllm_gate_kind { QLLM_GATE_SIGMOID = 0, QLLM_GATE_SILU = 1 };
 
 typedef struct qllm_recurrence {
@@ -1092,11 +1207,13 @@ typedef struct qllm_recurrence {
   const float* decay_base;     /* [heads * dim] */
   const float* rate_bias;      /* DELTA: [heads * dim] */
   const float* bonus;          /* BONUS: [heads * dim] */
-  const float* norm_weight;    /* [heads * dim] */
-  float* state;                /* [slot][heads][dim][dim], of slot 0 */
+  const float* norm_weight;    /* [heads * dim]; GATED: [vdim], for every head */
+  float* state;                /* [slot][heads][dim][vdim], of slot 0 */
   uint64_t slot_stride;        /* floats between slots */
   const uint32_t* step;        /* device words */
   uint32_t element;
+  uint32_t vdim;               /* 0 = dim; GATED may differ (vdim <= 1024) */
+  float read_scale;            /* GATED */
 } qllm_recurrence;
 
 /* `rows` tokens: output element [rows][output_stride] = o / rms(o) * norm *

@@ -384,6 +384,7 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(LinearArgs args) {
 }
 
 __global__ void linear_pack_kernel(const uint16_t* source, uint32_t rows, uint32_t columns,
+                                   uint64_t row_stride, uint64_t column_stride,
                                    uint16_t* packed, uint32_t packed_chunks,
                                    uint32_t first_tile, uint32_t tile_stride,
                                    uint32_t first_chunk, uint32_t chunks,
@@ -398,7 +399,7 @@ __global__ void linear_pack_kernel(const uint16_t* source, uint32_t rows, uint32
     const uint32_t row = tile * 16u + lane % 16u;
     const uint32_t column = chunk * 32u + lane / 16u * 8u + in_fragment % 8u;
     const uint16_t value = row < rows && column < columns
-                               ? source[uint64_t{row} * columns + column]
+                               ? source[row * row_stride + column * column_stride]
                                : uint16_t{0};
     packed[(uint64_t{first_tile + tile * tile_stride} * packed_chunks + first_chunk +
             chunk) * 512u + in_fragment] = value;
@@ -444,6 +445,17 @@ extern "C" int32_t qllm_linear_pack(const void* source_bf16, uint32_t rows, uint
                                     void* packed, uint32_t packed_columns,
                                     uint32_t first_tile, uint32_t tile_stride,
                                     uint32_t first_column, void* stream) {
+  return qllm_linear_pack_strided(source_bf16, rows, columns, columns, 1u, packed,
+                                  packed_columns, first_tile, tile_stride, first_column,
+                                  stream);
+}
+
+extern "C" int32_t qllm_linear_pack_strided(const void* source_bf16, uint32_t rows,
+                                            uint32_t columns, uint64_t row_stride,
+                                            uint64_t column_stride, void* packed,
+                                            uint32_t packed_columns, uint32_t first_tile,
+                                            uint32_t tile_stride, uint32_t first_column,
+                                            void* stream) {
   const uint32_t padded = (columns + 63u) / 64u * 64u;
   if (!source_bf16 || !packed || !rows || !columns || !tile_stride ||
       packed_columns % 64u || first_column % 64u || !aligned16(packed) ||
@@ -454,7 +466,7 @@ extern "C" int32_t qllm_linear_pack(const void* source_bf16, uint32_t rows, uint
   const uint32_t blocks =
       static_cast<uint32_t>(elements / 256u < 65536u ? (elements + 255u) / 256u : 65536u);
   linear_pack_kernel<<<blocks, 256, 0, as_stream(stream)>>>(
-      static_cast<const uint16_t*>(source_bf16), rows, columns,
+      static_cast<const uint16_t*>(source_bf16), rows, columns, row_stride, column_stride,
       static_cast<uint16_t*>(packed), packed_columns / 32u, first_tile, tile_stride,
       first_column / 32u, chunks, elements);
   return launched("linear pack");

@@ -16,9 +16,12 @@ struct NormArgs {
   qllm_token_shift shift;
 };
 
+// The stream with the partial sums added; with a branch norm the sums alone.
 __device__ __forceinline__ f32x4 stream_value4(const qllm_stream_norm_launch& l,
                                                uint32_t row, uint32_t piece) {
-  f32x4 value = reinterpret_cast<const f32x4*>(l.input + size_t{row} * l.width)[piece];
+  f32x4 value = l.branch_weight
+                    ? f32x4{}
+                    : reinterpret_cast<const f32x4*>(l.input + size_t{row} * l.width)[piece];
   // eight loads in flight at a time
   for (uint32_t first = 0; first < l.partial_count; first += 8u) {
     f32x4 part[8];
@@ -37,7 +40,7 @@ __device__ __forceinline__ f32x4 stream_value4(const qllm_stream_norm_launch& l,
 
 __device__ __forceinline__ float stream_value(const qllm_stream_norm_launch& l,
                                               uint32_t row, uint32_t column) {
-  float value = l.input[size_t{row} * l.width + column];
+  float value = l.branch_weight ? 0.0f : l.input[size_t{row} * l.width + column];
   for (uint32_t p = 0; p < l.partial_count; ++p)
     value += l.partials[(size_t{p} * l.rows + row) * l.partial_stride + column];
   return value;
@@ -82,10 +85,32 @@ __global__ __launch_bounds__(1024) void stream_norm_wide_kernel(NormArgs args) {
     held[i] = f32x4{};
     if (piece >= pieces) continue;
     held[i] = stream_value4(l, source, piece);
-    if (l.partial_count)
+    if (l.partial_count && !l.branch_weight)
       reinterpret_cast<f32x4*>(l.stream_out + size_t{row} * l.width)[piece] = held[i];
 #pragma unroll
     for (int c = 0; c < 4; ++c) squares = fmaf(held[i][c], held[i][c], squares);
+  }
+  if (l.branch_weight) {
+    f32x4 before[kHeld], weight[kHeld];
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i) {
+      const uint32_t piece = threadIdx.x + i * blockDim.x;
+      if (piece >= pieces) continue;
+      before[i] = reinterpret_cast<const f32x4*>(l.input + size_t{row} * l.width)[piece];
+      weight[i] = reinterpret_cast<const f32x4*>(l.branch_weight)[piece];
+    }
+    const float unit =
+        inverse_rms(block_sum(squares, scratch), l.width, l.branch_epsilon);
+    squares = 0.0f;
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i) {
+      const uint32_t piece = threadIdx.x + i * blockDim.x;
+      if (piece >= pieces) continue;
+      held[i] = before[i] + held[i] * unit * weight[i] * l.branch_scale;
+      reinterpret_cast<f32x4*>(l.stream_out + size_t{row} * l.width)[piece] = held[i];
+#pragma unroll
+      for (int c = 0; c < 4; ++c) squares = fmaf(held[i][c], held[i][c], squares);
+    }
   }
   const float inverse = inverse_rms(block_sum(squares, scratch), l.width, l.epsilon);
   const bool shifted = l.shift != nullptr;
@@ -153,8 +178,24 @@ __global__ __launch_bounds__(256) void stream_norm_narrow_kernel(NormArgs args) 
                            : nullptr;
   float squares = 0.0f;
   float before_squares = 0.0f;
-  for (uint32_t c = threadIdx.x; c < l.width; c += blockDim.x) {
+  float unit_branch = 0.0f;
+  if (l.branch_weight) {
+    float branch_squares = 0.0f;
+    for (uint32_t c = threadIdx.x; c < l.width; c += blockDim.x) {
+      const float value = stream_value(l, source, c);
+      branch_squares = fmaf(value, value, branch_squares);
+    }
+    unit_branch = inverse_rms(block_sum(branch_squares, scratch), l.width, l.branch_epsilon) *
+                  l.branch_scale;
+  }
+  const auto here_value = [&](uint32_t c) {
     const float value = stream_value(l, source, c);
+    return l.branch_weight ? l.input[size_t{row} * l.width + c] +
+                                 value * unit_branch * l.branch_weight[c]
+                           : value;
+  };
+  for (uint32_t c = threadIdx.x; c < l.width; c += blockDim.x) {
+    const float value = here_value(c);
     if (l.partial_count) l.stream_out[size_t{row} * l.width + c] = value;
     squares = fmaf(value, value, squares);
     if (shifted && !carried) {
@@ -166,7 +207,7 @@ __global__ __launch_bounds__(256) void stream_norm_narrow_kernel(NormArgs args) 
   const float before_inverse =
       inverse_rms(block_sum(before_squares, scratch), l.width, l.epsilon);
   for (uint32_t c = threadIdx.x; c < l.width; c += blockDim.x) {
-    const float unit = stream_value(l, source, c) * inverse;
+    const float unit = here_value(c) * inverse;
     for (int output = 0; output < 2; ++output)
       if (l.weight[output] && !(shifted && output == 0))
         store_element(static_cast<T*>(l.output[output]) +
@@ -226,11 +267,12 @@ extern "C" int32_t qllm_stream_norm(const qllm_stream_norm_launch* launch, void*
       launch->element > QLLM_ELEMENT_F32 ||
       (launch->partial_count &&
        (!launch->partials || !launch->stream_out || launch->stream_out == launch->input ||
-        launch->partial_stride < launch->width || launch->gather)))
+        launch->partial_stride < launch->width || launch->gather)) ||
+      (launch->branch_weight && (!launch->partial_count || launch->shift)))
     return fail(QLLM_INVALID_ARGUMENT, "invalid stream norm");
   bool wide = launch->width % 4u == 0u && launch->partial_stride % 4u == 0u &&
               aligned16(launch->input) && aligned16(launch->stream_out) &&
-              aligned16(launch->partials);
+              aligned16(launch->partials) && aligned16(launch->branch_weight);
   for (int i = 0; i < 2; ++i) {
     if (!launch->weight[i]) continue;
     const bool blended = i == 0 && launch->shift;

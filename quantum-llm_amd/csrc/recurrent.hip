@@ -1,5 +1,6 @@
-// Recurrent mixers with a matrix state per head: the generalised delta rule and
-// the bonus recurrence (include/qllm_kernels.h has the equations).  State,
+// Recurrent mixers with a matrix state per head: the generalised delta rule, the
+// bonus recurrence and gated linear attention (include/qllm_kernels.h has the
+// equations).  State,
 // decays, unit keys and rates are F32.
 //
 // The columns of a state (its value dimension) never meet: column j is a
@@ -23,7 +24,7 @@ struct RecurrenceArgs {
   qllm_recurrence_launch launch;
   float* prepared;   // [head][row][slots][padded dim]
   float* scalars;    // BONUS: [head][row] sum of r * bonus * k
-  float* outputs;    // [row][heads * dim]
+  float* outputs;    // [row][heads * vdim]
   uint32_t padded;   // dim padded to 16, 32, 64, 128 or 256
 };
 
@@ -42,8 +43,15 @@ __device__ __forceinline__ float gate_value(uint32_t kind, float x) {
 }
 
 __device__ __forceinline__ float decay_of(const qllm_recurrence& l, float inner) {
-  return l.kind == QLLM_RECURRENCE_DELTA ? expf(l.decay_scale * sigmoid_f32(inner))
-                                         : expf(-expf(inner));
+  if (l.kind == QLLM_RECURRENCE_DELTA) return expf(l.decay_scale * sigmoid_f32(inner));
+  if (l.kind == QLLM_RECURRENCE_BONUS) return expf(-expf(inner));
+  // a power of the sigmoid, through its logarithm
+  return expf(l.decay_scale * (fminf(inner, 0.0f) - log1pf(expf(-fabsf(inner)))));
+}
+
+// What the decay's low-rank product takes of its projection.
+__device__ __forceinline__ float low_value(const qllm_recurrence& l, float x) {
+  return l.kind == QLLM_RECURRENCE_GATED ? x : tanhf(x);
 }
 
 __device__ __forceinline__ void copy_carry(const RecurrenceArgs& args) {
@@ -184,6 +192,90 @@ __global__ __launch_bounds__(1024) void recurrence_step_kernel(RecurrenceArgs ar
   copy_carry(args);
 }
 
+// The same for gated linear attention, whose state may have more columns than
+// rows: a row group of threads per `vdim` columns, rows dealt in turn.  KPT = 0
+// streams the state instead of holding it.
+template <typename T, int KPT>
+__global__ __launch_bounds__(1024) void gated_step_kernel(RecurrenceArgs args) {
+  __shared__ float r[256], k[256], w[256], low[256];
+  __shared__ float part[1024];
+  __shared__ float scratch[16];
+  const qllm_recurrence& l = args.layer;
+  const auto& run = args.launch;
+  const uint32_t head = blockIdx.x;
+  const uint32_t dim = l.dim;
+  const uint32_t vdim = l.vdim;
+  const float* p = run.projections;
+  const uint32_t groups = 1024u / vdim;
+  const uint32_t group = threadIdx.x / vdim;
+  const uint32_t column = threadIdx.x - group * vdim;
+  const bool active = group < groups;
+  float* state = l.state + l.step[kStepSlot] * l.slot_stride + size_t{head} * dim * vdim +
+                 column;
+  constexpr int kHeld = KPT ? KPT : 1;
+  float s[kHeld];
+#pragma unroll
+  for (int i = 0; i < KPT; ++i) {
+    const uint32_t row = group + groups * i;
+    s[i] = active && row < dim ? state[size_t{row} * vdim] : 0.0f;
+  }
+  const float value = active ? p[run.v_column + head * vdim + column] : 0.0f;
+  const bool owner = threadIdx.x < vdim;
+  const float gate = owner ? p[run.gate_column + head * vdim + threadIdx.x] : 0.0f;
+  const float weight = owner ? l.norm_weight[threadIdx.x] : 0.0f;
+  for (uint32_t j = threadIdx.x; j < l.rank; j += blockDim.x)
+    low[j] = low_value(l, p[run.low_column + j]);
+  if (threadIdx.x < dim) {
+    r[threadIdx.x] = p[run.r_column + head * dim + threadIdx.x] * l.read_scale;
+    k[threadIdx.x] = p[run.k_column + head * dim + threadIdx.x];
+  }
+  __syncthreads();
+  // the low-rank products: 1024 / 256 = 4 threads per channel
+  const uint32_t channel = threadIdx.x / 4u;
+  float inner = 0.0f;
+  if (channel < dim) {
+    const uint16_t* up = static_cast<const uint16_t*>(l.decay_up_bf16) +
+                         (size_t{head} * dim + channel) * l.rank;
+#pragma unroll 8
+    for (uint32_t j = threadIdx.x % 4u; j < l.rank; j += 4u)
+      inner = fmaf(bf16_bits_to_f32(up[j]), low[j], inner);
+  }
+  inner += __shfl_xor(inner, 1, kWave);
+  inner += __shfl_xor(inner, 2, kWave);
+  if (channel < dim && threadIdx.x % 4u == 0u)
+    w[channel] = decay_of(l, inner + l.decay_base[head * dim + channel]);
+  __syncthreads();
+  float read = 0.0f;
+  if constexpr (KPT) {
+#pragma unroll
+    for (int i = 0; i < KPT; ++i) {
+      const uint32_t row = group + groups * i;
+      if (!active || row >= dim) continue;
+      s[i] = fmaf(k[row], value, w[row] * s[i]);
+      read = fmaf(r[row], s[i], read);
+      state[size_t{row} * vdim] = s[i];
+    }
+  } else if (active) {
+#pragma unroll 8
+    for (uint32_t row = group; row < dim; row += groups) {
+      const float fresh = fmaf(k[row], value, w[row] * state[size_t{row} * vdim]);
+      read = fmaf(r[row], fresh, read);
+      state[size_t{row} * vdim] = fresh;
+    }
+  }
+  part[threadIdx.x] = read;
+  __syncthreads();
+  float out = 0.0f;
+  if (owner)
+    for (uint32_t g = 0; g < groups; ++g) out += part[g * vdim + threadIdx.x];
+  const float squares = block_sum(owner ? out * out : 0.0f, scratch);
+  if (owner)
+    store_element(static_cast<T*>(run.output) + head * vdim + threadIdx.x,
+                  out / sqrtf(squares / static_cast<float>(vdim) + l.epsilon) * weight *
+                      gate_value(l.gate_kind, gate));
+  copy_carry(args);
+}
+
 // ---- prompts ---------------------------------------------------------------------
 
 constexpr uint32_t kRowsPerThread = 8;    // tokens a thread prepares
@@ -208,6 +300,7 @@ __global__ __launch_bounds__(256) void recurrence_prepare_kernel(RecurrenceArgs 
   const uint32_t row0 = blockIdx.x * block_rows;
   const uint32_t rows = min(block_rows, run.rows - row0);
   const bool delta = l.kind == QLLM_RECURRENCE_DELTA;
+  const bool gated = l.kind == QLLM_RECURRENCE_GATED;
   const float* block_projections = run.projections + size_t{row0} * run.stride;
   const uint32_t c = threadIdx.x % padded;
   const uint32_t group = threadIdx.x / padded;
@@ -221,11 +314,11 @@ __global__ __launch_bounds__(256) void recurrence_prepare_kernel(RecurrenceArgs 
     const float* p = block_projections +
                      size_t{min(group * kRowsPerThread + i, rows - 1u)} * run.stride + channel;
     key[i] = p[run.k_column];
-    read[i] = p[run.r_column];
+    read[i] = gated ? p[run.r_column] * l.read_scale : p[run.r_column];
     rate[i] = delta ? p[run.rate_column] : 0.0f;
   }
   // per token: sum of k^2, or of r * bonus * k
-  const float bonus = delta || !real ? 0.0f : l.bonus[channel];
+  const float bonus = delta || gated || !real ? 0.0f : l.bonus[channel];
 #pragma unroll
   for (uint32_t i = 0; i < kRowsPerThread; ++i) {
     key[i] = real ? key[i] : 0.0f;
@@ -254,8 +347,8 @@ __global__ __launch_bounds__(256) void recurrence_prepare_kernel(RecurrenceArgs 
       const uint32_t row = i / kRankChunk;
       const uint32_t j = i % kRankChunk;
       const float value =
-          tanhf(block_projections[size_t{min(row, rows - 1u)} * run.stride +
-                                  run.low_column + min(j0 + j, l.rank - 1u)]);
+          low_value(l, block_projections[size_t{min(row, rows - 1u)} * run.stride +
+                                         run.low_column + min(j0 + j, l.rank - 1u)]);
       low_tile[row][j] = j0 + j < l.rank ? value : 0.0f;
     }
     __syncthreads();
@@ -298,10 +391,12 @@ __global__ __launch_bounds__(256) void recurrence_prepare_kernel(RecurrenceArgs 
 }
 
 // Four waves, sixteen columns of one head; tokens in chunks of 1024 / padded.
-template <bool DELTA, int KPL>
+template <uint32_t KIND, int KPL>
 __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs args) {
+  constexpr bool DELTA = KIND == QLLM_RECURRENCE_DELTA;
+  constexpr bool BONUS = KIND == QLLM_RECURRENCE_BONUS;
   constexpr uint32_t kPadded = KPL * 16u;
-  constexpr uint32_t kVectors = DELTA ? 5u : 3u;
+  constexpr uint32_t kVectors = vectors_of(KIND);
   constexpr uint32_t kTokens = 1024u / kPadded;
   constexpr uint32_t kChunk = 1024u * kVectors;        // floats
   __shared__ f32x4 chunk[2][kChunk / 4u];
@@ -311,16 +406,17 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
   const auto& run = args.launch;
   const uint32_t head = blockIdx.y;
   const uint32_t dim = l.dim;
+  const uint32_t vdim = l.vdim;
   const uint32_t part = threadIdx.x % 16u;             // rows part * KPL ..
   const uint32_t column = blockIdx.x * 16u + threadIdx.x / 16u;
-  const bool real = column < dim;
+  const bool real = column < vdim;
 
-  float* state = l.state + l.step[kStepSlot] * l.slot_stride + size_t{head} * dim * dim;
+  float* state = l.state + l.step[kStepSlot] * l.slot_stride + size_t{head} * dim * vdim;
   float s[KPL];
 #pragma unroll
   for (int i = 0; i < KPL; ++i) {
     const uint32_t row = part * KPL + i;
-    s[i] = real && row < dim ? state[size_t{row} * dim + column] : 0.0f;
+    s[i] = real && row < dim ? state[size_t{row} * vdim + column] : 0.0f;
   }
 
   const f32x4* source = reinterpret_cast<const f32x4*>(
@@ -340,11 +436,11 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
     for (uint32_t i = 0; i < kValueLoads; ++i) {
       const uint32_t index = i * 256u + threadIdx.x;
       const uint32_t row = min(which * kTokens + index / 16u, run.rows - 1u);
-      const uint32_t c = min(blockIdx.x * 16u + index % 16u, dim - 1u);
+      const uint32_t c = min(blockIdx.x * 16u + index % 16u, vdim - 1u);
       next_values[i] =
-          run.projections[size_t{row} * run.stride + run.v_column + head * dim + c];
+          run.projections[size_t{row} * run.stride + run.v_column + head * vdim + c];
     }
-    if (!DELTA)
+    if (BONUS)
       next_bonus = args.scalars[size_t{head} * run.rows +
                                 min(which * kTokens + threadIdx.x % kTokens, run.rows - 1u)];
   };
@@ -365,7 +461,7 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
       const uint32_t index = i * 256u + threadIdx.x;
       if (index < kTokens * 16u) values[slot][index / 16u][index % 16u] = next_values[i];
     }
-    if (!DELTA && threadIdx.x < kTokens) bonus[slot][threadIdx.x] = next_bonus;
+    if (BONUS && threadIdx.x < kTokens) bonus[slot][threadIdx.x] = next_bonus;
   };
 
   // What a token brings to this lane, read from LDS one token ahead of its use.
@@ -412,11 +508,15 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
 #pragma unroll
       for (int i = 0; i < KPL; ++i) s[i] = fmaf(-au[i], dot, s[i]);
       return dot_with(r);
-    } else {
+    } else if constexpr (BONUS) {
       const float out = dot_with(r);
 #pragma unroll
       for (int i = 0; i < KPL; ++i) s[i] = fmaf(k[i], token.value, w[i] * s[i]);
       return out;
+    } else {
+#pragma unroll
+      for (int i = 0; i < KPL; ++i) s[i] = fmaf(k[i], token.value, w[i] * s[i]);
+      return dot_with(r);
     }
   };
 
@@ -440,11 +540,11 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
       }
       float out = row16_transposed_sum(parts);
       const uint32_t mine = first + part;
-      if (!DELTA && part < kBlock)
+      if (BONUS && part < kBlock)
         out = fmaf(bonus[slot][mine], values[slot][mine][threadIdx.x / 16u], out);
       const uint32_t row = which * kTokens + mine;
       if (real && part < kBlock && row < run.rows)
-        args.outputs[size_t{row} * l.heads * dim + head * dim + column] = out;
+        args.outputs[size_t{row} * l.heads * vdim + head * vdim + column] = out;
     }
     publish(1u - slot, which + 1u);
     __syncthreads();
@@ -452,7 +552,7 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
 #pragma unroll
   for (int i = 0; i < KPL; ++i) {
     const uint32_t row = part * KPL + i;
-    if (real && row < dim) state[size_t{row} * dim + column] = s[i];
+    if (real && row < dim) state[size_t{row} * vdim + column] = s[i];
   }
   copy_carry(args);
 }
@@ -465,44 +565,65 @@ __global__ __launch_bounds__(256) void recurrence_finish_kernel(RecurrenceArgs a
   const uint32_t item = blockIdx.x * 4u + threadIdx.x / kWave;
   if (item >= run.rows * l.heads) return;
   const uint32_t row = item / l.heads;
-  const uint32_t first = item % l.heads * l.dim;
+  const uint32_t vdim = l.vdim;
+  const uint32_t first = item % l.heads * vdim;
   const uint32_t lane = threadIdx.x % kWave;
-  const float* o = args.outputs + size_t{row} * l.heads * l.dim + first;
-  float held[4];
+  const float* o = args.outputs + size_t{row} * l.heads * vdim + first;
+  const float* gates = run.projections + size_t{row} * run.stride + run.gate_column + first;
+  const float* norm = l.norm_weight + (l.kind == QLLM_RECURRENCE_GATED ? 0u : first);
+  T* out = static_cast<T*>(run.output) + size_t{row} * run.output_stride + first;
+  constexpr uint32_t kHeld = 4;
+  float held[kHeld];
   float squares = 0.0f;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (uint32_t i = 0; i < kHeld; ++i) {
     const uint32_t c = lane + i * kWave;
-    held[i] = c < l.dim ? o[c] : 0.0f;
+    held[i] = c < vdim ? o[c] : 0.0f;
     squares = fmaf(held[i], held[i], squares);
   }
+  for (uint32_t c = lane + kHeld * kWave; c < vdim; c += kWave)
+    squares = fmaf(o[c], o[c], squares);
   squares = wave_sum(squares);
-  const float inverse = 1.0f / sqrtf(squares / static_cast<float>(l.dim) + l.epsilon);
+  const float inverse = 1.0f / sqrtf(squares / static_cast<float>(vdim) + l.epsilon);
+  const auto finish = [&](uint32_t c, float value) {
+    store_element(out + c, value * inverse * norm[c] * gate_value(l.gate_kind, gates[c]));
+  };
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const uint32_t c = lane + i * kWave;
-    if (c >= l.dim) continue;
-    const float gate = run.projections[size_t{row} * run.stride + run.gate_column + first + c];
-    store_element(static_cast<T*>(run.output) + size_t{row} * run.output_stride + first + c,
-                  held[i] * inverse * l.norm_weight[first + c] *
-                      gate_value(l.gate_kind, gate));
-  }
+  for (uint32_t i = 0; i < kHeld; ++i)
+    if (lane + i * kWave < vdim) finish(lane + i * kWave, held[i]);
+  for (uint32_t c = lane + kHeld * kWave; c < vdim; c += kWave) finish(c, o[c]);
 }
 
-template <bool DELTA>
+template <uint32_t KIND>
 void launch_scan(const RecurrenceArgs& args, hipStream_t stream) {
-  const dim3 grid((args.layer.dim + 15u) / 16u, args.layer.heads);
+  const dim3 grid((args.layer.vdim + 15u) / 16u, args.layer.heads);
   switch (args.padded) {
-    case 16u: recurrence_scan_kernel<DELTA, 1><<<grid, 256, 0, stream>>>(args); break;
-    case 32u: recurrence_scan_kernel<DELTA, 2><<<grid, 256, 0, stream>>>(args); break;
-    case 64u: recurrence_scan_kernel<DELTA, 4><<<grid, 256, 0, stream>>>(args); break;
-    case 128u: recurrence_scan_kernel<DELTA, 8><<<grid, 256, 0, stream>>>(args); break;
-    default: recurrence_scan_kernel<DELTA, 16><<<grid, 256, 0, stream>>>(args); break;
+    case 16u: recurrence_scan_kernel<KIND, 1><<<grid, 256, 0, stream>>>(args); break;
+    case 32u: recurrence_scan_kernel<KIND, 2><<<grid, 256, 0, stream>>>(args); break;
+    case 64u: recurrence_scan_kernel<KIND, 4><<<grid, 256, 0, stream>>>(args); break;
+    case 128u: recurrence_scan_kernel<KIND, 8><<<grid, 256, 0, stream>>>(args); break;
+    default: recurrence_scan_kernel<KIND, 16><<<grid, 256, 0, stream>>>(args); break;
   }
 }
 
 template <typename T>
+void launch_gated_step(const RecurrenceArgs& args, hipStream_t stream) {
+  const uint32_t groups = 1024u / args.layer.vdim;
+  const uint32_t rows = (args.layer.dim + groups - 1u) / groups;
+  if (rows <= 4u)
+    gated_step_kernel<T, 4><<<args.layer.heads, 1024, 0, stream>>>(args);
+  else if (rows <= 16u)
+    gated_step_kernel<T, 16><<<args.layer.heads, 1024, 0, stream>>>(args);
+  else
+    gated_step_kernel<T, 0><<<args.layer.heads, 1024, 0, stream>>>(args);
+}
+
+template <typename T>
 void launch_step(const RecurrenceArgs& args, hipStream_t stream) {
+  if (args.layer.kind == QLLM_RECURRENCE_GATED) {
+    launch_gated_step<T>(args, stream);
+    return;
+  }
   const uint32_t groups = 1024u / args.layer.dim;
   const uint32_t per_group = (args.layer.dim + groups - 1u) / groups;
   if (per_group <= 4u)
@@ -530,24 +651,30 @@ extern "C" size_t qllm_recurrence_workspace_bytes(const qllm_recurrence* recurre
                                                   uint32_t rows) {
   if (!recurrence || rows <= 1u) return 0u;
   return prepared_bytes(*recurrence, rows) + scalar_bytes(*recurrence, rows) +
-         size_t{rows} * recurrence->heads * recurrence->dim * 4u;
+         size_t{rows} * recurrence->heads *
+             (recurrence->vdim ? recurrence->vdim : recurrence->dim) * 4u;
 }
 
 extern "C" int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
                                         const qllm_recurrence_launch* launch,
                                         void* stream) {
   if (!recurrence || !launch) return fail(QLLM_INVALID_ARGUMENT, "invalid recurrence");
-  const qllm_recurrence& l = *recurrence;
+  qllm_recurrence l = *recurrence;
+  if (!l.vdim) l.vdim = l.dim;
   const bool delta = l.kind == QLLM_RECURRENCE_DELTA;
-  if (l.kind > QLLM_RECURRENCE_BONUS || !l.heads || !l.dim || l.dim > 256u || !l.rank ||
+  const bool gated = l.kind == QLLM_RECURRENCE_GATED;
+  if (l.kind > QLLM_RECURRENCE_GATED || l.vdim > 1024u || (!gated && l.vdim != l.dim) || !l.heads || !l.dim || l.dim > 256u || !l.rank ||
       l.rank > 256u || l.gate_kind > QLLM_GATE_SILU || l.element > QLLM_ELEMENT_F32 ||
       !l.decay_up_bf16 || !l.decay_base || !l.norm_weight || !l.state || !l.step ||
-      (delta ? !l.rate_bias : !l.bonus) || !launch->projections || !launch->output ||
-      !launch->rows || launch->output_stride < l.heads * l.dim ||
+      (delta ? !l.rate_bias : !gated && !l.bonus) || !launch->projections ||
+      !launch->output || !launch->rows || launch->output_stride < l.heads * l.vdim ||
       (launch->carry_to && (!launch->carry_from || !launch->carry_width)))
     return fail(QLLM_INVALID_ARGUMENT, "invalid recurrence");
-  for (const uint32_t column : {launch->r_column, launch->k_column, launch->v_column,
-                                launch->gate_column, delta ? launch->rate_column : 0u})
+  for (const uint32_t column : {launch->v_column, launch->gate_column})
+    if (column + l.heads * l.vdim > launch->stride)
+      return fail(QLLM_INVALID_ARGUMENT, "recurrence columns exceed the projection rows");
+  for (const uint32_t column :
+       {launch->r_column, launch->k_column, delta ? launch->rate_column : 0u})
     if (column + l.heads * l.dim > launch->stride)
       return fail(QLLM_INVALID_ARGUMENT, "recurrence columns exceed the projection rows");
   if (launch->low_column + l.rank > launch->stride)
@@ -576,9 +703,11 @@ extern "C" int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
                                    l.heads),
                               256, 0, hip_stream>>>(args);
   if (delta)
-    launch_scan<true>(args, hip_stream);
+    launch_scan<QLLM_RECURRENCE_DELTA>(args, hip_stream);
+  else if (gated)
+    launch_scan<QLLM_RECURRENCE_GATED>(args, hip_stream);
   else
-    launch_scan<false>(args, hip_stream);
+    launch_scan<QLLM_RECURRENCE_BONUS>(args, hip_stream);
   const uint32_t blocks = (launch->rows * l.heads + 3u) / 4u;
   if (f32)
     recurrence_finish_kernel<float><<<blocks, 256, 0, hip_stream>>>(args);

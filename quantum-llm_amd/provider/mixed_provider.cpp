@@ -49,6 +49,47 @@ float parameter_f32(const er::ParameterMap& parameters, std::string_view name) {
   return value;
 }
 
+double parameter_f64(const er::ParameterMap& parameters, std::string_view name) {
+  const double value = std::bit_cast<double>(parameter(parameters, name));
+  if (!(value > 0.0) || !std::isfinite(value))
+    throw std::runtime_error("operation parameter is not positive: " + std::string(name));
+  return value;
+}
+
+// Angles per position of `dims` rotated dimensions, and the factor on their cosine
+// and sine.  With a scaling, slow dimensions are stretched by `factor` and fast ones
+// stay, with a ramp between those that turn `slow` and `fast` times over the
+// original length (YaRN).
+struct Rotation final {
+  std::vector<double> frequencies;
+  double magnitude{1.0};
+};
+
+Rotation rotation_of(const er::ParameterMap& parameters, std::uint32_t dims) {
+  Rotation out;
+  const double base = parameter_f64(parameters, "rotary_base_f64_bits");
+  for (std::uint32_t i = 0; i < dims / 2U; ++i)
+    out.frequencies.push_back(std::pow(base, -2.0 * i / dims));
+  if (!parameters.contains("rotary_factor_f64_bits")) return out;
+  const double factor = parameter_f64(parameters, "rotary_factor_f64_bits");
+  const double original = parameter_f64(parameters, "rotary_original_f64_bits");
+  constexpr double kPi = 3.14159265358979323846;
+  const auto turning = [&](double turns) {
+    return dims * std::log(original / (2.0 * kPi * turns)) / (2.0 * std::log(base));
+  };
+  const double low = std::max(
+      std::floor(turning(parameter_f64(parameters, "rotary_fast_f64_bits"))), 0.0);
+  const double high = std::min(
+      std::ceil(turning(parameter_f64(parameters, "rotary_slow_f64_bits"))), dims - 1.0);
+  for (std::size_t i = 0; i < out.frequencies.size(); ++i) {
+    const double ramp = std::clamp(
+        (static_cast<double>(i) - low) / std::max(high - low, 0.001), 0.0, 1.0);
+    out.frequencies[i] *= ramp / factor + (1.0 - ramp);
+  }
+  out.magnitude = 0.1 * std::log(factor) + 1.0;
+  return out;
+}
+
 std::uint64_t elements_of(const er::ImmutableModelTensor& tensor) {
   std::uint64_t count = 1U;
   for (const auto size : tensor.shape) count *= size;
@@ -61,6 +102,13 @@ void require_matrix(const er::ImmutableModelTensor& tensor, std::uint64_t rows,
       tensor.shape[1] != columns || tensor.data_bytes != rows * columns * 2U ||
       !tensor.value.valid())
     throw std::runtime_error("weight matrix has the wrong type or shape: " + tensor.name);
+}
+
+// Enough workgroups for the chip where the rows alone are too few, each with a few
+// KiB per wave left to stream.
+std::uint32_t k_splits(std::uint32_t rows, std::uint32_t columns) {
+  const std::uint32_t tiles = rows / 16U;
+  return std::clamp(std::min((768U + tiles - 1U) / tiles, columns / 32U / 16U), 1U, 8U);
 }
 
 }  // namespace
@@ -86,12 +134,26 @@ struct Mi355MixedProvider::Block final {
   std::uint32_t mixer_columns{};   // padded
   std::uint32_t splits{1};
 
+  // sandwich: the output projection ends with the mixer's columns
+  bool sandwich{};
+  DeviceBuffer mixer_post_norm, ffn_post_norm;
+  float residual_scale{1.0F};
+  Matrix down;
+  std::uint32_t down_splits{1};
+
   // attention
   qllm_windowed_attention attention{};
   std::uint32_t rotary_dims{};
   std::uint32_t query_column{}, key_column{}, value_column{}, gate_column{};
   std::uint64_t value_blend{};
   DeviceBuffer frequencies, value_share, head_mix;
+
+  // latent attention
+  qllm_latent_attention latent{};
+  std::uint32_t latent_column{};
+  std::uint32_t query_rank{};      // 0 = queries straight from the input
+  Matrix query_up;
+  DeviceBuffer latent_norm, query_norm, key_up, key_up_transposed, value_up;
 
   // recurrence
   qllm_recurrence recurrence{};
@@ -127,6 +189,8 @@ er::WorkerProviderDefinition make_mi355_mixed_provider() {
            {kBlockWindowedAttention, 1U, 1U, validator},
            {kBlockDelta, 1U, 1U, validator},
            {kBlockBonus, 1U, 1U, validator},
+           {kBlockLatentAttention, 1U, 1U, validator},
+           {kBlockGatedLinear, 1U, 1U, validator},
            {kHeadBf16, 1U, 1U, validator}},
           nullptr};
 }
@@ -215,6 +279,30 @@ Mi355MixedProvider::Matrix Mi355MixedProvider::pack(std::uint32_t rows,
   return matrix;
 }
 
+DeviceBuffer Mi355MixedProvider::pack_heads(const er::ImmutableModelTensor& tensor,
+                                            std::uint32_t heads, std::uint32_t size,
+                                            std::uint32_t padded, bool transposed) {
+  const std::uint32_t width = tensor.shape.at(1);
+  const std::uint32_t rows = transposed ? width : size;
+  const std::uint32_t columns = transposed ? size : width;
+  const std::size_t bytes = qllm_linear_packed_bytes(heads * padded, columns);
+  DeviceBuffer packed(bytes, "allocate packed weights");
+  DeviceBuffer source(tensor.data_bytes, "allocate row-major weights");
+  hip_check(hipMemset(packed.get(), 0, bytes), "clear packed weights");
+  hip_check(hipMemcpy(source.get(), tensor.value.data + tensor.data_offset,
+                      tensor.data_bytes, hipMemcpyHostToDevice),
+            "upload weights");
+  hip_check(hipDeviceSynchronize(), "clear packed weights");
+  for (std::uint32_t head = 0; head < heads; ++head)
+    status_check(qllm_linear_pack_strided(
+        source.as<std::uint16_t>() + std::size_t{head} * size * width, rows, columns,
+        transposed ? 1U : width, transposed ? width : 1U, packed.get(),
+        round_up(columns, 64U), head * (padded / 16U), 1U, 0U, stream_));
+  hip_check(hipStreamSynchronize(static_cast<hipStream_t>(stream_)), "pack weights");
+  weight_bytes_ += bytes;
+  return packed;
+}
+
 void Mi355MixedProvider::prepare_block(Block& block,
                                        const er::OperationPreparationContext& context) {
   const auto& parameters = context.operation.parameters;
@@ -224,19 +312,28 @@ void Mi355MixedProvider::prepare_block(Block& block,
   block.epsilon = parameter_f32(parameters, "norm_epsilon_f32_bits");
   block.mixer_norm = upload_f32(tensor("mixer_norm"), g_.hidden);
   block.intermediate = parameter_or(parameters, "intermediate", 0U);
-  if (block.kind == Kind::attention)
+  block.sandwich = block.kind == Kind::latent || block.kind == Kind::gated;
+  std::uint32_t mixer_width{};
+  if (block.kind == Kind::attention) {
     prepare_attention(block, context);
-  else
+    mixer_width = block.attention.query_heads * block.attention.vdim;
+  } else if (block.kind == Kind::latent) {
+    prepare_latent(block, context);
+    mixer_width = block.latent.heads * block.latent.vdim;
+  } else {
     prepare_recurrence(block, context);
+    mixer_width = block.recurrence.heads * block.recurrence.vdim;
+  }
 
   const auto& output = tensor("output_projection");
-  const std::uint32_t mixer_width =
-      block.kind == Kind::attention ? block.attention.query_heads * block.attention.vdim
-                                    : block.recurrence.heads * block.recurrence.dim;
   require_matrix(output, g_.hidden, mixer_width);
   block.mixer_columns = round_up(mixer_width, 64U);
   std::vector<Part> joined{{&output, 0U, 1U, 0U}};
   std::uint32_t columns = block.mixer_columns;
+  if (block.sandwich) {
+    block.mixer_post_norm = upload_f32(tensor("mixer_post_norm"), g_.hidden);
+    block.residual_scale = parameter_f32(parameters, "residual_scale_f32_bits");
+  }
   if (block.intermediate) {
     block.activation = static_cast<std::uint32_t>(parameter(parameters, "activation"));
     block.ffn_norm = upload_f32(tensor("ffn_norm"), g_.hidden);
@@ -248,16 +345,28 @@ void Mi355MixedProvider::prepare_block(Block& block,
     require_matrix(down, g_.hidden, block.intermediate);
     const Part halves[]{{&gate, 0U, 2U, 0U}, {&up, 1U, 2U, 0U}};
     block.gate_up = pack(round_up(block.intermediate, 16U) * 2U, g_.hidden, halves);
-    joined.push_back({&down, 0U, 1U, block.mixer_columns});
-    columns += round_up(block.intermediate, 64U);
+    if (block.sandwich) {
+      const Part alone[]{{&down, 0U, 1U, 0U}};
+      block.ffn_post_norm = upload_f32(tensor("ffn_post_norm"), g_.hidden);
+      block.down = pack(g_.hidden, block.intermediate, alone);
+      block.down_splits = k_splits(block.down.rows, block.down.columns);
+    } else {
+      joined.push_back({&down, 0U, 1U, block.mixer_columns});
+      columns += round_up(block.intermediate, 64U);
+    }
   }
   block.output = pack(g_.hidden, columns, joined);
-  // enough workgroups for the chip where the rows alone are too few, each with
-  // a few KiB per wave left to stream
-  const std::uint32_t tiles = block.output.rows / 16U;
-  block.splits = std::clamp(std::min((768U + tiles - 1U) / tiles,
-                                     block.output.columns / 32U / 16U),
-                            1U, 8U);
+  block.splits = k_splits(block.output.rows, block.output.columns);
+}
+
+DeviceBuffer Mi355MixedProvider::upload_frequencies(const er::ParameterMap& parameters,
+                                                    std::uint32_t dims) {
+  const auto frequencies = rotation_of(parameters, dims).frequencies;
+  DeviceBuffer table(frequencies.size() * 8U, "allocate rotary table");
+  hip_check(hipMemcpy(table.get(), frequencies.data(), frequencies.size() * 8U,
+                      hipMemcpyHostToDevice),
+            "upload rotary table");
+  return table;
 }
 
 void Mi355MixedProvider::prepare_attention(Block& block,
@@ -280,19 +389,8 @@ void Mi355MixedProvider::prepare_attention(Block& block,
   block.rotary_dims = parameter_or(parameters, "rotary_dims", 0U);
   if (block.rotary_dims % 2U || block.rotary_dims > a.dim)
     throw std::runtime_error("rotary dimensions do not fit the head");
-  if (block.rotary_dims) {
-    const double base =
-        std::bit_cast<double>(parameter(parameters, "rotary_base_f64_bits"));
-    if (!(base > 0.0) || !std::isfinite(base))
-      throw std::runtime_error("rotary base is not positive");
-    std::vector<double> frequencies(block.rotary_dims / 2U);
-    for (std::size_t i = 0; i < frequencies.size(); ++i)
-      frequencies[i] = std::pow(base, -2.0 * static_cast<double>(i) / block.rotary_dims);
-    block.frequencies = DeviceBuffer(frequencies.size() * 8U, "allocate rotary table");
-    hip_check(hipMemcpy(block.frequencies.get(), frequencies.data(),
-                        frequencies.size() * 8U, hipMemcpyHostToDevice),
-              "upload rotary table");
-  }
+  if (block.rotary_dims)
+    block.frequencies = upload_frequencies(parameters, block.rotary_dims);
   if (const auto* mix = optional_tensor(context.tensors, "head_mix")) {
     block.head_mix = upload_f32(*mix, std::uint64_t{a.query_heads} * a.query_heads);
     a.head_mix = block.head_mix.as<float>();
@@ -325,23 +423,97 @@ void Mi355MixedProvider::prepare_attention(Block& block,
   block.projection_columns = rows;
 }
 
+void Mi355MixedProvider::prepare_latent(Block& block,
+                                        const er::OperationPreparationContext& context) {
+  const auto& parameters = context.operation.parameters;
+  auto& a = block.latent;
+  a.heads = static_cast<std::uint32_t>(parameter(parameters, "heads"));
+  a.dim = static_cast<std::uint32_t>(parameter(parameters, "dim"));
+  a.vdim = static_cast<std::uint32_t>(parameter(parameters, "vdim"));
+  a.rank = static_cast<std::uint32_t>(parameter(parameters, "latent_rank"));
+  a.rot_dim = parameter_or(parameters, "rotary_part", 0U);
+  a.rotary_dims = parameter_or(parameters, "rotary_dims", 0U);
+  if (a.rotary_dims % 2U || a.rotary_dims > a.rot_dim)
+    throw std::runtime_error("rotary dimensions do not fit the shared key part");
+  a.window = parameter_or(parameters, "window", 0U);
+  a.scale = parameter_f32(parameters, "score_scale_f32_bits");
+  a.epsilon = block.epsilon;
+  a.rotary_magnitude = 1.0F;
+  if (a.rotary_dims) {
+    block.frequencies = upload_frequencies(parameters, a.rotary_dims);
+    a.frequencies = block.frequencies.as<double>();
+    a.rotary_magnitude = static_cast<float>(rotation_of(parameters, a.rotary_dims).magnitude);
+  }
+  a.page_tokens = g_.kv_page_tokens;
+  a.element = g_.element;
+  block.latent_norm = upload_f32(tensor_for(context.tensors, "latent_norm"), a.rank);
+  a.latent_norm = block.latent_norm.as<float>();
+  const auto& key_up = tensor_for(context.tensors, "key_up");
+  const auto& value_up = tensor_for(context.tensors, "value_up");
+  require_matrix(key_up, std::uint64_t{a.heads} * a.dim, a.rank);
+  require_matrix(value_up, std::uint64_t{a.heads} * a.vdim, a.rank);
+  block.key_up = pack_heads(key_up, a.heads, a.dim, round_up(a.dim, 32U), false);
+  block.key_up_transposed = pack_heads(key_up, a.heads, a.dim, round_up(a.rank, 32U), true);
+  block.value_up = pack_heads(value_up, a.heads, a.vdim, round_up(a.vdim, 16U), false);
+  a.key_up = block.key_up.get();
+  a.key_up_transposed = block.key_up_transposed.get();
+  a.value_up = block.value_up.get();
+
+  std::vector<Part> parts;
+  std::uint32_t rows = 0U;
+  const auto place = [&](const char* role, std::uint32_t count) {
+    const auto& tensor = tensor_for(context.tensors, role);
+    require_matrix(tensor, count, g_.hidden);
+    const std::uint32_t column = rows;
+    parts.push_back({&tensor, rows / 16U, 1U, 0U});
+    rows += round_up(count, 16U);
+    return column;
+  };
+  const std::uint32_t query_width = a.heads * (a.dim + a.rot_dim);
+  if (const auto* down = optional_tensor(context.tensors, "query_down")) {
+    block.query_rank = down->shape.at(0);
+    block.query_column = place("query_down", block.query_rank);
+    block.query_norm =
+        upload_f32(tensor_for(context.tensors, "query_latent_norm"), block.query_rank);
+    const auto& up = tensor_for(context.tensors, "query_up");
+    require_matrix(up, query_width, block.query_rank);
+    const Part alone[]{{&up, 0U, 1U, 0U}};
+    block.query_up = pack(query_width, block.query_rank, alone);
+  } else {
+    block.query_column = place("query_projection", query_width);
+  }
+  block.latent_column = place("latent_down", a.rank + a.rot_dim);
+  if (optional_tensor(context.tensors, "output_gate"))
+    block.gate_column = place("output_gate", a.heads * a.vdim);
+  block.projections.push_back({pack(rows, g_.hidden, parts), 0U, 0U});
+  block.projection_columns = rows;
+}
+
 void Mi355MixedProvider::prepare_recurrence(
     Block& block, const er::OperationPreparationContext& context) {
   const auto& parameters = context.operation.parameters;
   auto& r = block.recurrence;
   const bool delta = block.kind == Kind::delta;
-  r.kind = delta ? QLLM_RECURRENCE_DELTA : QLLM_RECURRENCE_BONUS;
+  const bool gated = block.kind == Kind::gated;
+  r.kind = delta   ? QLLM_RECURRENCE_DELTA
+           : gated ? QLLM_RECURRENCE_GATED
+                   : QLLM_RECURRENCE_BONUS;
   r.gate_kind = delta ? QLLM_GATE_SIGMOID : QLLM_GATE_SILU;
   r.heads = static_cast<std::uint32_t>(parameter(parameters, "heads"));
   r.dim = static_cast<std::uint32_t>(parameter(parameters, "dim"));
+  r.vdim = parameter_or(parameters, "vdim", r.dim);
   r.element = g_.element;
   r.epsilon = block.epsilon;
   const std::uint32_t channels = r.heads * r.dim;
+  const std::uint32_t values = r.heads * r.vdim;
   if (delta) {
     r.unit_epsilon = parameter_f32(parameters, "unit_epsilon_f32_bits");
     r.decay_scale = parameter_f32(parameters, "decay_scale_f32_bits");
     block.rate_bias = upload_f32(tensor_for(context.tensors, "rate_bias"), channels);
     r.rate_bias = block.rate_bias.as<float>();
+  } else if (gated) {
+    r.decay_scale = parameter_f32(parameters, "decay_scale_f32_bits");
+    r.read_scale = parameter_f32(parameters, "read_scale_f32_bits");
   } else {
     block.bonus = upload_f32(tensor_for(context.tensors, "bonus"), channels);
     r.bonus = block.bonus.as<float>();
@@ -355,7 +527,8 @@ void Mi355MixedProvider::prepare_recurrence(
   require_matrix(up, channels, r.rank);
   block.decay_up = upload_raw(up);
   block.decay_base = upload_f32(tensor_for(context.tensors, "decay_base"), channels);
-  block.output_norm = upload_f32(tensor_for(context.tensors, "output_norm"), channels);
+  block.output_norm =
+      upload_f32(tensor_for(context.tensors, "output_norm"), gated ? r.vdim : channels);
   r.decay_up_bf16 = block.decay_up.get();
   r.decay_base = block.decay_base.as<float>();
   r.norm_weight = block.output_norm.as<float>();
@@ -369,12 +542,12 @@ void Mi355MixedProvider::prepare_recurrence(
   std::vector<Wanted> wanted{
       {"read_projection", "read_shift", channels, &block.r_column},
       {"key_projection", "key_shift", channels, &block.key_column},
-      {"value_projection", "value_shift", channels, &block.value_column},
-      {"gate_projection_mixer", "gate_shift", channels, &block.gate_column},
+      {"value_projection", "value_shift", values, &block.value_column},
+      {"gate_projection_mixer", "gate_shift", values, &block.gate_column},
       {"decay_down", "decay_shift", r.rank, &block.low_column}};
   if (delta)
     wanted.push_back({"rate_projection", nullptr, channels, &block.rate_column});
-  const bool shifted = !delta;
+  const bool shifted = block.kind == Kind::bonus;
   std::vector<Part> parts;
   std::uint32_t rows = 0U;
   for (const auto& item : wanted) {
@@ -434,6 +607,10 @@ er::PrepareOperationResult Mi355MixedProvider::prepare(
         block->kind = Kind::delta;
       else if (capability == kBlockBonus)
         block->kind = Kind::bonus;
+      else if (capability == kBlockLatentAttention)
+        block->kind = Kind::latent;
+      else if (capability == kBlockGatedLinear)
+        block->kind = Kind::gated;
       else
         return {{er::ErrorCode::invalid_argument,
                  "capability is not provided: " + capability},
@@ -468,7 +645,7 @@ void Mi355MixedProvider::finalize_locked() {
   for (auto& item : blocks_) {
     Block& block = *item;
     projection_stride_ = std::max(projection_stride_, block.projection_columns);
-    joined_stride_ = std::max(joined_stride_, block.output.columns);
+    joined_stride_ = std::max({joined_stride_, block.output.columns, block.down.columns});
     shift_inputs_ = std::max(shift_inputs_, static_cast<std::uint32_t>(block.shifts.size()));
     if (block.kind == Kind::attention) {
       auto& a = block.attention;
@@ -478,10 +655,17 @@ void Mi355MixedProvider::finalize_locked() {
       if (!a.window) pages_expire_ = false;
       widest_window_ = std::max(widest_window_, a.window);
       most_sinks_ = std::max(most_sinks_, a.sinks);
+    } else if (block.kind == Kind::latent) {
+      auto& a = block.latent;
+      a.layer_offset = page_bytes_;
+      page_bytes_ +=
+          qllm_latent_layer_bytes(g_.kv_page_tokens, a.rank, a.rot_dim, g_.element);
+      if (!a.window) pages_expire_ = false;
+      widest_window_ = std::max(widest_window_, a.window);
     } else {
       block.state_offset = state_floats_;
       state_floats_ += std::uint64_t{block.recurrence.heads} * block.recurrence.dim *
-                       block.recurrence.dim;
+                       block.recurrence.vdim;
       state_floats_ = (state_floats_ + 3U) / 4U * 4U;
       if (!block.shifts.empty()) {
         block.carry_offset = state_floats_;
@@ -523,6 +707,10 @@ void Mi355MixedProvider::finalize_locked() {
       block.attention.page_table = page_table_.as<void*>();
       block.attention.pages_per_slot = static_cast<std::uint32_t>(pages);
       block.attention.step = step;
+    } else if (block.kind == Kind::latent) {
+      block.latent.page_table = page_table_.as<void*>();
+      block.latent.pages_per_slot = static_cast<std::uint32_t>(pages);
+      block.latent.step = step;
     } else {
       block.recurrence.state = states_.as<float>() + block.state_offset;
       block.recurrence.slot_stride = state_floats_;
@@ -532,12 +720,31 @@ void Mi355MixedProvider::finalize_locked() {
   finalized_ = true;
 }
 
-// Buffers for batches of up to `rows` rows; they only grow.
-void Mi355MixedProvider::ensure_workspace(std::uint32_t rows) {
-  if (rows <= workspace_rows_) return;
+std::size_t Mi355MixedProvider::scratch_bytes_for(std::uint32_t rows,
+                                                  std::uint32_t last_position) const {
+  std::size_t bytes = 16U;
+  for (const auto& item : blocks_) {
+    const Block& block = *item;
+    if (block.kind == Kind::attention)
+      bytes = std::max(bytes, qllm_windowed_attention_workspace_bytes(&block.attention, rows,
+                                                                      last_position));
+    else if (block.kind == Kind::latent)
+      bytes = std::max(bytes, qllm_latent_attention_workspace_bytes(&block.latent, rows,
+                                                                    last_position));
+    else
+      bytes = std::max(bytes, qllm_recurrence_workspace_bytes(&block.recurrence, rows));
+  }
+  return bytes;
+}
+
+// Buffers for batches of up to `rows` rows that end at or before last_position; they
+// only grow.  A few rows find room wherever they stand.
+void Mi355MixedProvider::ensure_workspace(std::uint32_t rows, std::uint32_t last_position) {
+  if (rows <= workspace_rows_ && scratch_bytes_for(rows, last_position) <= scratch_bytes_)
+    return;
   std::uint32_t size = 64U;
   while (size < rows) size *= 2U;
-  size = std::min(std::max(size, rows), std::max(g_.chunk_rows, 64U));
+  size = std::min(std::max({size, rows, workspace_rows_}), std::max(g_.chunk_rows, 64U));
   if (step_graph_) {   // it addresses the buffers that are about to go
     (void)hipGraphExecDestroy(static_cast<hipGraphExec_t>(step_graph_));
     step_graph_ = nullptr;
@@ -549,21 +756,31 @@ void Mi355MixedProvider::ensure_workspace(std::uint32_t rows) {
     hip_check(hipMemset(buffer.get(), 0, std::max<std::size_t>(bytes, 16U)), what);
     return buffer;
   };
+  const std::uint32_t last = g_.max_context - 1U;
+  // room for the context to double
+  const std::uint32_t ahead = static_cast<std::uint32_t>(
+      std::min<std::uint64_t>(last, std::uint64_t{2U} * std::max(last_position, size)));
+  std::size_t scratch = std::max(scratch_bytes_, scratch_bytes_for(size, ahead));
+  for (std::uint32_t few = 1U; few <= std::min(size, kSmallBatch); ++few)
+    scratch = std::max(scratch, scratch_bytes_for(few, last));
   std::size_t query = 0U;
   std::size_t kept = 0U;
-  std::size_t scratch = 16U;
+  std::size_t query_rank = 0U;
+  std::size_t query_width = 0U;
   std::size_t partial_rows = 0U;
   for (const auto& item : blocks_) {
     const Block& block = *item;
-    partial_rows = std::max<std::size_t>(partial_rows, block.splits);
+    partial_rows = std::max<std::size_t>(
+        partial_rows, std::max(block.splits, block.down_splits) * kSmallBatch);
+    if (block.sandwich) partial_rows = std::max<std::size_t>(partial_rows, size);
     if (block.kind == Kind::attention) {
       const auto& a = block.attention;
       query = std::max(query, std::size_t{a.query_heads} * a.key_stride);
       kept = std::max(kept, std::size_t{a.kv_heads} * a.vdim);
-      scratch = std::max(scratch, qllm_windowed_attention_workspace_bytes(
-                                      &a, size, g_.max_context - 1U));
-    } else {
-      scratch = std::max(scratch, qllm_recurrence_workspace_bytes(&block.recurrence, size));
+      scratch = std::max(scratch, qllm_windowed_attention_workspace_bytes(&a, size, last));
+    } else if (block.kind == Kind::latent && block.query_rank) {
+      query_rank = std::max<std::size_t>(query_rank, block.query_up.columns);
+      query_width = std::max<std::size_t>(query_width, block.query_up.rows);
     }
   }
   workspace_rows_ = 0U;
@@ -576,9 +793,11 @@ void Mi355MixedProvider::ensure_workspace(std::uint32_t rows) {
                         "allocate projections");
   joined_ = zeroed(std::size_t{size} * joined_stride_ * element, "allocate layer outputs");
   query_ = zeroed(std::size_t{size} * query * element, "allocate queries");
+  query_latents_ = zeroed(std::size_t{size} * query_rank * element, "allocate query latents");
+  queries_ = zeroed(std::size_t{size} * query_width * 4U, "allocate latent queries");
   kept_values_ = zeroed(std::size_t{size} * kept * 4U, "allocate kept values");
   shift_last_ = zeroed(std::size_t{round_up(g_.hidden, 4U)} * 4U, "allocate shifted row");
-  partials_ = zeroed(partial_rows * kSmallBatch * round_up(g_.hidden, 4U) * 4U,
+  partials_ = zeroed(partial_rows * round_up(g_.hidden, 4U) * 4U,
                      "allocate partial sums");
   scratch_ = zeroed(scratch, "allocate mixer scratch");
   scratch_bytes_ = scratch;
@@ -676,7 +895,7 @@ void Mi355MixedProvider::begin_batch(MixedRequestState& state,
       throw std::runtime_error("embedding token exceeds vocabulary");
   for (const auto row : state.logit_rows)
     if (row >= rows) throw std::runtime_error("logit row exceeds the batch");
-  ensure_workspace(rows);
+  ensure_workspace(rows, first_position + rows - 1U);
   const auto stream = static_cast<hipStream_t>(stream_);
   void** table =
       page_table_.as<void*>() + std::size_t{state.slot} * slots_.pages_per_slot();
@@ -703,6 +922,7 @@ void Mi355MixedProvider::begin_batch(MixedRequestState& state,
 void Mi355MixedProvider::enqueue_embedding(std::uint32_t rows) {
   stream_index_ = 0U;
   pending_partials_ = 0U;
+  pending_branch_ = {};
   status_check(qllm_embedding_bf16_batch(
       embedding_.get(), g_.vocabulary, step_.as<std::uint32_t>() + kStepWords,
       hidden_[0].as<float>(), rows, g_.hidden, embedding_scale_, stream_));
@@ -765,8 +985,149 @@ void Mi355MixedProvider::enqueue_recurrence(Block& block, std::uint32_t rows) {
   status_check(qllm_recurrence_rows(&block.recurrence, &launch, stream_));
 }
 
+void Mi355MixedProvider::enqueue_latent(Block& block, std::uint32_t rows,
+                                        std::uint32_t last_position) {
+  auto& a = block.latent;
+  qllm_latent_store_launch store{};
+  store.projections = projections_.as<float>();
+  store.stride = projection_stride_;
+  store.latent_column = block.latent_column;
+  store.rows = rows;
+  if (block.query_rank) {
+    store.query_column = block.query_column;
+    store.query_rank = block.query_rank;
+    store.query_norm = block.query_norm.as<float>();
+    store.query_out = query_latents_.get();
+    store.query_stride = block.query_up.columns;
+  }
+  status_check(qllm_latent_store(&a, &store, stream_));
+
+  qllm_latent_launch launch{};
+  launch.query = projections_.as<float>() + block.query_column;
+  launch.query_stride = projection_stride_;
+  if (block.query_rank) {
+    qllm_linear_segment s{};
+    s.weights = block.query_up.data.get();
+    s.input = query_latents_.get();
+    s.output = queries_.get();
+    s.rows = block.query_up.rows;
+    s.columns = block.query_up.columns;
+    s.input_stride = block.query_up.columns;
+    s.output_stride = block.query_up.rows;
+    s.output_columns = a.heads * (a.dim + a.rot_dim);
+    s.epilogue = QLLM_LINEAR_STORE;
+    status_check(qllm_linear_batch(&s, 1U, rows, g_.element, stream_));
+    launch.query = queries_.as<float>();
+    launch.query_stride = block.query_up.rows;
+  }
+  launch.gate =
+      block.gate_column ? projections_.as<float>() + block.gate_column : nullptr;
+  launch.gate_stride = projection_stride_;
+  launch.output = joined_.get();
+  launch.output_stride = block.output.columns;
+  launch.rows = rows;
+  launch.maximum_position = last_position;
+  launch.workspace = scratch_.get();
+  launch.workspace_bytes = scratch_bytes_;
+  status_check(qllm_latent_attention_rows(&a, &launch, stream_));
+}
+
+void Mi355MixedProvider::enqueue_mixer(Block& block, std::uint32_t rows,
+                                       std::uint32_t last_position) {
+  if (block.kind == Kind::attention)
+    enqueue_attention(block, rows, last_position);
+  else if (block.kind == Kind::latent)
+    enqueue_latent(block, rows, last_position);
+  else
+    enqueue_recurrence(block, rows);
+}
+
+qllm_stream_norm_launch Mi355MixedProvider::stream_norm(std::uint32_t rows, float epsilon) {
+  qllm_stream_norm_launch norm{};
+  norm.input = hidden_[stream_index_].as<float>();
+  norm.rows = rows;
+  norm.width = g_.hidden;
+  norm.epsilon = epsilon;
+  norm.element = g_.element;
+  norm.step = step_.as<std::uint32_t>();
+  if (pending_partials_) {
+    norm.partials = partials_.as<float>();
+    norm.partial_count = pending_partials_;
+    norm.partial_stride = round_up(g_.hidden, 4U);
+    norm.branch_weight = pending_branch_.weight;
+    norm.branch_scale = pending_branch_.scale;
+    norm.branch_epsilon = pending_branch_.epsilon;
+    stream_index_ = 1U - stream_index_;
+    norm.stream_out = hidden_[stream_index_].as<float>();
+    pending_partials_ = 0U;
+    pending_branch_ = {};
+  }
+  return norm;
+}
+
+// Mixer and feed-forward one after the other; each leaves its output as partial
+// sums (a single one, from a tall batch) that the next norm takes.
+void Mi355MixedProvider::enqueue_sandwich(Block& block, std::uint32_t rows,
+                                          std::uint32_t last_position) {
+  const auto normed = [&](const DeviceBuffer& weight) {
+    auto norm = stream_norm(rows, block.epsilon);
+    norm.weight[0] = weight.as<float>();
+    norm.output[0] = inputs_.get();
+    norm.stride[0] = mixer_stride_;
+    status_check(qllm_stream_norm(&norm, stream_));
+  };
+  const auto project = [&](const Matrix& matrix, std::uint32_t splits,
+                           const DeviceBuffer& post_norm) {
+    const bool split = g_.element == QLLM_ELEMENT_BF16 && rows <= kSmallBatch;
+    qllm_linear_segment s{};
+    s.weights = matrix.data.get();
+    s.input = joined_.get();
+    s.output = partials_.get();
+    s.rows = matrix.rows;
+    s.columns = matrix.columns;
+    s.input_stride = matrix.columns;
+    s.output_stride = round_up(g_.hidden, 4U);
+    s.output_columns = g_.hidden;
+    s.epilogue = split ? QLLM_LINEAR_PARTIALS : QLLM_LINEAR_STORE;
+    s.splits = split ? splits : 0U;
+    status_check(qllm_linear_batch(&s, 1U, rows, g_.element, stream_));
+    pending_partials_ = split ? splits : 1U;
+    pending_branch_ = {post_norm.as<float>(), block.residual_scale, block.epsilon};
+  };
+  qllm_linear_segment s{};
+  s.input = inputs_.get();
+  s.input_stride = mixer_stride_;
+
+  normed(block.mixer_norm);
+  const auto& projection = block.projections.front();
+  s.weights = projection.matrix.data.get();
+  s.output = projections_.get();
+  s.rows = projection.matrix.rows;
+  s.columns = projection.matrix.columns;
+  s.output_stride = projection_stride_;
+  s.output_columns = projection.matrix.rows;
+  s.epilogue = QLLM_LINEAR_STORE;
+  status_check(qllm_linear_batch(&s, 1U, rows, g_.element, stream_));
+  enqueue_mixer(block, rows, last_position);
+  project(block.output, block.splits, block.mixer_post_norm);
+  if (!block.intermediate) return;
+
+  normed(block.ffn_norm);
+  s.weights = block.gate_up.data.get();
+  s.output = joined_.get();
+  s.rows = block.gate_up.rows;
+  s.columns = block.gate_up.columns;
+  s.output_stride = block.down.columns;
+  s.output_columns = block.intermediate;
+  s.epilogue = QLLM_LINEAR_GATED;
+  s.activation = block.activation;
+  status_check(qllm_linear_batch(&s, 1U, rows, g_.element, stream_));
+  project(block.down, block.down_splits, block.ffn_post_norm);
+}
+
 void Mi355MixedProvider::enqueue_block(Block& block, std::uint32_t rows,
                                        std::uint32_t last_position) {
+  if (block.sandwich) return enqueue_sandwich(block, rows, last_position);
   const std::size_t element = g_.element == QLLM_ELEMENT_F32 ? 4U : 2U;
   const auto input = [&](std::uint32_t index) {
     return static_cast<void*>(inputs_.as<std::uint8_t>() +
@@ -774,9 +1135,8 @@ void Mi355MixedProvider::enqueue_block(Block& block, std::uint32_t rows,
   };
   const std::uint32_t ffn_input = std::max(shift_inputs_, 1U);
 
-  qllm_stream_norm_launch norm{};
   qllm_token_shift shift{};
-  norm.input = hidden_[stream_index_].as<float>();
+  auto norm = stream_norm(rows, block.epsilon);
   norm.weight[0] = block.mixer_norm.as<float>();
   norm.output[0] = input(0U);
   norm.stride[0] = mixer_stride_;
@@ -784,19 +1144,6 @@ void Mi355MixedProvider::enqueue_block(Block& block, std::uint32_t rows,
     norm.weight[1] = block.ffn_norm.as<float>();
     norm.output[1] = input(ffn_input);
     norm.stride[1] = mixer_stride_;
-  }
-  norm.rows = rows;
-  norm.width = g_.hidden;
-  norm.epsilon = block.epsilon;
-  norm.element = g_.element;
-  norm.step = step_.as<std::uint32_t>();
-  if (pending_partials_) {
-    norm.partials = partials_.as<float>();
-    norm.partial_count = pending_partials_;
-    norm.partial_stride = round_up(g_.hidden, 4U);
-    stream_index_ = 1U - stream_index_;
-    norm.stream_out = hidden_[stream_index_].as<float>();
-    pending_partials_ = 0U;
   }
   if (!block.shifts.empty()) {
     shift.count = static_cast<std::uint32_t>(block.shifts.size());
@@ -841,10 +1188,7 @@ void Mi355MixedProvider::enqueue_block(Block& block, std::uint32_t rows,
   }
   status_check(qllm_linear_batch(segments.data(), static_cast<std::uint32_t>(segments.size()),
                                  rows, g_.element, stream_));
-  if (block.kind == Kind::attention)
-    enqueue_attention(block, rows, last_position);
-  else
-    enqueue_recurrence(block, rows);
+  enqueue_mixer(block, rows, last_position);
 
   qllm_linear_segment s{};
   s.weights = block.output.data.get();
@@ -869,18 +1213,7 @@ void Mi355MixedProvider::enqueue_block(Block& block, std::uint32_t rows,
 
 void Mi355MixedProvider::settle_stream(std::uint32_t rows) {
   if (!pending_partials_) return;
-  qllm_stream_norm_launch norm{};
-  norm.input = hidden_[stream_index_].as<float>();
-  stream_index_ = 1U - stream_index_;
-  norm.stream_out = hidden_[stream_index_].as<float>();
-  norm.partials = partials_.as<float>();
-  norm.partial_count = pending_partials_;
-  norm.partial_stride = round_up(g_.hidden, 4U);
-  norm.rows = rows;
-  norm.width = g_.hidden;
-  norm.epsilon = final_epsilon_;
-  norm.element = g_.element;
-  pending_partials_ = 0U;
+  const auto norm = stream_norm(rows, final_epsilon_);
   status_check(qllm_stream_norm(&norm, stream_));
 }
 
@@ -888,26 +1221,12 @@ void Mi355MixedProvider::settle_stream(std::uint32_t rows) {
 // the rows listed in gather_.
 void Mi355MixedProvider::enqueue_head(std::uint32_t batch_rows, std::uint32_t first,
                                       std::uint32_t count, bool gather) {
-  qllm_stream_norm_launch norm{};
-  if (pending_partials_ && batch_rows == 1U) {
-    norm.partials = partials_.as<float>();
-    norm.partial_count = pending_partials_;
-    norm.partial_stride = round_up(g_.hidden, 4U);
-    norm.input = hidden_[stream_index_].as<float>();
-    stream_index_ = 1U - stream_index_;
-    norm.stream_out = hidden_[stream_index_].as<float>();
-    pending_partials_ = 0U;
-  } else {
-    settle_stream(batch_rows);
-    norm.input = hidden_[stream_index_].as<float>() + std::size_t{first} * g_.hidden;
-  }
+  if (batch_rows != 1U) settle_stream(batch_rows);
+  auto norm = stream_norm(count, final_epsilon_);
+  norm.input += std::size_t{first} * g_.hidden;
   norm.weight[0] = final_norm_.as<float>();
   norm.output[0] = head_input_.get();
   norm.stride[0] = mixer_stride_;
-  norm.rows = count;
-  norm.width = g_.hidden;
-  norm.epsilon = final_epsilon_;
-  norm.element = g_.element;
   norm.gather = gather ? gather_.as<std::uint32_t>() : nullptr;
   status_check(qllm_stream_norm(&norm, stream_));
   qllm_linear_segment s{};

@@ -1,13 +1,17 @@
 // MI355X provider for mixed-layer decoders: layers of different kinds on one
 // F32 residual stream, bf16 weights, bf16 or F32 arithmetic.
 //
-// Every layer is one operation, a parallel block: one norm launch (which also
+// Every layer is one operation.  A parallel block: one norm launch (which also
 // adds the partial sums of the layer before), one launch for all projections
 // of mixer and feed-forward with the activation in its epilogue, the mixer,
 // and one launch for both output projections, laid side by side along K.
-// Three mixers: windowed attention with mixed heads over the paged cache, the
-// generalised delta rule, and the bonus recurrence over token-shifted inputs,
-// whose states live beside the pages in their request's slot.
+// A sandwich block runs its mixer and its feed-forward one after the other,
+// each between a norm of its input and a norm of its output; the latter is taken
+// by the norm launch that follows, with the sublayer's partial sums.
+// Five mixers: windowed attention with mixed heads and latent attention over the
+// paged cache, and the generalised delta rule, the bonus recurrence over
+// token-shifted inputs and gated linear attention, whose states live beside the
+// pages in their request's slot.
 //
 // A batch is any run of consecutive tokens of one request.  A single token is
 // replayed from a captured graph: kernels read token, position and slot from
@@ -38,6 +42,8 @@ inline constexpr char kBlockWindowedAttention[] =
     "block.parallel.windowed-attention.mixed-heads.v1";
 inline constexpr char kBlockDelta[] = "block.parallel.general-delta.v1";
 inline constexpr char kBlockBonus[] = "block.parallel.bonus-recurrence.token-shift.v1";
+inline constexpr char kBlockLatentAttention[] = "block.sandwich.latent-attention.v1";
+inline constexpr char kBlockGatedLinear[] = "block.sandwich.gated-linear-attention.v1";
 inline constexpr char kHeadBf16[] = "head.rmsnorm.logits.bf16.v1";
 
 // Parameter value_blend of a windowed attention block.
@@ -108,7 +114,7 @@ class Mi355MixedProvider final : public DecoderProvider {
   [[nodiscard]] er::Status copy_hidden(std::uint32_t rows, float* host);
 
  private:
-  enum class Kind { embedding, attention, delta, bonus, head };
+  enum class Kind { embedding, attention, latent, delta, bonus, gated, head };
   struct Matrix final {
     DeviceBuffer data;
     std::uint32_t rows{};      // packed
@@ -127,17 +133,30 @@ class Mi355MixedProvider final : public DecoderProvider {
   Matrix pack(std::uint32_t rows, std::uint32_t columns, std::span<const Part> parts);
   DeviceBuffer upload_raw(const er::ImmutableModelTensor& tensor);
   DeviceBuffer upload_f32(const er::ImmutableModelTensor& tensor, std::uint64_t elements);
+  // Packed per-head matrices: rows of the tensor cut into `heads` parts of `size`
+  // rows, each padded to `padded` rows of the packed matrix (of its columns, when
+  // transposed).
+  DeviceBuffer pack_heads(const er::ImmutableModelTensor& tensor, std::uint32_t heads,
+                          std::uint32_t size, std::uint32_t padded, bool transposed);
+  DeviceBuffer upload_frequencies(const er::ParameterMap& parameters, std::uint32_t dims);
   void prepare_block(Block& block, const er::OperationPreparationContext& context);
   void prepare_attention(Block& block, const er::OperationPreparationContext& context);
+  void prepare_latent(Block& block, const er::OperationPreparationContext& context);
   void prepare_recurrence(Block& block, const er::OperationPreparationContext& context);
 
   // execution
   void finalize_locked();
-  void ensure_workspace(std::uint32_t rows);
+  std::size_t scratch_bytes_for(std::uint32_t rows, std::uint32_t last_position) const;
+  void ensure_workspace(std::uint32_t rows, std::uint32_t last_position);
   void begin_batch(MixedRequestState& state, std::span<const std::uint32_t> tokens,
                    std::uint32_t first_position);
   void enqueue_embedding(std::uint32_t rows);
   void enqueue_block(Block& block, std::uint32_t rows, std::uint32_t last_position);
+  void enqueue_sandwich(Block& block, std::uint32_t rows, std::uint32_t last_position);
+  void enqueue_mixer(Block& block, std::uint32_t rows, std::uint32_t last_position);
+  // Norm launch over the stream with what partial sums are pending.
+  [[nodiscard]] qllm_stream_norm_launch stream_norm(std::uint32_t rows, float epsilon);
+  void enqueue_latent(Block& block, std::uint32_t rows, std::uint32_t last_position);
   void enqueue_attention(Block& block, std::uint32_t rows, std::uint32_t last_position);
   void enqueue_recurrence(Block& block, std::uint32_t rows);
   void settle_stream(std::uint32_t rows);   // adds what partial sums are pending
@@ -195,6 +214,8 @@ class Mi355MixedProvider final : public DecoderProvider {
   DeviceBuffer projections_;
   DeviceBuffer joined_;          // mixer output | activation
   DeviceBuffer query_;
+  DeviceBuffer query_latents_;   // normed, element
+  DeviceBuffer queries_;         // F32, from query latents
   DeviceBuffer kept_values_;
   DeviceBuffer shift_last_;
   DeviceBuffer partials_;
@@ -212,6 +233,13 @@ class Mi355MixedProvider final : public DecoderProvider {
 
   std::uint32_t stream_index_{}; // which of hidden_ holds the stream
   std::uint32_t pending_partials_{};
+  // the norm pending partial sums pass on their way into the stream, if any
+  struct Branch final {
+    const float* weight{};
+    float scale{};
+    float epsilon{};
+  };
+  Branch pending_branch_;
   std::uint32_t batch_rows_{};
   void* step_graph_{};
   bool use_graphs_{true};

@@ -131,6 +131,40 @@ void bind(er::BindingMap& tensors, const std::string& prefix,
   for (const auto& [role, name] : roles) tensors.emplace(role, prefix + name);
 }
 
+std::uint64_t f64_bits(const json::Object& object, std::string_view key,
+                       std::string_view where) {
+  return std::bit_cast<std::uint64_t>(json::required(object, key, where).number(key));
+}
+
+// A rotation's dimensions, base and - when there is one - stretched frequencies.
+void rotary(const json::Object& rot, er::ParameterMap& parameters) {
+  parameters["rotary_dims"] = u32(rot, "dims", "mixer.rot");
+  parameters["rotary_base_f64_bits"] = f64_bits(rot, "base", "mixer.rot");
+  if (const auto* scaling = optional_object(rot, "scaling"))
+    for (const auto& [name, key] : std::initializer_list<std::pair<const char*, const char*>>{
+             {"rotary_factor_f64_bits", "factor"},
+             {"rotary_original_f64_bits", "original"},
+             {"rotary_fast_f64_bits", "fast"},
+             {"rotary_slow_f64_bits", "slow"}})
+      parameters[name] = f64_bits(*scaling, key, "mixer.rot.scaling");
+}
+
+// A dense gated feed-forward behind its norm.
+void dense_feed_forward(const json::Object& mlp, std::uint32_t activation,
+                        const std::string& prefix, er::ParameterMap& parameters,
+                        er::BindingMap& tensors) {
+  const auto& kind = json::required(mlp, "kind", "layer.mlp").string("mlp.kind");
+  if (kind != "dense")
+    throw std::runtime_error("feed-forward kind is not supported: " + kind);
+  parameters["intermediate"] = positive(mlp, "ff", "layer.mlp");
+  parameters["activation"] = activation;
+  bind(tensors, prefix,
+       {{"ffn_norm", "norm2"},
+        {"gate_projection", "mlp.gate"},
+        {"up_projection", "mlp.up"},
+        {"down_projection", "mlp.down"}});
+}
+
 // ---- Zatupel -----------------------------------------------------------------
 // Parallel layers with two norms: a mixer (windowed attention with mixed heads,
 // generalised delta rule, or bonus recurrence over token-shifted inputs) and a
@@ -165,16 +199,7 @@ er::ModelDescriptor describe_zatupel(const json::Object& config,
     bind(tensors, prefix, {{"mixer_norm", "norm1"}});
 
     if (const auto* mlp = optional_object(layer, "mlp")) {
-      const auto& kind = json::required(*mlp, "kind", "layer.mlp").string("mlp.kind");
-      if (kind != "dense")
-        throw std::runtime_error("feed-forward kind is not supported: " + kind);
-      parameters["intermediate"] = positive(*mlp, "ff", "layer.mlp");
-      parameters["activation"] = QLLM_ACTIVATION_GELU_TANH;
-      bind(tensors, prefix,
-           {{"ffn_norm", "norm2"},
-            {"gate_projection", "mlp.gate"},
-            {"up_projection", "mlp.up"},
-            {"down_projection", "mlp.down"}});
+      dense_feed_forward(*mlp, QLLM_ACTIVATION_GELU_TANH, prefix, parameters, tensors);
     }
 
     parameters["heads"] = positive(mixer, "heads", "layer.mixer");
@@ -184,10 +209,8 @@ er::ModelDescriptor describe_zatupel(const json::Object& config,
       parameters["kv_heads"] = positive(mixer, "kv_heads", "layer.mixer");
       parameters["vdim"] = positive(mixer, "vdim", "layer.mixer");
       parameters["score_scale_f32_bits"] = number_bits(mixer, "scale", "layer.mixer");
-      if (const auto* rotary = optional_object(mixer, "rot")) {
-        parameters["rotary_dims"] = u32(*rotary, "dims", "mixer.rot");
-        parameters["rotary_base_f64_bits"] = std::bit_cast<std::uint64_t>(
-            json::required(*rotary, "base", "mixer.rot").number("mixer.rot.base"));
+      if (const auto* turned = optional_object(mixer, "rot")) {
+        rotary(*turned, parameters);
       }
       if (const auto* mask = optional_object(mixer, "mask")) {
         parameters["window"] = positive(*mask, "size", "mixer.mask");
@@ -247,7 +270,95 @@ er::ModelDescriptor describe_zatupel(const json::Object& config,
   return model;
 }
 
-constexpr ModelDesign kDesigns[]{{"Zatupel", &describe_zatupel}};
+// ---- Nametar -----------------------------------------------------------------
+// Layers with a norm before and after each sublayer: a mixer (latent attention
+// without positions and with an output gate, windowed latent attention with a
+// query latent and a rotated shared key part, or gated linear attention), then a
+// gated feed-forward or none.
+
+er::ModelDescriptor describe_nametar(const json::Object& config,
+                                     er::IModelTensorStore&) {
+  er::ModelDescriptor model;
+  model.architecture_id = "nametar";
+  model.vocab_size = positive(config, "vocab", "config");
+  model.hidden_size = positive(config, "width", "config");
+  model.max_context_tokens = kDefaultMaximumContext;
+  const auto& norm = json::required(config, "norm", "config").object("config.norm");
+  const auto epsilon = number_bits(norm, "eps", "config.norm");
+  const auto residual_scale = number_bits(config, "residual_mult", "config");
+  const auto& embedding =
+      json::required(config, "embedding", "config").object("config.embedding");
+
+  ProgramBuilder program(model);
+  program.embedding(kEmbeddingBf16,
+                    {{"scale_f32_bits", number_bits(embedding, "scale", "embedding")}},
+                    {{"weight", "embed"}});
+  std::size_t index = 0U;
+  for (const auto& entry : json::required(config, "layers", "config").array("layers")) {
+    const auto& layer = entry.object("layer");
+    const auto& mixer = json::required(layer, "mixer", "layer").object("layer.mixer");
+    const auto& type = json::required(layer, "type", "layer").string("layer.type");
+    const std::string prefix = "l" + std::to_string(index++) + ".";
+    const std::string mix = prefix + "mix.";
+    er::ParameterMap parameters{{"norm_epsilon_f32_bits", epsilon},
+                                {"residual_scale_f32_bits", residual_scale}};
+    er::BindingMap tensors;
+    bind(tensors, prefix, {{"mixer_norm", "norm1"}, {"mixer_post_norm", "norm1b"}});
+    if (const auto* mlp = optional_object(layer, "mlp")) {
+      dense_feed_forward(*mlp, QLLM_ACTIVATION_SILU, prefix, parameters, tensors);
+      bind(tensors, prefix, {{"ffn_post_norm", "norm2b"}});
+    }
+
+    const auto dim = positive(mixer, "dim", "layer.mixer");
+    parameters["heads"] = positive(mixer, "heads", "layer.mixer");
+    parameters["dim"] = dim;
+    parameters["vdim"] = positive(mixer, "vdim", "layer.mixer");
+    bind(tensors, mix, {{"output_projection", "o"}});
+    if (type == "latent_attention" || type == "latent_attention_2") {
+      parameters["latent_rank"] = positive(mixer, "kv_rank", "layer.mixer");
+      parameters["score_scale_f32_bits"] = number_bits(mixer, "scale", "layer.mixer");
+      bind(tensors, mix,
+           {{"latent_down", "dkv"},
+            {"latent_norm", "dkv.norm"},
+            {"key_up", "uk"},
+            {"value_up", "uv"}});
+      if (type == "latent_attention") {
+        bind(tensors, mix, {{"query_projection", "q"}, {"output_gate", "g"}});
+      } else {
+        bind(tensors, mix,
+             {{"query_down", "dq"}, {"query_latent_norm", "dq.norm"}, {"query_up", "uq"}});
+        parameters["rotary_part"] = positive(mixer, "rot_dim", "layer.mixer");
+        rotary(json::required(mixer, "rot", "layer.mixer").object("mixer.rot"), parameters);
+        const auto& mask = json::required(mixer, "mask", "layer.mixer").object("mixer.mask");
+        parameters["window"] = positive(mask, "size", "mixer.mask");
+      }
+      program.block(kBlockLatentAttention, std::move(parameters), std::move(tensors));
+    } else if (type == "gla") {
+      const double tau = json::required(mixer, "tau", "layer.mixer").number("mixer.tau");
+      if (!(tau > 0.0)) throw std::runtime_error("tau must be positive");
+      parameters["decay_scale_f32_bits"] = f32_bits(1.0 / tau);
+      parameters["read_scale_f32_bits"] = f32_bits(1.0 / std::sqrt(double(dim)));
+      bind(tensors, mix,
+           {{"read_projection", "q"},
+            {"key_projection", "k"},
+            {"value_projection", "v"},
+            {"gate_projection_mixer", "g"},
+            {"decay_down", "a1"},
+            {"decay_up", "a2"},
+            {"decay_base", "a2.b"},
+            {"output_norm", "norm"}});
+      program.block(kBlockGatedLinear, std::move(parameters), std::move(tensors));
+    } else {
+      throw std::runtime_error("mixer type is not supported: " + type);
+    }
+  }
+  program.head(kHeadBf16, {{"norm_epsilon_f32_bits", epsilon}},
+               {{"norm", "final.norm"}, {"weight", "head"}});
+  return model;
+}
+
+constexpr ModelDesign kDesigns[]{{"Zatupel", &describe_zatupel},
+                                 {"Nametar", &describe_nametar}};
 
 }  // namespace
 

@@ -95,7 +95,8 @@ class Q8AttentionLaunch(Structure):
 ELEMENT_BF16 = 0
 ELEMENT_F32 = 1
 LINEAR_STORE, LINEAR_ADD, LINEAR_GATED, LINEAR_PARTIALS = range(4)
-RECURRENCE_DELTA, RECURRENCE_BONUS = range(2)
+RECURRENCE_DELTA, RECURRENCE_BONUS, RECURRENCE_GATED = range(3)
+ATTENTION_GENERAL, ATTENTION_SPLIT, ATTENTION_PROMPT = range(3)
 
 
 class LinearSegment(Structure):
@@ -116,7 +117,9 @@ class StreamNormLaunch(Structure):
                 ("weight", c_void_p * 2), ("output", c_void_p * 2),
                 ("stride", c_uint32 * 2), ("rows", c_uint32), ("width", c_uint32),
                 ("epsilon", c_float), ("element", c_uint32),
-                ("shift", POINTER(TokenShift)), ("gather", c_void_p), ("step", c_void_p)]
+                ("shift", POINTER(TokenShift)), ("gather", c_void_p), ("step", c_void_p),
+                ("branch_weight", c_void_p), ("branch_scale", c_float),
+                ("branch_epsilon", c_float)]
 
 
 class WindowedAttention(Structure):
@@ -144,6 +147,33 @@ class AttentionLaunch(Structure):
                 ("workspace_bytes", c_size_t)]
 
 
+class LatentAttention(Structure):
+    _fields_ = [("heads", c_uint32), ("dim", c_uint32), ("vdim", c_uint32),
+                ("rank", c_uint32), ("rot_dim", c_uint32), ("rotary_dims", c_uint32),
+                ("window", c_uint32), ("scale", c_float), ("epsilon", c_float),
+                ("rotary_magnitude", c_float), ("frequencies", c_void_p),
+                ("latent_norm", c_void_p), ("key_up", c_void_p),
+                ("key_up_transposed", c_void_p), ("value_up", c_void_p),
+                ("page_tokens", c_uint32), ("pages_per_slot", c_uint32),
+                ("layer_offset", c_uint64), ("page_table", c_void_p), ("step", c_void_p),
+                ("element", c_uint32)]
+
+
+class LatentStoreLaunch(Structure):
+    _fields_ = [("projections", c_void_p), ("stride", c_uint32),
+                ("latent_column", c_uint32), ("query_column", c_uint32),
+                ("query_rank", c_uint32), ("query_norm", c_void_p),
+                ("query_out", c_void_p), ("query_stride", c_uint32), ("rows", c_uint32)]
+
+
+class LatentLaunch(Structure):
+    _fields_ = [("query", c_void_p), ("query_stride", c_uint32), ("gate", c_void_p),
+                ("gate_stride", c_uint32), ("output", c_void_p),
+                ("output_stride", c_uint32), ("rows", c_uint32),
+                ("maximum_position", c_uint32), ("workspace", c_void_p),
+                ("workspace_bytes", c_size_t)]
+
+
 class Recurrence(Structure):
     _fields_ = [("kind", c_uint32), ("heads", c_uint32), ("dim", c_uint32),
                 ("rank", c_uint32), ("gate_kind", c_uint32), ("epsilon", c_float),
@@ -151,7 +181,7 @@ class Recurrence(Structure):
                 ("decay_up_bf16", c_void_p), ("decay_base", c_void_p),
                 ("rate_bias", c_void_p), ("bonus", c_void_p), ("norm_weight", c_void_p),
                 ("state", c_void_p), ("slot_stride", c_uint64), ("step", c_void_p),
-                ("element", c_uint32)]
+                ("element", c_uint32), ("vdim", c_uint32), ("read_scale", c_float)]
 
 
 class RecurrenceLaunch(Structure):
@@ -236,6 +266,7 @@ SIGNATURES = {
     "qllm_apply_presence_penalty_rows": (c_int32, [c_void_p, c_size_t, c_void_p, c_void_p, c_uint32, c_uint32, c_float, c_void_p]),
     "qllm_mark_presence": (c_int32, [c_void_p, c_void_p, c_uint32, c_uint32, c_void_p]),
     "qllm_linear_packed_bytes": (c_size_t, [c_uint32, c_uint32]),
+    "qllm_linear_pack_strided": (c_int32, [c_void_p, c_uint32, c_uint32, c_uint64, c_uint64, c_void_p, c_uint32, c_uint32, c_uint32, c_uint32, c_void_p]),
     "qllm_linear_pack": (c_int32, [c_void_p, c_uint32, c_uint32, c_void_p, c_uint32, c_uint32, c_uint32, c_uint32, c_void_p]),
     "qllm_linear_batch": (c_int32, [POINTER(LinearSegment), c_uint32, c_uint32, c_uint32, c_void_p]),
     "qllm_embedding_bf16_batch": (c_int32, [c_void_p, c_uint32, c_void_p, c_void_p, c_uint32, c_uint32, c_float, c_void_p]),
@@ -245,6 +276,11 @@ SIGNATURES = {
     "qllm_windowed_attention_workspace_bytes": (c_size_t, [POINTER(WindowedAttention), c_uint32, c_uint32]),
     "qllm_windowed_attention_form": (c_uint32, [POINTER(WindowedAttention), c_uint32]),
     "qllm_windowed_attention_rows": (c_int32, [POINTER(WindowedAttention), POINTER(AttentionLaunch), c_void_p]),
+    "qllm_latent_layer_bytes": (c_size_t, [c_uint32, c_uint32, c_uint32, c_uint32]),
+    "qllm_latent_store": (c_int32, [POINTER(LatentAttention), POINTER(LatentStoreLaunch), c_void_p]),
+    "qllm_latent_attention_form": (c_uint32, [POINTER(LatentAttention), c_uint32]),
+    "qllm_latent_attention_workspace_bytes": (c_size_t, [POINTER(LatentAttention), c_uint32, c_uint32]),
+    "qllm_latent_attention_rows": (c_int32, [POINTER(LatentAttention), POINTER(LatentLaunch), c_void_p]),
     "qllm_recurrence_workspace_bytes": (c_size_t, [POINTER(Recurrence), c_uint32]),
     "qllm_recurrence_rows": (c_int32, [POINTER(Recurrence), POINTER(RecurrenceLaunch), c_void_p]),
     "qllm_fill_random": (c_int32, [c_void_p, c_size_t, c_uint32, c_uint64, c_void_p]),
