@@ -283,55 +283,97 @@ def measure_long_contexts(qp, np, rows):
 # Layers of about the size of a 1B and of a 7B model, four of them: attention,
 # generalised delta rule, bonus recurrence, attention.
 MIXED_SIZES = {
-    "width-2048": dict(width=2048, ff=5632, heads=16, kv_heads=4, recurrent_heads=32),
-    "width-4096": dict(width=4096, ff=14336, heads=32, kv_heads=8, recurrent_heads=64),
+    "width-2048": dict(width=2048, ff=5632, heads=16, kv_heads=4, recurrent_heads=32,
+                       query_rank=768),
+    "width-4096": dict(width=4096, ff=14336, heads=32, kv_heads=8, recurrent_heads=64,
+                       query_rank=1536),
 }
 MIXED_WINDOW, MIXED_KEPT, MIXED_VOCABULARY = 1024, 4, 32000
 
 
-def measure_mixed(qp, np, prompt_tokens, steps, warmup):
-    """Prefill and greedy decode of the mixed-layer decoder (bf16, random
-    weights) beside the dense FP4 decoder with as many layers of the same width,
-    feed-forward, heads and vocabulary.  Prefill: from the call to the token
-    after the prompt.  Decode: one token after the other through the program,
-    each read back by the host; the dense decoder's one-row target pass is
-    replayed back to back (its decode step is speculative).  Bytes are those of
+def measure_folder(qp, np, config, shapes, prompt_tokens, steps, warmup):
+    """Prefill and greedy decode of a model folder's design (bf16, random weights).
+    Prefill: from the call to the token after the prompt.  Decode: one token after
+    the other through the program, each read back by the host.  Bytes are those of
     the weights a token reads."""
     import shutil
     import tempfile
 
     import mixed_model as mm
 
+    folder = tempfile.mkdtemp()
+    try:
+        mm.write_folder(folder, config, mm.TiledWeights(shapes, 1))
+        model = qp.Model(folder, prompt_tokens + warmup + steps + 8, kv_page_tokens=256)
+    finally:
+        shutil.rmtree(folder, ignore_errors=True)
+    tokens = np.random.default_rng(0).integers(0, config["vocab"], prompt_tokens)
+    prefill = []
+    for _ in range(4):                   # the first one allocates and is not counted
+        request = model.begin()
+        begin = time.perf_counter()
+        _, token = model.step(request, tokens)
+        prefill.append(time.perf_counter() - begin)
+        if len(prefill) < 4:
+            model.end(request)
+    for index in range(warmup + steps):
+        if index == warmup:
+            begin = time.perf_counter()
+        _, token = model.step(request, [token])
+    decode = (time.perf_counter() - begin) / steps
+    read = model.telemetry("provider_weight_bytes") - 2 * config["vocab"] * config["width"]
+    model.close()
+    return {"prefill_tok_s": round(prompt_tokens / min(prefill[1:]), 1),
+            "prefill_ms": round(1e3 * min(prefill[1:]), 3),
+            "decode_tok_s": round(1.0 / decode, 1),
+            "decode_us_per_token": round(1e6 * decode, 1),
+            "decode_weight_GBps": round(read / decode / 1e9, 1)}
+
+
+def mixed_configuration(size):
+    import mixed_model as mm
+
+    attention = mm.attention(size["heads"], size["kv_heads"], 128, 128, MIXED_WINDOW,
+                             MIXED_KEPT)
+    layers = [attention, mm.general_delta(size["recurrent_heads"], 64),
+              mm.wkv(size["recurrent_heads"], 64), attention]
+    config = mm.configuration(MIXED_VOCABULARY, size["width"], layers, [size["ff"]] * 4)
+    return config, mm.shapes(config, 64)
+
+
+def latent_configuration(size):
+    import latent_model as lm
+
+    windowed = lm.windowed_latent(size["heads"], 128, 64, 128, 512, size["query_rank"],
+                                  MIXED_WINDOW, scaling=lm.yarn(8.0, 4096))
+    recurrent = lm.gla(size["recurrent_heads"] // 2, 64, 128)
+    layers = [recurrent, windowed, lm.latent(size["heads"], 128, 128, 512), windowed]
+    config = lm.configuration(MIXED_VOCABULARY, size["width"], layers, [size["ff"]] * 4)
+    return config, lm.shapes(config, 64)
+
+
+def measure_latent(qp, np, prompt_tokens, steps, warmup):
+    """The latent-attention decoder beside the mixed-layer decoder with as many
+    layers of the same width, feed-forward, heads, state size and vocabulary."""
     report = {}
     for name, size in MIXED_SIZES.items():
-        attention = mm.attention(size["heads"], size["kv_heads"], 128, 128, MIXED_WINDOW,
-                                 MIXED_KEPT)
-        layers = [attention, mm.general_delta(size["recurrent_heads"], 64),
-                  mm.wkv(size["recurrent_heads"], 64), attention]
-        config = mm.configuration(MIXED_VOCABULARY, size["width"], layers, [size["ff"]] * 4)
-        folder = tempfile.mkdtemp()
-        try:
-            mm.write_folder(folder, config, mm.TiledWeights(config, 1))
-            model = qp.Model(folder, prompt_tokens + warmup + steps + 8, kv_page_tokens=256)
-        finally:
-            shutil.rmtree(folder, ignore_errors=True)
-        tokens = np.random.default_rng(0).integers(0, MIXED_VOCABULARY, prompt_tokens)
-        prefill = []
-        for _ in range(4):               # the first one allocates and is not counted
-            request = model.begin()
-            begin = time.perf_counter()
-            _, token = model.step(request, tokens)
-            prefill.append(time.perf_counter() - begin)
-            if len(prefill) < 4:
-                model.end(request)
-        for index in range(warmup + steps):
-            if index == warmup:
-                begin = time.perf_counter()
-            _, token = model.step(request, [token])
-        decode = (time.perf_counter() - begin) / steps
-        read = model.telemetry("provider_weight_bytes") - 2 * MIXED_VOCABULARY * size["width"]
-        model.close()
+        report[name] = measure_folder(qp, np, *latent_configuration(size), prompt_tokens,
+                                      steps, warmup)
+        other = measure_folder(qp, np, *mixed_configuration(size), prompt_tokens, steps,
+                               warmup)
+        report[name].update({"mixed_" + key: value for key, value in other.items()})
+    return report
 
+
+def measure_mixed(qp, np, prompt_tokens, steps, warmup):
+    """The mixed-layer decoder beside the dense FP4 decoder with as many layers of
+    the same width, feed-forward, heads and vocabulary.  The dense decoder's one-row
+    target pass is replayed back to back (its decode step is speculative)."""
+    report = {}
+    for name, size in MIXED_SIZES.items():
+        report[name] = measure_folder(qp, np, *mixed_configuration(size), prompt_tokens,
+                                      steps, warmup)
+        tokens = np.random.default_rng(0).integers(0, MIXED_VOCABULARY, prompt_tokens)
         geometry = dict(MODEL)
         geometry.update(hidden=size["width"], intermediate=size["ff"], layers=4,
                         query_heads=size["heads"], kv_heads=size["kv_heads"],
@@ -355,16 +397,11 @@ def measure_mixed(qp, np, prompt_tokens, steps, warmup):
         dense.synchronize_stream()
         dense_decode = (time.perf_counter() - begin) / steps
         dense.close()
-        report[name] = {
-            "prefill_tok_s": round(prompt_tokens / min(prefill[1:]), 1),
-            "prefill_ms": round(1e3 * min(prefill[1:]), 3),
-            "decode_tok_s": round(1.0 / decode, 1),
-            "decode_us_per_token": round(1e6 * decode, 1),
-            "decode_weight_GBps": round(read / decode / 1e9, 1),
+        report[name].update({
             "dense_fp4_prefill_tok_s": round(prompt_tokens / min(dense_prefill[1:]), 1),
             "dense_fp4_prefill_ms": round(1e3 * min(dense_prefill[1:]), 3),
             "dense_fp4_one_row_pass_us": round(1e6 * dense_decode, 1),
-        }
+        })
     return report
 
 
@@ -393,7 +430,12 @@ def main():
                         help="measure the mixed-layer decoder (prefill and decode at "
                              "two sizes, beside the dense decoder) instead of the "
                              "verify step")
-    parser.add_argument("--mixed-prompt-tokens", type=int, default=4096)
+    parser.add_argument("--latent", action="store_true",
+                        help="measure the latent-attention decoder (prefill and decode "
+                             "at two sizes, beside the mixed-layer decoder) instead of "
+                             "the verify step")
+    parser.add_argument("--mixed-prompt-tokens", type=int, default=4096,
+                        help="prompt length of --mixed and --latent")
     parser.add_argument("--calibration-copy", action="store_true",
                         help="also run one 256 MiB device copy (a kernel of known "
                              "traffic to scale hardware counters by)")
@@ -414,16 +456,19 @@ def main():
         return 1
     rows = MODEL["draft_depth"] + 1
     steps, warmup = arguments.steps, arguments.warmup
-    if arguments.mixed:
-        report = measure_mixed(qp, np, arguments.mixed_prompt_tokens, steps, warmup)
+    if arguments.mixed or arguments.latent:
+        measure, kind, design = ((measure_latent, "latent-attention", "Nametar")
+                                 if arguments.latent else
+                                 (measure_mixed, "mixed-layer", "Zatupel"))
+        report = measure(qp, np, arguments.mixed_prompt_tokens, steps, warmup)
         first = report["width-2048"]
         print(json.dumps({
-            "metric": "mixed-layer decoder decode tok/s", "value": first["decode_tok_s"],
+            "metric": kind + " decoder decode tok/s", "value": first["decode_tok_s"],
             "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
             "ms_per_step": round(first["decode_us_per_token"] / 1e3, 4),
             "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
             "dtype": "bf16", "data": "synthetic", "sizes": report,
-            "config": {"model": "Zatupel-shaped, 4 layers, random weights",
+            "config": {"model": design + "-shaped, 4 layers, random weights",
                        "global_batch": 1, "seq_len": arguments.mixed_prompt_tokens,
                        "parallelism": "none"}}))
         return 0
