@@ -26,8 +26,8 @@ namespace {
 constexpr uint32_t kTile = 32;               // tokens
 constexpr uint32_t kFragment = 512;          // elements, 16 x 32
 constexpr uint32_t kSplitRows = 32;          // rows of the split form
-constexpr uint32_t kMaximumSplits = 128;
-constexpr uint32_t kMaximumLds = 160u * 1024u;
+constexpr uint32_t kMaximumSplits = 64;       // a lane each when the parts are added
+constexpr uint32_t kValueThreads = 1024;
 constexpr float kLog2e = 1.4426950408889634f;
 
 using Latent = qllm_latent_attention;
@@ -60,13 +60,21 @@ __device__ __forceinline__ bool visible(const Latent& a, uint32_t position, uint
   return key <= position && (!a.window || position - key < a.window);
 }
 
-// Fragments of the 16 tokens that start at `token`.
+// The request's row of the page table, and the fragments of the 16 tokens that
+// start at `token`.
+__device__ __forceinline__ void* const* pages_of(const Latent& a) {
+  return a.page_table + size_t{a.step[kStepSlot]} * a.pages_per_slot;
+}
 template <typename T>
-__device__ __forceinline__ T* cache_block(const Latent& a, uint32_t token) {
-  void* const page =
-      a.page_table[size_t{a.step[kStepSlot]} * a.pages_per_slot + token / a.page_tokens];
+__device__ __forceinline__ T* cache_block(const Latent& a, void* const* pages,
+                                          uint32_t token) {
+  void* const page = pages[token / a.page_tokens];
   return reinterpret_cast<T*>(static_cast<uint8_t*>(page) + a.layer_offset) +
          size_t{token % a.page_tokens / 16u} * row_chunks(a) * kFragment;
+}
+template <typename T>
+__device__ __forceinline__ T* cache_block(const Latent& a, uint32_t token) {
+  return cache_block<T>(a, pages_of(a), token);
 }
 
 // Value d of a rotated vector x (its dimensions from rotary_dims on stay).
@@ -95,17 +103,14 @@ struct StoreArgs {
   qllm_latent_store_launch launch;
 };
 
-// A wave per row and task: the cache row, or the query latent.
+// A workgroup per row and task: the cache row, or the query latent.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_store_kernel(StoreArgs args) {
+  __shared__ float scratch[16];
   const Latent& a = args.attention;
   const auto& run = args.launch;
-  const uint32_t tasks = run.query_rank ? 2u : 1u;
-  const uint32_t item = blockIdx.x * 4u + threadIdx.x / kWave;
-  const uint32_t lane = threadIdx.x % kWave;
-  if (item >= run.rows * tasks) return;
-  const uint32_t row = item / tasks;
-  const bool query = item % tasks == 1u;
+  const uint32_t row = blockIdx.x;
+  const bool query = blockIdx.y == 1u;
   const float* source = run.projections + size_t{row} * run.stride +
                         (query ? run.query_column : run.latent_column);
   const uint32_t rank = query ? run.query_rank : a.rank;
@@ -115,43 +120,47 @@ __global__ __launch_bounds__(256) void latent_store_kernel(StoreArgs args) {
   float squares = 0.0f;
 #pragma unroll
   for (uint32_t i = 0; i < kHeld; ++i) {
-    const uint32_t d = i * kWave + lane;
+    const uint32_t d = i * blockDim.x + threadIdx.x;
     held[i] = d < rank ? source[d] : 0.0f;
     weight[i] = d < rank ? norm[d] : 0.0f;
   }
+  const uint32_t position = a.step[kStepPosition] + row;
+  T* const block = cache_block<T>(a, position);
+  const uint32_t n = position % 16u;
+  if (!query) {
+    // threads from the far end: the latent's own fall to the first ones
+    const uint32_t d = blockDim.x - 1u - threadIdx.x;
+    T* const shared = block + size_t{chunks_of(a.rank)} * kFragment;
+    for (uint32_t at = d; at < chunks_of(a.rot_dim) * 32u; at += blockDim.x)
+      store_element(shared + size_t{at / 32u} * kFragment + in_fragment(n, at % 32u),
+                    at < a.rot_dim ? rotated(a, source + a.rank, at, position) : 0.0f);
+  }
 #pragma unroll
   for (uint32_t i = 0; i < kHeld; ++i) squares = fmaf(held[i], held[i], squares);
-  for (uint32_t d = kHeld * kWave + lane; d < rank; d += kWave)
+  for (uint32_t d = kHeld * blockDim.x + threadIdx.x; d < rank; d += blockDim.x)
     squares = fmaf(source[d], source[d], squares);
   const float inverse =
-      1.0f / sqrtf(wave_sum(squares) / static_cast<float>(rank) + a.epsilon);
+      1.0f / sqrtf(block_sum(squares, scratch) / static_cast<float>(rank) + a.epsilon);
   const auto put_all = [&](auto put, uint32_t padded) {
 #pragma unroll
     for (uint32_t i = 0; i < kHeld; ++i) {
-      const uint32_t d = i * kWave + lane;
+      const uint32_t d = i * blockDim.x + threadIdx.x;
       if (d < padded) put(d, held[i] * inverse * weight[i]);
     }
-    for (uint32_t d = kHeld * kWave + lane; d < padded; d += kWave)
+    for (uint32_t d = kHeld * blockDim.x + threadIdx.x; d < padded; d += blockDim.x)
       put(d, d < rank ? source[d] * inverse * norm[d] : 0.0f);
   };
   if (query) {
     T* out = static_cast<T*>(run.query_out) + size_t{row} * run.query_stride;
     put_all([&](uint32_t d, float value) { store_element(out + d, value); },
             run.query_stride);
-    return;
+  } else {
+    put_all(
+        [&](uint32_t d, float value) {
+          store_element(block + size_t{d / 32u} * kFragment + in_fragment(n, d % 32u), value);
+        },
+        chunks_of(a.rank) * 32u);
   }
-  const uint32_t position = a.step[kStepPosition] + row;
-  T* block = cache_block<T>(a, position);
-  const uint32_t n = position % 16u;
-  put_all(
-      [&](uint32_t d, float value) {
-        store_element(block + size_t{d / 32u} * kFragment + in_fragment(n, d % 32u), value);
-      },
-      chunks_of(a.rank) * 32u);
-  T* shared = block + size_t{chunks_of(a.rank)} * kFragment;
-  for (uint32_t d = lane; d < chunks_of(a.rot_dim) * 32u; d += kWave)
-    store_element(shared + size_t{d / 32u} * kFragment + in_fragment(n, d % 32u),
-                  d < a.rot_dim ? rotated(a, source + a.rank, d, position) : 0.0f);
 }
 
 struct AttentionArgs {
@@ -339,14 +348,13 @@ __global__ __launch_bounds__(256) void latent_prompt_query_kernel(AttentionArgs 
   const float* source = run.query + size_t{row} * run.query_stride + size_t{head} * width;
   uint16_t* out = args.query + size_t{item} * padded;
   const uint32_t position = a.step[kStepPosition] + row;
-  for (uint32_t d = lane; d < padded; d += kWave) {
-    float value = 0.0f;
-    if (d < a.dim)
-      value = source[d];
-    else if (d >= plain && d - plain < a.rot_dim)
-      value = rotated(a, source + a.dim, d - plain, position);
-    store_element(out + d, value);
-  }
+  const auto value = [&](uint32_t d) {
+    if (d < a.dim) return source[d];
+    return d >= plain && d - plain < a.rot_dim ? rotated(a, source + a.dim, d - plain, position)
+                                               : 0.0f;
+  };
+  for (uint32_t d = 2u * lane; d < padded; d += 2u * kWave)
+    *reinterpret_cast<uint32_t*>(out + d) = pack_bf16(value(d), value(d + 1u));
 }
 
 // ---- split form --------------------------------------------------------------------
@@ -395,11 +403,11 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
     const uint32_t c = wave + 4u * i;
     q[i] = c < chunks ? *reinterpret_cast<const i32x4*>(query + c * 32u) : i32x4{};
   }
-  i32x4 staged[kLoads];
+  void* const* const pages = pages_of(a);
   const uint32_t pieces = 2u * chunks * kWave;
-  const auto fetch = [&](uint32_t t) __attribute__((always_inline)) {
+  const auto fetch = [&](i32x4 (&staged)[kLoads], uint32_t t) __attribute__((always_inline)) {
     const i32x4* source =
-        reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(a, t * kTile));
+        reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(a, pages, t * kTile));
 #pragma unroll
     for (int i = 0; i < kLoads; ++i) {
       const uint32_t piece = i * 256u + threadIdx.x;
@@ -410,16 +418,15 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
   float maximum = -INFINITY;
   float total = 0.0f;
   f32x4 sum[R] = {};
-  uint32_t at = begin + blockIdx.x;
-  if (at < end) fetch(at);
-  for (; at < end; at += gridDim.x) {
+  // `staged` holds tile `at` and takes the one after next
+  const auto take = [&](i32x4 (&staged)[kLoads], uint32_t at) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < kLoads; ++i) {
       const uint32_t piece = i * 256u + threadIdx.x;
       if (piece < pieces) reinterpret_cast<i32x4*>(tile)[piece] = staged[i];
     }
     __syncthreads();
-    if (at + gridDim.x < end) fetch(at + gridDim.x);
+    if (at + 2u * gridDim.x < end) fetch(staged, at + 2u * gridDim.x);
     f32x4 s[2] = {};
 #pragma unroll
     for (int i = 0; i < kQuery; ++i) {
@@ -477,6 +484,17 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
       sum[j] = mfma_bf16(i32x4{left[0], left[1], right[0], right[1]}, weights, sum[j]);
     }
     __syncthreads();
+  };
+  i32x4 even[kLoads], odd[kLoads];
+  uint32_t next = begin + blockIdx.x;
+  if (next < end) fetch(even, next);
+  if (next + gridDim.x < end) fetch(odd, next + gridDim.x);
+  while (next < end) {
+    take(even, next);
+    next += gridDim.x;
+    if (next >= end) break;
+    take(odd, next);
+    next += gridDim.x;
   }
   if (item >= items) return;
   total += __shfl_xor(total, 16, kWave);
@@ -495,94 +513,136 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
   }
 }
 
+// Groups of threads that add the parts, a thread four latent values.
+__host__ __device__ __forceinline__ uint32_t value_groups(const Latent& a) {
+  return kValueThreads / (chunks_of(a.rank) * 8u);
+}
+
+// Their sums in LDS, later the sums that cross from wave to wave.
+__host__ __device__ __forceinline__ uint32_t added_quads(const Latent& a) {
+  const uint32_t groups = value_groups(a) > 16u ? value_groups(a) : 16u;
+  const uint32_t quads = groups * chunks_of(a.rank) * 8u;
+  return quads > kValueThreads ? quads : kValueThreads;
+}
+
 // The parts of one head and up to 16 rows added, then through the value map: a
-// wave per 16 values.
-__global__ __launch_bounds__(256) void latent_value_kernel(AttentionArgs args) {
-  extern __shared__ float dynamic[];
+// wave per 16 values and half of the latent.
+__global__ __launch_bounds__(kValueThreads) void latent_value_kernel(AttentionArgs args) {
+  extern __shared__ f32x4 dynamic[];
+  __shared__ float share[16][kMaximumSplits];
   const Latent& a = args.attention;
   const auto& run = args.launch;
-  const uint32_t head = blockIdx.y;
-  const uint32_t row0 = blockIdx.z * 16u;
+  const uint32_t head = blockIdx.x;
+  const uint32_t row0 = blockIdx.y * 16u;
   const uint32_t rows = min(16u, run.rows - row0);
   const uint32_t items = run.rows * a.heads;
   const uint32_t latent = chunks_of(a.rank) * 32u;
+  const uint32_t quads = latent / 4u;
   const uint32_t stride = latent + 8u;                        // LDS row, elements
-  float* share = dynamic;                                     // [rows][splits]
-  uint16_t* mean = reinterpret_cast<uint16_t*>(share + 16u * args.splits);   // [16][stride]
+  const uint32_t groups = value_groups(a);
+  f32x4* const added = dynamic;                               // [row][part][quads]
+  uint16_t* const mean =
+      reinterpret_cast<uint16_t*>(added + added_quads(a));         // [16][stride]
   const uint32_t wave = threadIdx.x / kWave;
   const uint32_t lane = threadIdx.x % kWave;
-  for (uint32_t row = wave; row < 16u; row += 4u) {
-    if (row >= rows) break;
-    const uint32_t item = (row0 + row) * a.heads + head;
-    float m[kMaximumSplits / kWave], t[kMaximumSplits / kWave];
-    float top = -INFINITY;
-#pragma unroll
-    for (uint32_t i = 0; i < kMaximumSplits / kWave; ++i) {
-      const uint32_t split = i * kWave + lane;
-      const float* pair = args.maxima + (size_t{split} * items + item) * 2u;
-      m[i] = split < args.splits ? pair[0] : -INFINITY;
-      t[i] = split < args.splits ? pair[1] : 0.0f;
-      top = fmaxf(top, m[i]);
-    }
-    top = wave_max(top);
-    float total = 0.0f;
-#pragma unroll
-    for (uint32_t i = 0; i < kMaximumSplits / kWave; ++i) {
-      m[i] = __builtin_amdgcn_exp2f(m[i] - top);
-      total = fmaf(m[i], t[i], total);
-    }
-    total = wave_sum(total);
-#pragma unroll
-    for (uint32_t i = 0; i < kMaximumSplits / kWave; ++i) {
-      const uint32_t split = i * kWave + lane;
-      if (split < args.splits) share[row * args.splits + split] = m[i] / total;
-    }
-  }
-  __syncthreads();
-  for (uint32_t i = threadIdx.x; i < 16u * latent; i += blockDim.x) {
-    const uint32_t row = i / latent;
-    const uint32_t r = i % latent;
-    float value = 0.0f;
-    if (row < rows) {
-      const float* part = args.sums + size_t{(row0 + row) * a.heads + head} * latent + r;
-      const float* weight = share + row * args.splits;
-      for (uint32_t first = 0; first < args.splits; first += 8u) {
-        float piece[8];
-        // a part whose weight is zero may never have been written
-#pragma unroll
-        for (uint32_t s = 0; s < 8u; ++s) {
-          const bool there = first + s < args.splits && weight[min(first + s, args.splits - 1u)] > 0.0f;
-          piece[s] = there ? part[size_t{first + s} * items * latent] * weight[first + s] : 0.0f;
-        }
-#pragma unroll
-        for (uint32_t s = 0; s < 8u; ++s) value += piece[s];
-      }
-    }
-    store_element(mean + row * stride + r, value);
-  }
-  __syncthreads();
-  const uint32_t tile = blockIdx.x * 4u + wave;
-  if (tile >= value_tiles(a)) return;
+
+  // this wave's first weights, on their way meanwhile
   const uint32_t column = lane % 16u;
   const uint32_t quarter = lane / 16u;
   const uint32_t chunks = packed_chunks(a.rank);
-  const i32x4* weights = static_cast<const i32x4*>(a.value_up) +
-                         (size_t{head} * value_tiles(a) + tile) * chunks * kWave + lane;
-  f32x4 sum = {};
-#pragma unroll 4
-  for (uint32_t c = 0; c < chunks_of(a.rank); ++c)
-    sum = mfma_bf16(weights[c * kWave],
-                    *reinterpret_cast<const i32x4*>(mean + column * stride + c * 32u +
-                                                    8u * quarter),
-                    sum);
-  if (column >= rows) return;
-  const uint32_t row = row0 + column;
-  for (uint32_t i = 0; i < 4u; ++i) {
-    const uint32_t n = tile * 16u + 4u * quarter + i;
-    if (n >= a.vdim) break;
-    const uint32_t at = head * a.vdim + n;
-    store_element(static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride + at,
-                  sum[i] * gate_of(run, row, at));
+  const uint32_t half_chunks = (chunks_of(a.rank) + 1u) / 2u;
+  const uint32_t units = value_tiles(a) * 2u;
+  constexpr uint32_t kAhead = 8;
+  i32x4 ahead[kAhead];
+  const auto weights_of = [&](uint32_t unit) {
+    return static_cast<const i32x4*>(a.value_up) +
+           ((size_t{head} * value_tiles(a) + unit / 2u) * chunks + unit % 2u * half_chunks) *
+               kWave + lane;
+  };
+  const auto count_of = [&](uint32_t unit) {
+    return unit % 2u ? chunks_of(a.rank) - half_chunks : half_chunks;
+  };
+  if (wave < units)
+#pragma unroll
+    for (uint32_t c = 0; c < kAhead; ++c)
+      if (c < count_of(wave)) ahead[c] = weights_of(wave)[c * kWave];
+
+  if (wave < rows) {
+    const uint32_t item = (row0 + wave) * a.heads + head;
+    const float* pair = args.maxima + (size_t{min(lane, args.splits - 1u)} * items + item) * 2u;
+    const float m = lane < args.splits ? pair[0] : -INFINITY;
+    const float t = lane < args.splits ? pair[1] : 0.0f;
+    const float factor = __builtin_amdgcn_exp2f(m - wave_max(m));
+    share[wave][lane] = factor / wave_sum(factor * t);
+  }
+  __syncthreads();
+  // a row's parts over as many groups as there are; every group a row if not
+  const uint32_t per_row = max(groups / rows, 1u);
+  const uint32_t group = threadIdx.x / quads;
+  const uint32_t quad = threadIdx.x % quads;
+  if (group < groups)
+    for (uint32_t row = group / per_row; row < rows; row += groups / per_row) {
+      const uint32_t mine = group % per_row;
+      const f32x4* part = reinterpret_cast<const f32x4*>(args.sums) +
+                          size_t{(row0 + row) * a.heads + head} * quads + quad;
+      f32x4 sum = {};
+      for (uint32_t first = mine; first < args.splits; first += 8u * per_row) {
+        f32x4 piece[8];
+        // a part whose share is zero may never have been written
+#pragma unroll
+        for (uint32_t s = 0; s < 8u; ++s) {
+          const uint32_t split = first + s * per_row;
+          const float weight = split < args.splits ? share[row][split] : 0.0f;
+          piece[s] = weight > 0.0f ? part[size_t{split} * items * quads] * weight : f32x4{};
+        }
+#pragma unroll
+        for (uint32_t s = 0; s < 8u; ++s) sum += piece[s];
+      }
+      added[(row * per_row + mine) * quads + quad] = sum;
+    }
+  __syncthreads();
+  for (uint32_t i = threadIdx.x; i < 16u * quads; i += blockDim.x) {
+    const uint32_t row = i / quads;
+    const uint32_t at = i % quads;
+    f32x4 sum = {};
+    if (row < rows)
+      for (uint32_t p = 0; p < per_row; ++p) sum += added[(row * per_row + p) * quads + at];
+    *reinterpret_cast<i32x2*>(mean + row * stride + at * 4u) =
+        i32x2{static_cast<int>(pack_bf16(sum[0], sum[1])),
+              static_cast<int>(pack_bf16(sum[2], sum[3]))};
+  }
+  __syncthreads();
+  for (uint32_t base = 0; base < units; base += kValueThreads / kWave) {
+    const uint32_t unit = base + wave;
+    f32x4 sum = {};
+    if (unit < units) {
+      const uint16_t* operand =
+          mean + column * stride + unit % 2u * half_chunks * 32u + 8u * quarter;
+      const uint32_t count = count_of(unit);
+#pragma unroll
+      for (uint32_t c = 0; c < kAhead; ++c) {
+        if (c >= count) continue;
+        const i32x4 w = base ? weights_of(unit)[c * kWave] : ahead[c];
+        sum = mfma_bf16(w, *reinterpret_cast<const i32x4*>(operand + c * 32u), sum);
+      }
+      for (uint32_t c = kAhead; c < count; ++c)
+        sum = mfma_bf16(weights_of(unit)[c * kWave],
+                        *reinterpret_cast<const i32x4*>(operand + c * 32u), sum);
+      if (unit % 2u) added[wave * kWave + lane] = sum;
+    }
+    __syncthreads();
+    if (unit < units && unit % 2u == 0u && column < rows) {
+      sum += added[(wave + 1u) * kWave + lane];
+      const uint32_t row = row0 + column;
+      for (uint32_t i = 0; i < 4u; ++i) {
+        const uint32_t n = unit / 2u * 16u + 4u * quarter + i;
+        if (n >= a.vdim) break;
+        const uint32_t at = head * a.vdim + n;
+        store_element(static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride + at,
+                      sum[i] * gate_of(run, row, at));
+      }
+    }
+    __syncthreads();
   }
 }
 
@@ -699,14 +759,16 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
   const uint32_t lane = threadIdx.x % kWave;
   const uint32_t column = lane % 16u;
   const uint32_t quarter = lane / 16u;
-  // contiguous ranges of (head, row block) per XCD; long rows first
+  // contiguous ranges of (head, row block) per XCD; the longest blocks of one head
+  // beside the shortest of the next
   const uint32_t row_blocks = (run.rows + kPromptRows - 1u) / kPromptRows;
   const uint32_t per_xcd = gridDim.x / 8u;
   const uint32_t work = blockIdx.x < per_xcd * 8u
                             ? blockIdx.x % 8u * per_xcd + blockIdx.x / 8u
                             : blockIdx.x;
   const uint32_t head = work / row_blocks;
-  const uint32_t block0 = (row_blocks - 1u - work % row_blocks) * kPromptRows;
+  const uint32_t ordinal = work % row_blocks;
+  const uint32_t block0 = (head % 2u ? ordinal : row_blocks - 1u - ordinal) * kPromptRows;
   const uint32_t row0 = block0 + wave * 16u * MT;         // of this wave
   const uint32_t first = a.step[kStepPosition];
   const uint32_t dim_chunks = chunks_of(a.dim);
@@ -737,15 +799,17 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
   __syncthreads();   // what no load reaches is zero
 
   // fragment f of a tile: half, key chunk; then value tiles
-  i32x4 loads[kLoads];
-  const auto fetch = [&](uint32_t tile) __attribute__((always_inline)) {
+  void* const* const pages = pages_of(a);
+  const auto fetch = [&](i32x4 (&loads)[kLoads], uint32_t tile) __attribute__((always_inline)) {
     const size_t place = size_t{head} * args.tiles + (tile - args.tile0);
     const i32x4* keys =
         reinterpret_cast<const i32x4*>(args.keys + place * 2u * dim_chunks * kFragment);
     const i32x4* values =
         reinterpret_cast<const i32x4*>(args.values + place * tiles_v * kFragment);
     const i32x4* cached =
-        reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(a, tile * kTile));
+        rot_chunks
+            ? reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(a, pages, tile * kTile))
+            : nullptr;
 #pragma unroll
     for (int i = 0; i < kLoads; ++i) {
       const uint32_t f = wave + 4u * i;
@@ -762,7 +826,8 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
       }
     }
   };
-  const auto publish = [&](uint32_t slot) __attribute__((always_inline)) {
+  const auto publish = [&](const i32x4 (&loads)[kLoads], uint32_t slot)
+      __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < kLoads; ++i) {
       const uint32_t f = wave + 4u * i;
@@ -771,89 +836,106 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
     }
   };
   const float unit = a.scale * kLog2e;
-  float maximum[MT], total[MT];
+  // weights are taken relative to `base`, a maximum that may be out of date by
+  // kSlack (a factor of 2^kSlack at most); it starts below every score
+  constexpr float kSlack = 8.0f;
+  float base[MT], total[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
-    maximum[m] = -INFINITY;
+    base[m] = -INFINITY;
     total[m] = 0.0f;
   }
   f32x4 out[MT][NV] = {};
   const uint32_t wave_first = first + row0;
   const uint32_t wave_last = first + min(row0 + 16u * MT, run.rows) - 1u;
   const bool idle = row0 >= run.rows;
-  fetch(begin);
-  publish(0u);
-  __syncthreads();
-  for (uint32_t tile = begin; tile < end; ++tile) {
+  const auto compute = [&](uint32_t tile) __attribute__((always_inline)) {
     const uint32_t slot = (tile - begin) & 1u;
-    if (tile + 1u < end) fetch(tile + 1u);
     const uint32_t key0 = tile * kTile;
-    // some row of the wave sees some key
-    const bool useful = !idle && key0 <= wave_last &&
-                        (!a.window || key0 + kTile - 1u + a.window > wave_first);
-    if (useful) {
-      const bool open = key0 + kTile - 1u <= wave_first &&
-                        (!a.window || wave_last - key0 < a.window);
-      f32x4 s[MT][2] = {};
+    // no row of the wave sees any key
+    if (idle || key0 > wave_last || (a.window && key0 + kTile - 1u + a.window <= wave_first))
+      return;
+    const bool open =
+        key0 + kTile - 1u <= wave_first && (!a.window || wave_last - key0 < a.window);
+    f32x4 s[MT][2] = {};
+#pragma unroll
+    for (int c = 0; c < NK; ++c)
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        const i32x4 k = staged[slot][(half * NK + c) * kWave + lane];
+#pragma unroll
+        for (int m = 0; m < MT; ++m) s[m][half] = mfma_bf16(k, q[m][c], s[m][half]);
+      }
+    float top[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+#pragma unroll
+      for (int half = 0; half < 2; ++half) s[m][half] *= unit;
+      if (!open) {
+        const uint32_t position = wave_first + m * 16u + column;
+#pragma unroll
+        for (int half = 0; half < 2; ++half)
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (!visible(a, position, key0 + half * 16u + 4u * quarter + i))
+              s[m][half][i] = -INFINITY;
+      }
+      top[m] = fmaxf(fmaxf(fmaxf(s[m][0][0], s[m][0][1]), fmaxf(s[m][0][2], s[m][0][3])),
+                     fmaxf(fmaxf(s[m][1][0], s[m][1][1]), fmaxf(s[m][1][2], s[m][1][3])));
+    }
+    i32x4 weights[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      if (__any(top[m] > base[m] + kSlack)) {
+        float fresh = fmaxf(top[m], __shfl_xor(top[m], 16, kWave));
+        fresh = fmaxf(fresh, __shfl_xor(fresh, 32, kWave));
+        fresh = fmaxf(fresh, base[m]);
+        // a row that has seen nothing yet keeps its sums, which are zero
+        const float fade =
+            base[m] == -INFINITY ? 0.0f : __builtin_amdgcn_exp2f(base[m] - fresh);
+        base[m] = fresh;
+        total[m] *= fade;
+#pragma unroll
+        for (int t = 0; t < NV; ++t) out[m][t] *= fade;
+      }
+      const float offset = base[m] == -INFINITY ? 0.0f : base[m];
+      float fresh = 0.0f;
 #pragma unroll
       for (int half = 0; half < 2; ++half)
 #pragma unroll
-        for (int c = 0; c < NK; ++c) {
-          const i32x4 k = staged[slot][(half * NK + c) * kWave + lane];
-#pragma unroll
-          for (int m = 0; m < MT; ++m) s[m][half] = mfma_bf16(k, q[m][c], s[m][half]);
+        for (int i = 0; i < 4; ++i) {
+          s[m][half][i] = __builtin_amdgcn_exp2f(s[m][half][i] - offset);
+          fresh += s[m][half][i];
         }
-      i32x4 weights[MT];
-      float fade[MT];
-#pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        const uint32_t position = wave_first + m * 16u + column;
-        float top = maximum[m];
-#pragma unroll
-        for (int half = 0; half < 2; ++half)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            float value = s[m][half][i] * unit;
-            if (!open && !visible(a, position, key0 + half * 16u + 4u * quarter + i))
-              value = -INFINITY;
-            s[m][half][i] = value;
-            top = fmaxf(top, value);
-          }
-        top = fmaxf(top, __shfl_xor(top, 16, kWave));
-        top = fmaxf(top, __shfl_xor(top, 32, kWave));
-        // a row that has seen nothing yet: keep the exponents' argument finite
-        const float base = top == -INFINITY ? 0.0f : top;
-        fade[m] = __builtin_amdgcn_exp2f(maximum[m] - base);
-        maximum[m] = top;
-        float fresh = 0.0f;
-#pragma unroll
-        for (int half = 0; half < 2; ++half)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            s[m][half][i] = __builtin_amdgcn_exp2f(s[m][half][i] - base);
-            fresh += s[m][half][i];
-          }
-        total[m] = fmaf(total[m], fade[m], fresh);
-        weights[m] = i32x4{static_cast<int>(pack_bf16(s[m][0][0], s[m][0][1])),
-                           static_cast<int>(pack_bf16(s[m][0][2], s[m][0][3])),
-                           static_cast<int>(pack_bf16(s[m][1][0], s[m][1][1])),
-                           static_cast<int>(pack_bf16(s[m][1][2], s[m][1][3]))};
-      }
-      // sums shrink only where a maximum has grown
-#pragma unroll
-      for (int m = 0; m < MT; ++m)
-        if (__any(fade[m] != 1.0f))
-#pragma unroll
-          for (int t = 0; t < NV; ++t) out[m][t] *= fade[m];
-#pragma unroll
-      for (int t = 0; t < NV; ++t) {
-        const i32x4 v = staged[slot][(2 * NK + t) * kWave + lane];
-#pragma unroll
-        for (int m = 0; m < MT; ++m) out[m][t] = mfma_bf16(v, weights[m], out[m][t]);
-      }
+      total[m] += fresh;
+      weights[m] = i32x4{static_cast<int>(pack_bf16(s[m][0][0], s[m][0][1])),
+                         static_cast<int>(pack_bf16(s[m][0][2], s[m][0][3])),
+                         static_cast<int>(pack_bf16(s[m][1][0], s[m][1][1])),
+                         static_cast<int>(pack_bf16(s[m][1][2], s[m][1][3]))};
     }
-    if (tile + 1u < end) publish(1u - slot);
+#pragma unroll
+    for (int t = 0; t < NV; ++t) {
+      const i32x4 v = staged[slot][(2 * NK + t) * kWave + lane];
+#pragma unroll
+      for (int m = 0; m < MT; ++m) out[m][t] = mfma_bf16(v, weights[m], out[m][t]);
+    }
+  };
+  // a tile is fetched two iterations and published one before its turn
+  i32x4 even[kLoads], odd[kLoads];
+  fetch(even, begin);
+  if (begin + 1u < end) fetch(odd, begin + 1u);
+  publish(even, 0u);
+  if (begin + 2u < end) fetch(even, begin + 2u);
+  __syncthreads();
+  const auto turn = [&](i32x4 (&loads)[kLoads], uint32_t tile) __attribute__((always_inline)) {
+    compute(tile);
+    if (tile + 1u < end) publish(loads, (tile + 1u - begin) & 1u);
+    if (tile + 3u < end) fetch(loads, tile + 3u);
     __syncthreads();
+  };
+  for (uint32_t tile = begin; tile < end; tile += 2u) {
+    turn(odd, tile);
+    if (tile + 1u < end) turn(even, tile + 1u);
   }
   if (idle) return;
 #pragma unroll
@@ -936,8 +1018,8 @@ size_t general_bytes(const Latent& a) {
   return (size_t{a.dim} + a.rot_dim + 2u * a.rank + kTile) * 4u;
 }
 
-size_t value_bytes(const Latent& a, uint32_t splits) {
-  return size_t{16u} * splits * 4u + size_t{16u} * (chunks_of(a.rank) * 32u + 8u) * 2u;
+size_t value_bytes(const Latent& a) {
+  return size_t{added_quads(a)} * 16u + size_t{16u} * (chunks_of(a.rank) * 32u + 8u) * 2u;
 }
 
 }  // namespace
@@ -962,11 +1044,11 @@ extern "C" int32_t qllm_latent_store(const qllm_latent_attention* attention,
         launch->query_column + launch->query_rank > launch->stride)))
     return fail(QLLM_INVALID_ARGUMENT, "invalid latent store");
   const StoreArgs args{*attention, *launch};
-  const uint32_t items = launch->rows * (launch->query_rank ? 2u : 1u);
+  const dim3 grid(launch->rows, launch->query_rank ? 2u : 1u);
   if (attention->element == QLLM_ELEMENT_F32)
-    latent_store_kernel<float><<<(items + 3u) / 4u, 256, 0, as_stream(stream)>>>(args);
+    latent_store_kernel<float><<<grid, 256, 0, as_stream(stream)>>>(args);
   else
-    latent_store_kernel<uint16_t><<<(items + 3u) / 4u, 256, 0, as_stream(stream)>>>(args);
+    latent_store_kernel<uint16_t><<<grid, 256, 0, as_stream(stream)>>>(args);
   return launched("latent store");
 }
 
@@ -1071,7 +1153,7 @@ extern "C" int32_t qllm_latent_attention_rows(const qllm_latent_attention* atten
     latent_split_kernel<4><<<grid, 256, 0, hip_stream>>>(args);
   else
     latent_split_kernel<8><<<grid, 256, 0, hip_stream>>>(args);
-  latent_value_kernel<<<dim3((value_tiles(a) + 3u) / 4u, a.heads, row_tiles), 256,
-                        value_bytes(a, args.splits), hip_stream>>>(args);
+  latent_value_kernel<<<dim3(a.heads, row_tiles), kValueThreads, value_bytes(a),
+                        hip_stream>>>(args);
   return launched("latent split attention");
 }

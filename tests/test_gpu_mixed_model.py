@@ -10,11 +10,9 @@ import mixed_model as mm
 import mixer_oracle as mo
 import qllm_provider as qp
 import worker_client as wc
+from model_util import LIMIT, Case, continuation, distance, feed
 
 pytestmark = pytest.mark.gpu
-
-# differences of logits: root mean square over root mean square
-LIMIT = {"fp32": 2e-5, "bf16": 2.5e-2}
 
 
 def configurations():
@@ -43,44 +41,19 @@ def configurations():
 CONFIGS = configurations()
 
 
-class Case:
-    def __init__(self, name, folder, tokens=210):
-        self.config = CONFIGS[name]
-        self.weights = mm.random_weights(self.config, 11)
-        self.path = mm.write_folder(folder, self.config, self.weights)
-        rng = np.random.default_rng(4)
-        self.tokens = rng.integers(0, self.config["vocab"], tokens)
-        self.logits, self.streams = mo.forward(self.config, mm.float64(self.weights),
-                                               self.tokens)
+def case_of(name, folder):
+    config = CONFIGS[name]
+    return Case(config, mm.random_weights(config, 11), mo.forward, folder)
 
 
 @pytest.fixture(scope="module", params=list(CONFIGS))
 def case(request, tmp_path_factory):
-    return Case(request.param, tmp_path_factory.mktemp(request.param))
+    return case_of(request.param, tmp_path_factory.mktemp(request.param))
 
 
 @pytest.fixture(scope="module")
 def mixed(tmp_path_factory):
-    return Case("mixed", tmp_path_factory.mktemp("one"))
-
-
-def distance(got, want):
-    got, want = np.asarray(got, np.float64), np.asarray(want, np.float64)
-    return np.sqrt(np.mean((got - want) ** 2, axis=-1) / np.mean(want ** 2))
-
-
-def feed(model, request, tokens, counts):
-    """Logits of every position, the tokens cut into portions of these sizes
-    (the last one repeated)."""
-    out, at = [], 0
-    for index in range(len(tokens)):
-        count = min(counts[min(index, len(counts) - 1)], len(tokens) - at)
-        logits, _ = model.step(request, tokens[at:at + count], range(count))
-        out.append(logits)
-        at += count
-        if at == len(tokens):
-            break
-    return np.concatenate(out)
+    return case_of("mixed", tmp_path_factory.mktemp("one"))
 
 
 def test_streams_after_every_layer(case):
@@ -193,18 +166,6 @@ def test_missing_and_misshapen_tensors_are_named(tmp_path):
     wrong["l0.mlp.up"] = weights["l0.mlp.up"][:8]
     with pytest.raises(qp.ProviderError, match="l0.mlp.up"):
         qp.Model(mm.write_folder(tmp_path / "b", config, wrong), 64)
-
-
-def continuation(case, prompt, count):
-    """Greedy tokens of the plain statement, and how close its choices were."""
-    tokens, margins = list(prompt), []
-    weights = mm.float64(case.weights)
-    for _ in range(count):
-        row = mo.forward(case.config, weights, tokens)[0][-1]
-        top = np.sort(row)[-2:]
-        margins.append(top[1] - top[0])
-        tokens.append(int(row.argmax()))
-    return tokens[len(prompt):], min(margins)
 
 
 def test_greedy_generation_through_the_worker(mixed):

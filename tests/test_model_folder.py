@@ -5,6 +5,7 @@ import struct
 
 import pytest
 
+import latent_model as lm
 import mixed_model as mm
 import qllm_provider as qp
 
@@ -41,6 +42,31 @@ def test_unknown_mixer_and_feed_forward_are_named(tmp_path):
     assert "convolution" in refusal(folder(tmp_path, layers=[layer]))
     layer = {"type": "wkv", "mixer": {"heads": 1, "dim": 8}, "mlp": {"kind": "routed", "ff": 4}}
     assert "routed" in refusal(folder(tmp_path / "b", layers=[layer]))
+
+
+def test_latent_layers_with_missing_keys(tmp_path):
+    def refused(kind, key, value=None):
+        layer = {"windowed": lm.windowed_latent(2, 8, 4, 8, 12, 10, 5),
+                 "latent": lm.latent(2, 8, 8, 12), "gla": lm.gla(2, 8, 8)}[kind]
+        config = lm.configuration(32, 16, [layer], [16])
+        place = config["layers"][0]["mixer"]
+        *path, last = key.split(".")
+        for part in path:
+            place = place[part]
+        if value is None:
+            del place[last]
+        else:
+            place[last] = value
+        path = mm.write_folder(tmp_path / (kind + key), config, lm.random_weights(
+            lm.configuration(32, 16, [lm.latent(2, 8, 8, 12)], [16]), 1))
+        return refusal(path)
+
+    for key in ("heads", "dim", "vdim", "kv_rank", "scale", "rot_dim", "rot", "mask.size",
+                "rot.base", "rot.dims", "rot.scaling.factor", "rot.scaling.slow"):
+        assert key.split(".")[-1] in refused("windowed", key), key
+    assert "kv_rank" in refused("latent", "kv_rank")
+    assert "tau" in refused("gla", "tau")
+    assert "tau" in refused("gla", "tau", 0)
 
 
 def test_broken_tensor_files(tmp_path):
