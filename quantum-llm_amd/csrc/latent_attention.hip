@@ -323,7 +323,6 @@ __global__ __launch_bounds__(256) void latent_query_kernel(AttentionArgs args) {
                          (size_t{head} * tiles + tile) * chunks * kWave + lane;
   const float* q = source + size_t{min(column, rows - 1u)} * run.query_stride;
   f32x4 sum = {};
-#pragma unroll 4
   for (uint32_t c = 0; c < chunks_of(a.dim); ++c)
     sum = mfma_bf16(weights[c * kWave], query_operand(q, c * 32u + 8u * quarter, a.dim), sum);
   if (column < rows)
@@ -648,10 +647,18 @@ __global__ __launch_bounds__(kValueThreads) void latent_value_kernel(AttentionAr
 
 // ---- prompt form -------------------------------------------------------------------
 
-// Keys or values of the expanded tiles: a wave holds 64 tokens x 4 weight tiles.
+constexpr uint32_t kExpandBlocks = 8;        // sixteen tokens each, per workgroup
+constexpr uint32_t kExpandTiles = 16;        // of weights, per workgroup
+
+// Keys or values of the expanded tiles: four waves side by side along the weight
+// tiles, four tiles each, the latents of 128 tokens shared through LDS a chunk of
+// 32 at a time.
 template <bool VALUES>
 __device__ __forceinline__ void expand_unit(const AttentionArgs& args, uint32_t unit_tiles,
-                                            uint32_t unit_tokens) {
+                                            uint32_t unit_tokens,
+                                            i32x4 (&shared)[2][kExpandBlocks * kWave]) {
+  constexpr uint32_t WT = kExpandTiles / 4u;
+  constexpr uint32_t MB = kExpandBlocks;
   const Latent& a = args.attention;
   const uint32_t wave = threadIdx.x / kWave;
   const uint32_t lane = threadIdx.x % kWave;
@@ -659,61 +666,73 @@ __device__ __forceinline__ void expand_unit(const AttentionArgs& args, uint32_t 
   const uint32_t quarter = lane / 16u;
   const uint32_t per_head = VALUES ? value_tiles(a) : chunks_of(a.dim) * 2u;
   const uint32_t weight_tiles = a.heads * per_head;
-  const uint32_t first_weight = unit_tiles * 8u + wave % 2u * 4u;
-  const uint32_t first_block = unit_tokens * 8u + wave / 2u * 4u;   // 16 tokens each
+  const uint32_t first_weight = unit_tiles * kExpandTiles + wave * WT;
+  const uint32_t first_block = unit_tokens * MB;
   const uint32_t blocks = args.tiles * 2u;
-  if (first_weight >= weight_tiles || first_block >= blocks) return;
   const uint32_t chunks = packed_chunks(a.rank);
   const uint32_t latent_chunks = chunks_of(a.rank);
-  const i32x4* weights[4];
-  const i32x4* latents[4];
+  const i32x4* weights[WT];
 #pragma unroll
-  for (uint32_t i = 0; i < 4u; ++i) {
+  for (uint32_t i = 0; i < WT; ++i)
     weights[i] = static_cast<const i32x4*>(VALUES ? a.value_up : a.key_up) +
                  size_t{min(first_weight + i, weight_tiles - 1u)} * chunks * kWave + lane;
-    latents[i] = reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(
-                     a, args.tile0 * kTile + min(first_block + i, blocks - 1u) * 16u)) +
-                 lane;
-  }
-  f32x4 sum[4][4] = {};      // [weight tile][token block]
-  i32x4 w[2][4], x[2][4];
+  // a wave fetches two of the eight token blocks
+  const i32x4* latents[2];
+#pragma unroll
+  for (uint32_t i = 0; i < 2u; ++i)
+    latents[i] =
+        reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(
+            a, args.tile0 * kTile + min(first_block + wave * 2u + i, blocks - 1u) * 16u)) +
+        lane;
+  f32x4 sum[WT][MB] = {};
+  i32x4 w[2][WT], x[2];
   const auto load = [&](uint32_t c, auto parity) __attribute__((always_inline)) {
     constexpr int P = decltype(parity)::value;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      w[P][i] = weights[i][c * kWave];
-      x[P][i] = latents[i][c * kWave];
-    }
+    for (uint32_t i = 0; i < WT; ++i) w[P][i] = weights[i][c * kWave];
+#pragma unroll
+    for (uint32_t i = 0; i < 2u; ++i) x[i] = latents[i][c * kWave];
+  };
+  const auto publish = [&](auto parity) __attribute__((always_inline)) {
+    constexpr int P = decltype(parity)::value;
+#pragma unroll
+    for (uint32_t i = 0; i < 2u; ++i) shared[P][(wave * 2u + i) * kWave + lane] = x[i];
+    __syncthreads();
   };
   const auto multiply = [&](auto parity) __attribute__((always_inline)) {
     constexpr int P = decltype(parity)::value;
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
+    for (uint32_t j = 0; j < MB; ++j) {
+      const i32x4 tokens = shared[P][j * kWave + lane];
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        sum[i][j] = VALUES ? mfma_bf16(x[P][j], w[P][i], sum[i][j])
-                           : mfma_bf16(w[P][i], x[P][j], sum[i][j]);
+      for (uint32_t i = 0; i < WT; ++i)
+        sum[i][j] = VALUES ? mfma_bf16(tokens, w[P][i], sum[i][j])
+                           : mfma_bf16(w[P][i], tokens, sum[i][j]);
+    }
   };
   constexpr std::integral_constant<int, 0> even{};
   constexpr std::integral_constant<int, 1> odd{};
   load(0u, even);
+  publish(even);
   uint32_t c = 0;
   for (; c + 2u <= latent_chunks; c += 2u) {
     load(c + 1u, odd);
     multiply(even);
+    publish(odd);
     load(min(c + 2u, latent_chunks - 1u), even);
     multiply(odd);
+    publish(even);
   }
   if (c < latent_chunks) multiply(even);
 
 #pragma unroll
-  for (uint32_t i = 0; i < 4u; ++i) {
+  for (uint32_t i = 0; i < WT; ++i) {
     const uint32_t at = first_weight + i;
     if (at >= weight_tiles) break;
     const uint32_t head = at / per_head;
     const uint32_t part = at % per_head;
 #pragma unroll
-    for (uint32_t j = 0; j < 4u; ++j) {
+    for (uint32_t j = 0; j < MB; ++j) {
       const uint32_t block = first_block + j;
       if (block >= blocks) break;
       const i32x2 four{static_cast<int>(pack_bf16(sum[i][j][0], sum[i][j][1])),
@@ -738,10 +757,11 @@ __device__ __forceinline__ void expand_unit(const AttentionArgs& args, uint32_t 
 
 __global__ __launch_bounds__(256, 2) void latent_expand_kernel(AttentionArgs args,
                                                                uint32_t key_units) {
+  __shared__ i32x4 shared[2][kExpandBlocks * kWave];
   if (blockIdx.x < key_units)
-    expand_unit<false>(args, blockIdx.x, blockIdx.y);
+    expand_unit<false>(args, blockIdx.x, blockIdx.y, shared);
   else
-    expand_unit<true>(args, blockIdx.x - key_units, blockIdx.y);
+    expand_unit<true>(args, blockIdx.x - key_units, blockIdx.y, shared);
 }
 
 constexpr uint32_t kPromptRows = 128;
@@ -1124,10 +1144,11 @@ extern "C" int32_t qllm_latent_attention_rows(const qllm_latent_attention* atten
     args.tile0 = a.window && first + 1u > a.window ? (first + 1u - a.window) / kTile : 0u;
     args.tiles = launch->maximum_position / kTile + 1u - args.tile0;
     latent_prompt_query_kernel<<<(rows * a.heads + 3u) / 4u, 256, 0, hip_stream>>>(args);
-    const uint32_t key_units = (a.heads * chunks_of(a.dim) * 2u + 7u) / 8u;
-    const uint32_t value_units = (a.heads * value_tiles(a) + 7u) / 8u;
-    latent_expand_kernel<<<dim3(key_units + value_units, (args.tiles * 2u + 7u) / 8u), 256, 0,
-                           hip_stream>>>(args, key_units);
+    const auto units = [](uint32_t count, uint32_t each) { return (count + each - 1u) / each; };
+    const uint32_t key_units = units(a.heads * chunks_of(a.dim) * 2u, kExpandTiles);
+    const uint32_t value_units = units(a.heads * value_tiles(a), kExpandTiles);
+    latent_expand_kernel<<<dim3(key_units + value_units, units(args.tiles * 2u, kExpandBlocks)),
+                           256, 0, hip_stream>>>(args, key_units);
     const uint32_t chunks = chunks_of(a.dim) + chunks_of(a.rot_dim);
     if (chunks <= 2u)
       launch_prompt<2>(args, hip_stream);

@@ -14,6 +14,19 @@
 // low-rank projection, rates) is prepared before, the output norm and gate
 // follow after, both over all tokens at once.  One token (decode) is one
 // launch that does all of it with a workgroup per head.
+//
+// Where the state only decays by rows and takes up outer products (bonus, gated),
+// prompts go through F32 matrix products in chunks of sixteen tokens instead.  With
+// D(j, i) the product of the decays of tokens j + 1 .. i, a chunk that starts from S
+// has the outputs
+//   o_i = (r_i * D(start, i))^T S + sum over j <= i of (r_i . (k_j * D(j, i))) v_j
+// and leaves D(start, end) S + sum of (k_j * D(j, end)) v_j^T.  The decays are
+// multiplied up pair by pair and none divides, so no product exceeds one: nothing
+// overflows, and what underflows is gone token by token as well.  The chunks' own
+// matrices are made for all chunks at once; a wave then walks them with sixteen
+// columns of the state in its accumulators, which stand as the next product's
+// operand as they are.  Long prompts are cut into segments walked side by side:
+// once for the states they add, which are then joined, and once for the outputs.
 #include "mixed_common.hpp"
 
 namespace qllm {
@@ -25,6 +38,13 @@ struct RecurrenceArgs {
   float* prepared;   // [head][row][slots][padded dim]
   float* scalars;    // BONUS: [head][row] sum of r * bonus * k
   float* outputs;    // [row][heads * vdim]
+  // chunks of sixteen tokens:
+  float* chunks;     // [head][chunk]: chunk_floats(padded)
+  float* starts;     // [segment][head][dim][vdim]
+  float* totals;     // [segment][head][padded dim]: all decays of the segment
+  uint32_t chunk_count;      // of a head
+  uint32_t segments;
+  uint32_t segment_chunks;
   uint32_t padded;   // dim padded to 16, 32, 64, 128 or 256
 };
 
@@ -56,7 +76,7 @@ __device__ __forceinline__ float low_value(const qllm_recurrence& l, float x) {
 
 __device__ __forceinline__ void copy_carry(const RecurrenceArgs& args) {
   const auto& run = args.launch;
-  if (blockIdx.x != 0 || blockIdx.y != 0 || !run.carry_to) return;
+  if (blockIdx.x != 0 || blockIdx.y != 0 || blockIdx.z != 0 || !run.carry_to) return;
   float* carry = run.carry_to + args.layer.step[kStepSlot] * args.layer.slot_stride;
   for (uint32_t c = threadIdx.x; c < run.carry_width; c += blockDim.x)
     carry[c] = run.carry_from[c];
@@ -557,6 +577,235 @@ __global__ __launch_bounds__(256) void recurrence_scan_kernel(RecurrenceArgs arg
   copy_carry(args);
 }
 
+// ---- prompts in chunks of sixteen tokens ---------------------------------------
+
+constexpr uint32_t kChunk = 16;
+constexpr uint32_t kMaximumSegments = 16;
+
+// A chunk's matrices: reads times the decays so far [token][padded], keys times the
+// decays to come, transposed [padded][token], weights [token][earlier token], all
+// decays [padded].
+__host__ __device__ constexpr uint32_t chunk_floats(uint32_t padded) {
+  return 2u * kChunk * padded + kChunk * kChunk + padded;
+}
+
+// Sixteen lanes per token j of a chunk, KPL channels each.
+template <uint32_t KIND, int KPL>
+__global__ __launch_bounds__(256) void recurrence_chunk_kernel(RecurrenceArgs args) {
+  constexpr bool BONUS = KIND == QLLM_RECURRENCE_BONUS;
+  constexpr uint32_t kPadded = KPL * 16u;
+  constexpr uint32_t kVectors = vectors_of(KIND);
+  __shared__ float reads[kChunk][kPadded];
+  __shared__ float decays[kChunk][kPadded];
+  const auto& run = args.launch;
+  const uint32_t head = blockIdx.y;
+  const uint32_t j = threadIdx.x / 16u;
+  const uint32_t part = threadIdx.x % 16u;
+  const uint32_t row = blockIdx.x * kChunk + j;
+  const bool there = row < run.rows;
+  const float* source =
+      args.prepared + (size_t{head} * run.rows + min(row, run.rows - 1u)) * kVectors * kPadded +
+      part * KPL;
+  float read[KPL], key[KPL];
+#pragma unroll
+  for (int i = 0; i < KPL; ++i) {
+    // tokens past the last one: decays of 1 and zeros, which change nothing
+    read[i] = there ? source[i] : 0.0f;
+    key[i] = there ? source[kPadded + i] : 0.0f;
+    reads[j][part * KPL + i] = read[i];
+    decays[j][part * KPL + i] = there ? source[2u * kPadded + i] : 1.0f;
+  }
+  const float own = BONUS && there ? args.scalars[size_t{head} * run.rows + row] : 0.0f;
+  __syncthreads();
+  float weight[kChunk];
+  float all[KPL];
+#pragma unroll
+  for (int i = 0; i < KPL; ++i) all[i] = 1.0f;
+#pragma unroll
+  for (uint32_t t = 0; t < kChunk; ++t) {
+    // BONUS reads before token t's decay, GATED after it
+    float dot = 0.0f;
+#pragma unroll
+    for (int i = 0; i < KPL; ++i) {
+      const float decay = decays[t][part * KPL + i];
+      const float faded = t > j ? key[i] * decay : key[i];
+      dot = fmaf(reads[t][part * KPL + i], BONUS ? key[i] : faded, dot);
+      key[i] = faded;
+      read[i] *= BONUS ? (t < j ? decay : 1.0f) : (t <= j ? decay : 1.0f);
+      all[i] *= decay;
+    }
+    weight[t] = (BONUS ? t > j : t >= j) ? dot : 0.0f;
+  }
+  // lane t of token j: what output t takes of value j
+  float mine = row16_transposed_sum(weight);
+  if (BONUS && part == j) mine = own;
+  float* out = args.chunks +
+               (size_t{head} * args.chunk_count + blockIdx.x) * chunk_floats(kPadded);
+  float* transposed = out + kChunk * kPadded;
+#pragma unroll
+  for (int i = 0; i < KPL; ++i) {
+    out[j * kPadded + part * KPL + i] = read[i];
+    transposed[(part * KPL + i) * kChunk + j] = key[i];
+    if (j == 0u) transposed[kChunk * kPadded + kChunk * kChunk + part * KPL + i] = all[i];
+  }
+  transposed[kChunk * kPadded + part * kChunk + j] = mine;
+}
+
+// A wave per sixteen columns of one head's state, TILES = padded dim / 16.  With
+// OUTPUTS the segment's outputs from its starting state; without, the state it ends
+// with when it starts from zero (the first one: from the request's).
+template <bool OUTPUTS, int TILES>
+__global__ __launch_bounds__(256, 1) void recurrence_walk_kernel(RecurrenceArgs args) {
+  constexpr uint32_t kPadded = TILES * 16u;
+  constexpr uint32_t kPieces = chunk_floats(kPadded) / 4u;
+  const qllm_recurrence& l = args.layer;
+  const auto& run = args.launch;
+  const uint32_t head = blockIdx.y;
+  const uint32_t segment = blockIdx.z;
+  const uint32_t dim = l.dim;
+  const uint32_t vdim = l.vdim;
+  const uint32_t lane = threadIdx.x % kWave;
+  const uint32_t quarter = lane / 16u;
+  const uint32_t first_column = (blockIdx.x * 4u + threadIdx.x / kWave) * 16u;
+  const uint32_t column = first_column + lane % 16u;
+  const bool real = column < vdim;
+  if (OUTPUTS) copy_carry(args);
+  if (first_column >= vdim) return;
+
+  const bool several = args.segments > 1u;
+  float* const request =
+      l.state + l.step[kStepSlot] * l.slot_stride + size_t{head} * dim * vdim;
+  float* const kept = args.starts + (size_t{segment} * l.heads + head) * dim * vdim;
+  const float* const from = OUTPUTS && several ? kept : request;
+  f32x4 state[TILES];
+#pragma unroll
+  for (int d = 0; d < TILES; ++d)
+#pragma unroll
+    for (uint32_t i = 0; i < 4u; ++i) {
+      const uint32_t row = d * 16u + 4u * quarter + i;
+      state[d][i] = real && row < dim && (OUTPUTS || segment == 0u)
+                        ? from[size_t{row} * vdim + column]
+                        : 0.0f;
+    }
+  f32x4 faded[TILES];
+#pragma unroll
+  for (int d = 0; d < TILES; ++d) faded[d] = f32x4{1.0f, 1.0f, 1.0f, 1.0f};
+
+  struct Chunk {
+    f32x4 reads[OUTPUTS ? TILES : 1];
+    f32x4 keys[TILES];
+    f32x4 weights;
+    f32x4 decays[TILES];
+    float values[4];
+  };
+  const f32x4* const source =
+      reinterpret_cast<const f32x4*>(args.chunks) + size_t{head} * args.chunk_count * kPieces;
+  const float* const value_column = run.projections + run.v_column + head * vdim +
+                                    min(column, vdim - 1u);
+  const auto fetch = [&](Chunk& c, uint32_t which) __attribute__((always_inline)) {
+    const f32x4* at = source + size_t{which} * kPieces;
+    if constexpr (OUTPUTS) {
+#pragma unroll
+      for (int d = 0; d < TILES; ++d)
+        c.reads[d] = at[(lane % 16u) * (kPadded / 4u) + d * 4u + quarter];
+      c.weights = at[2u * kChunk * kPadded / 4u + lane % 16u * (kChunk / 4u) + quarter];
+    }
+#pragma unroll
+    for (int d = 0; d < TILES; ++d) {
+      c.keys[d] = at[kChunk * kPadded / 4u + (d * 16u + lane % 16u) * (kChunk / 4u) + quarter];
+      c.decays[d] = at[(2u * kChunk * kPadded + kChunk * kChunk) / 4u + d * 4u + quarter];
+    }
+#pragma unroll
+    for (uint32_t e = 0; e < 4u; ++e) {
+      const uint32_t row = min(which * kChunk + 4u * quarter + e, run.rows - 1u);
+      c.values[e] = value_column[size_t{row} * run.stride];
+    }
+  };
+  const auto advance = [&](const Chunk& c, uint32_t which) __attribute__((always_inline)) {
+    if constexpr (OUTPUTS) {
+      f32x4 sum[4] = {};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        sum[e] = __builtin_amdgcn_mfma_f32_16x16x4f32(c.weights[e], c.values[e], sum[e], 0, 0, 0);
+#pragma unroll
+        for (int d = 0; d < TILES; ++d)
+          sum[e] = __builtin_amdgcn_mfma_f32_16x16x4f32(c.reads[d][e], state[d][e], sum[e], 0,
+                                                        0, 0);
+      }
+      const f32x4 out = (sum[0] + sum[1]) + (sum[2] + sum[3]);
+#pragma unroll
+      for (uint32_t i = 0; i < 4u; ++i) {
+        const uint32_t row = which * kChunk + 4u * quarter + i;
+        if (real && row < run.rows)
+          args.outputs[(size_t{row} * l.heads + head) * vdim + column] = out[i];
+      }
+    }
+#pragma unroll
+    for (int d = 0; d < TILES; ++d) {
+      state[d] *= c.decays[d];
+      if constexpr (!OUTPUTS) faded[d] *= c.decays[d];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+#pragma unroll
+      for (int d = 0; d < TILES; ++d)
+        state[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(c.keys[d][e], c.values[e], state[d], 0,
+                                                        0, 0);
+  };
+  const uint32_t begin = segment * args.segment_chunks;
+  const uint32_t end = min(begin + args.segment_chunks, args.chunk_count);
+  Chunk even, odd;
+  fetch(even, begin);
+  uint32_t which = begin;
+  while (which < end) {
+    fetch(odd, min(which + 1u, end - 1u));
+    advance(even, which);
+    if (++which >= end) break;
+    fetch(even, min(which + 1u, end - 1u));
+    advance(odd, which);
+    ++which;
+  }
+  if (OUTPUTS && segment + 1u != args.segments) return;
+  float* const to = OUTPUTS ? request : kept;
+#pragma unroll
+  for (int d = 0; d < TILES; ++d)
+#pragma unroll
+    for (uint32_t i = 0; i < 4u; ++i) {
+      const uint32_t row = d * 16u + 4u * quarter + i;
+      if (real && row < dim) to[size_t{row} * vdim + column] = state[d][i];
+    }
+  if (OUTPUTS || first_column || lane % 16u) return;
+#pragma unroll
+  for (int d = 0; d < TILES; ++d)
+    reinterpret_cast<f32x4*>(args.totals)[(size_t{segment} * l.heads + head) * (kPadded / 4u) +
+                                          d * 4u + quarter] = faded[d];
+}
+
+// The states that segments end with become the states they start from.
+__global__ __launch_bounds__(256) void recurrence_join_kernel(RecurrenceArgs args) {
+  const qllm_recurrence& l = args.layer;
+  const uint32_t elements = l.heads * l.dim * l.vdim;
+  const uint32_t at = blockIdx.x * blockDim.x + threadIdx.x;
+  if (at >= elements) return;
+  const uint32_t row = at / l.vdim;      // over all heads
+  const float* total = args.totals + size_t{row / l.dim} * args.padded + row % l.dim;
+  float end[kMaximumSegments], fade[kMaximumSegments];
+#pragma unroll
+  for (uint32_t z = 0; z + 1u < kMaximumSegments; ++z) {
+    const bool there = z + 1u < args.segments;
+    end[z] = there ? args.starts[size_t{z} * elements + at] : 0.0f;
+    fade[z] = z && there ? total[size_t{z} * l.heads * args.padded] : 0.0f;
+  }
+  args.starts[at] = l.state[l.step[kStepSlot] * l.slot_stride + at];
+  float state = 0.0f;
+#pragma unroll
+  for (uint32_t z = 0; z + 1u < kMaximumSegments; ++z) {
+    if (z + 1u >= args.segments) continue;
+    state = fmaf(fade[z], state, end[z]);
+    args.starts[size_t{z + 1u} * elements + at] = state;
+  }
+}
+
 // Output norm and gate: a wave per (token, head).
 template <typename T>
 __global__ __launch_bounds__(256) void recurrence_finish_kernel(RecurrenceArgs args) {
@@ -606,6 +855,32 @@ void launch_scan(const RecurrenceArgs& args, hipStream_t stream) {
   }
 }
 
+template <uint32_t KIND, int TILES>
+void launch_chunks(const RecurrenceArgs& args, hipStream_t stream) {
+  const qllm_recurrence& l = args.layer;
+  recurrence_chunk_kernel<KIND, TILES>
+      <<<dim3(args.chunk_count, l.heads), 256, 0, stream>>>(args);
+  const uint32_t columns = (l.vdim + 63u) / 64u;
+  if (args.segments > 1u) {
+    // the last segment's own end comes with its outputs
+    recurrence_walk_kernel<false, TILES>
+        <<<dim3(columns, l.heads, args.segments - 1u), 256, 0, stream>>>(args);
+    recurrence_join_kernel<<<(l.heads * l.dim * l.vdim + 255u) / 256u, 256, 0, stream>>>(args);
+  }
+  recurrence_walk_kernel<true, TILES>
+      <<<dim3(columns, l.heads, args.segments), 256, 0, stream>>>(args);
+}
+
+template <uint32_t KIND>
+void launch_chunks_of(const RecurrenceArgs& args, hipStream_t stream) {
+  switch (args.padded) {
+    case 16u: launch_chunks<KIND, 1>(args, stream); break;
+    case 32u: launch_chunks<KIND, 2>(args, stream); break;
+    case 64u: launch_chunks<KIND, 4>(args, stream); break;
+    default: launch_chunks<KIND, 8>(args, stream); break;
+  }
+}
+
 template <typename T>
 void launch_gated_step(const RecurrenceArgs& args, hipStream_t stream) {
   const uint32_t groups = 1024u / args.layer.vdim;
@@ -642,6 +917,39 @@ size_t scalar_bytes(const qllm_recurrence& l, uint32_t rows) {
   return (size_t{l.heads} * rows * 4u + 15u) / 16u * 16u;
 }
 
+size_t output_bytes(const qllm_recurrence& l, uint32_t rows) {
+  return (size_t{rows} * l.heads * l.vdim * 4u + 15u) / 16u * 16u;
+}
+
+constexpr uint32_t kChunkedRows = 64;        // shorter batches go token by token
+constexpr uint32_t kSegmentRows = 256;       // at least
+
+bool goes_in_chunks(const qllm_recurrence& l, uint32_t rows) {
+  return l.kind != QLLM_RECURRENCE_DELTA && l.dim <= 128u && rows >= kChunkedRows;
+}
+
+// Segments of a prompt: a few waves for every SIMD of the chip.
+uint32_t segments_for(const qllm_recurrence& l, uint32_t rows) {
+  const uint32_t waves = l.heads * ((l.vdim + 15u) / 16u);
+  const uint32_t wanted = (2048u + waves - 1u) / waves;
+  const uint32_t most = rows / kSegmentRows;
+  const uint32_t segments = wanted < most ? wanted : most;
+  return segments > kMaximumSegments ? kMaximumSegments : segments ? segments : 1u;
+}
+
+size_t chunk_bytes(const qllm_recurrence& l, uint32_t rows) {
+  return size_t{l.heads} * ((rows + kChunk - 1u) / kChunk) * chunk_floats(padded_dim(l.dim)) *
+         4u;
+}
+
+size_t start_bytes(const qllm_recurrence& l, uint32_t segments) {
+  return (size_t{segments} * l.heads * l.dim * l.vdim * 4u + 15u) / 16u * 16u;
+}
+
+size_t total_bytes(const qllm_recurrence& l, uint32_t segments) {
+  return size_t{segments} * l.heads * padded_dim(l.dim) * 4u;
+}
+
 }  // namespace
 }  // namespace qllm
 
@@ -650,9 +958,14 @@ using namespace qllm;
 extern "C" size_t qllm_recurrence_workspace_bytes(const qllm_recurrence* recurrence,
                                                   uint32_t rows) {
   if (!recurrence || rows <= 1u) return 0u;
-  return prepared_bytes(*recurrence, rows) + scalar_bytes(*recurrence, rows) +
-         size_t{rows} * recurrence->heads *
-             (recurrence->vdim ? recurrence->vdim : recurrence->dim) * 4u;
+  qllm_recurrence l = *recurrence;
+  if (!l.vdim) l.vdim = l.dim;
+  size_t bytes = prepared_bytes(l, rows) + scalar_bytes(l, rows) + output_bytes(l, rows);
+  if (goes_in_chunks(l, rows)) {
+    const uint32_t segments = segments_for(l, rows);
+    bytes += chunk_bytes(l, rows) + start_bytes(l, segments) + total_bytes(l, segments);
+  }
+  return bytes;
 }
 
 extern "C" int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
@@ -680,7 +993,10 @@ extern "C" int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
   if (launch->low_column + l.rank > launch->stride)
     return fail(QLLM_INVALID_ARGUMENT, "recurrence columns exceed the projection rows");
   const auto hip_stream = as_stream(stream);
-  RecurrenceArgs args{l, *launch, nullptr, nullptr, nullptr, padded_dim(l.dim)};
+  RecurrenceArgs args{};
+  args.layer = l;
+  args.launch = *launch;
+  args.padded = padded_dim(l.dim);
   const bool f32 = l.element == QLLM_ELEMENT_F32;
   if (launch->rows == 1u) {
     if (f32)
@@ -696,13 +1012,29 @@ extern "C" int32_t qllm_recurrence_rows(const qllm_recurrence* recurrence,
   auto* bytes = static_cast<uint8_t*>(launch->workspace);
   args.prepared = reinterpret_cast<float*>(bytes);
   args.scalars = reinterpret_cast<float*>(bytes + prepared_bytes(l, launch->rows));
-  args.outputs = reinterpret_cast<float*>(bytes + prepared_bytes(l, launch->rows) +
-                                          scalar_bytes(l, launch->rows));
+  bytes += prepared_bytes(l, launch->rows) + scalar_bytes(l, launch->rows);
+  args.outputs = reinterpret_cast<float*>(bytes);
+  bytes += output_bytes(l, launch->rows);
   const uint32_t prepare_rows = 256u / args.padded * kRowsPerThread;
   recurrence_prepare_kernel<<<dim3((launch->rows + prepare_rows - 1u) / prepare_rows,
                                    l.heads),
                               256, 0, hip_stream>>>(args);
-  if (delta)
+  if (goes_in_chunks(l, launch->rows)) {
+    const uint32_t segments = segments_for(l, launch->rows);
+    args.chunks = reinterpret_cast<float*>(bytes);
+    bytes += chunk_bytes(l, launch->rows);
+    args.starts = reinterpret_cast<float*>(bytes);
+    bytes += start_bytes(l, segments);
+    args.totals = reinterpret_cast<float*>(bytes);
+    args.chunk_count = (launch->rows + kChunk - 1u) / kChunk;
+    args.segment_chunks = (args.chunk_count + segments - 1u) / segments;
+    // none is empty
+    args.segments = (args.chunk_count + args.segment_chunks - 1u) / args.segment_chunks;
+    if (gated)
+      launch_chunks_of<QLLM_RECURRENCE_GATED>(args, hip_stream);
+    else
+      launch_chunks_of<QLLM_RECURRENCE_BONUS>(args, hip_stream);
+  } else if (delta)
     launch_scan<QLLM_RECURRENCE_DELTA>(args, hip_stream);
   else if (gated)
     launch_scan<QLLM_RECURRENCE_GATED>(args, hip_stream);

@@ -445,3 +445,26 @@ def test_decays_near_both_ends(device):
     close(got, want, F32, "outputs", factor=2.0)
     state = layer.state[layer.slot_stride:layer.slot_stride + 2 * 8 * 16].cpu().numpy()
     close(state.reshape(2, 8, 16).astype(np.float64), states, F32, "state", factor=4.0)
+
+
+@pytest.mark.parametrize("element", [F32, BF16])
+@pytest.mark.parametrize("heads,dim,vdim,tau", [(2, 64, 128, 16.0), (1, 20, 36, 1.0),
+                                                (3, 16, 256, 4.0), (1, 130, 8, 16.0),
+                                                (1, 32, 300, 8.0)])
+def test_long_prompts_in_segments(device, element, heads, dim, vdim, tau):
+    rng = np.random.default_rng(dim)
+    layer = Gated(device, element, heads, dim, vdim, 6, tau, rng)
+    projections = mm.bf16(rng.standard_normal((1300, layer.stride)))
+    want, states = layer.expected(projections)
+    n = heads * dim * vdim
+    for counts in ([1300], [600, 1, 699], [100, 530, 515, 155]):
+        layer.state.zero_()
+        got, at = [], 0
+        for count in counts:
+            got.append(layer.run(projections[at:at + count]))
+            at += count
+        close(np.concatenate(got), want, element, str(counts), factor=2.0)
+        state = layer.state[layer.slot_stride:layer.slot_stride + n].cpu().numpy()
+        close(state.reshape(heads, dim, vdim).astype(np.float64), states, F32, "state",
+              factor=4.0)
+        assert torch.all(layer.state[:layer.slot_stride] == 0)

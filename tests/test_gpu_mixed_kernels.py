@@ -465,6 +465,29 @@ def test_recurrences_in_portions(device, element, kind, heads, dim, rank):
     close(layer.run(projections), want, element, "whole", factor=2.0)
 
 
+@pytest.mark.parametrize("element", [F32, BF16])
+@pytest.mark.parametrize("kind", [qh.RECURRENCE_DELTA, qh.RECURRENCE_BONUS])
+@pytest.mark.parametrize("heads,dim", [(2, 64), (1, 24), (1, 130)])
+def test_recurrences_over_long_prompts(device, element, kind, heads, dim):
+    rng = np.random.default_rng(dim + kind)
+    layer = Recurrence(device, element, kind, heads, dim, 6, rng)
+    projections = mm.bf16(rng.standard_normal((1300, layer.stride)))
+    projections[:, layer.columns[1]:layer.columns[2]] *= np.float32(2 / np.sqrt(dim))
+    want, states = layer.expected(projections)
+    n = heads * dim * dim
+    for counts in ([1300], [600, 1, 699], [100, 530, 515, 155]):
+        layer.state.zero_()
+        got, at = [], 0
+        for count in counts:
+            got.append(layer.run(projections[at:at + count]))
+            at += count
+        close(np.concatenate(got), want, element, str(counts), factor=2.0)
+        state = layer.state[layer.slot_stride:layer.slot_stride + n].cpu().numpy()
+        close(state.reshape(heads, dim, dim).astype(np.float64), states, F32, "state",
+              factor=4.0)
+        assert torch.all(layer.state[:layer.slot_stride] == 0)
+
+
 def test_launches_turn_down_what_does_not_fit(device):
     layer = Attention(device, BF16, 4, 2, 64, 64, 32, 2, None, 0.125, context=128)
     bad = qh.RopeStoreLaunch(layer.table.data_ptr(), 8, 0, 0, 0, 0, None, None, None, None,
