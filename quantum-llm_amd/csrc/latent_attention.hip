@@ -26,7 +26,8 @@ namespace {
 constexpr uint32_t kTile = 32;               // tokens
 constexpr uint32_t kFragment = 512;          // elements, 16 x 32
 constexpr uint32_t kSplitRows = 32;          // rows of the split form
-constexpr uint32_t kMaximumSplits = 64;       // a lane each when the parts are added
+constexpr uint32_t kMaximumSplits = 128;      // two for a lane when the parts are added
+constexpr uint32_t kSplitsFirst = 64;         // of one tile each, before they take several
 constexpr uint32_t kValueThreads = 1024;
 constexpr float kLog2e = 1.4426950408889634f;
 
@@ -75,6 +76,13 @@ __device__ __forceinline__ T* cache_block(const Latent& a, void* const* pages,
 template <typename T>
 __device__ __forceinline__ T* cache_block(const Latent& a, uint32_t token) {
   return cache_block<T>(a, pages_of(a), token);
+}
+
+// Pieces of a page for operand loads.  A pointer read from memory could point
+// anywhere; said to be global, its loads count on their own and complete in order.
+typedef const __attribute__((address_space(1))) i32x4 global_piece;
+__device__ __forceinline__ global_piece* as_global(const void* pieces) {
+  return (global_piece*)(pieces);
 }
 
 // Value d of a rotated vector x (its dimensions from rotary_dims on stay).
@@ -178,6 +186,57 @@ struct AttentionArgs {
 __device__ __forceinline__ float gate_of(const qllm_latent_launch& run, uint32_t row,
                                          uint32_t column) {
   return run.gate ? sigmoid_f32(run.gate[size_t{row} * run.gate_stride + column]) : 1.0f;
+}
+
+// Rows of outputs and gates can be taken four values at a time.
+__device__ __forceinline__ bool in_fours(const Latent& a, const qllm_latent_launch& run) {
+  return (a.vdim | run.output_stride | run.gate_stride) % 4u == 0u &&
+         (reinterpret_cast<uintptr_t>(run.gate) & 15u) == 0u &&
+         (reinterpret_cast<uintptr_t>(run.output) & 7u) == 0u;
+}
+
+// Gates of N times four values of a head, the first four from n on, the others 16
+// apart; no load depends on whether they exist.
+template <int N>
+__device__ __forceinline__ void take_gates(f32x4 (&gate)[N], const Latent& a,
+                                           const qllm_latent_launch& run, uint32_t row,
+                                           uint32_t head, uint32_t n) {
+  if (!run.gate) {
+#pragma unroll
+    for (int t = 0; t < N; ++t) gate[t] = f32x4{1.0f, 1.0f, 1.0f, 1.0f};
+    return;
+  }
+  const float* source = run.gate + size_t{row} * run.gate_stride + head * a.vdim;
+  if (in_fours(a, run)) {
+#pragma unroll
+    for (int t = 0; t < N; ++t)
+      gate[t] = *reinterpret_cast<const f32x4*>(source + min(n + t * 16u, a.vdim - 4u));
+  } else {
+#pragma unroll
+    for (int t = 0; t < N; ++t)
+#pragma unroll
+      for (uint32_t i = 0; i < 4u; ++i)
+        gate[t][i] = source[min(n + t * 16u + i, a.vdim - 1u)];
+  }
+#pragma unroll
+  for (int t = 0; t < N; ++t)
+#pragma unroll
+    for (uint32_t i = 0; i < 4u; ++i) gate[t][i] = sigmoid_f32(gate[t][i]);
+}
+
+__device__ __forceinline__ void store_four(const Latent& a, const qllm_latent_launch& run,
+                                           uint32_t row, uint32_t head, uint32_t n,
+                                           f32x4 value) {
+  if (n >= a.vdim) return;
+  uint16_t* out = static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride +
+                  head * a.vdim + n;
+  if (in_fours(a, run)) {
+    *reinterpret_cast<i32x2*>(out) =
+        i32x2{static_cast<int>(pack_bf16(value[0], value[1])),
+              static_cast<int>(pack_bf16(value[2], value[3]))};
+  } else {
+    for (uint32_t i = 0; i < 4u && n + i < a.vdim; ++i) store_element(out + i, value[i]);
+  }
 }
 
 // ---- general form ----------------------------------------------------------------
@@ -377,8 +436,9 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
   constexpr int kLoads = (kChunks + 1) / 2;          // 16-byte pieces per thread and tile
   __shared__ __attribute__((aligned(16))) uint16_t tile[2 * kChunks * kFragment];
   __shared__ f32x4 parts[4][2][kWave];
+  static_assert(kLoads * 256 == 2 * kChunks * kWave);
   const Latent& a = args.attention;
-  const uint32_t wave = threadIdx.x / kWave;
+  const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
   const uint32_t lane = threadIdx.x % kWave;
   const uint32_t quarter = lane / 16u;
   const uint32_t items = args.launch.rows * a.heads;
@@ -394,24 +454,33 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
   const uint32_t begin = first_tile(a, low);
   const uint32_t end = high / kTile + 1u;
 
+  // No load or matrix product below depends on a condition - places past the end
+  // are clamped to one that exists - so that a wait for one tile's loads leaves the
+  // next one's in flight.  Chunks of the query past the last one are zero.
   i32x4 q[kQuery];
+  uint32_t key_at[kQuery];
   const uint16_t* query =
       args.query + size_t{min(item, items - 1u)} * chunks * 32u + 8u * quarter;
 #pragma unroll
   for (int i = 0; i < kQuery; ++i) {
-    const uint32_t c = wave + 4u * i;
-    q[i] = c < chunks ? *reinterpret_cast<const i32x4*>(query + c * 32u) : i32x4{};
+    const uint32_t c = min(wave + 4u * i, chunks - 1u);
+    const i32x4 stored = *reinterpret_cast<const i32x4*>(query + c * 32u);
+    q[i] = wave + 4u * i < chunks ? stored : i32x4{};
+    key_at[i] = c * kWave + lane;
   }
   void* const* const pages = pages_of(a);
-  const uint32_t pieces = 2u * chunks * kWave;
+  const uint32_t last_piece = 2u * chunks * kWave - 1u;
+  const auto page_for = [&](uint32_t t) {
+    return as_global(cache_block<const uint16_t>(a, pages, min(t, end - 1u) * kTile));
+  };
+  global_piece* ahead = page_for(begin + blockIdx.x);   // of the next fetch
   const auto fetch = [&](i32x4 (&staged)[kLoads], uint32_t t) __attribute__((always_inline)) {
-    const i32x4* source =
-        reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(a, pages, t * kTile));
+    global_piece* const source = ahead;
+    ahead = page_for(t + gridDim.x);
 #pragma unroll
-    for (int i = 0; i < kLoads; ++i) {
-      const uint32_t piece = i * 256u + threadIdx.x;
-      if (piece < pieces) staged[i] = source[piece];
-    }
+    for (int i = 0; i < kLoads; ++i)
+      staged[i] = source[min(i * 256u + threadIdx.x, last_piece)];
+    __builtin_amdgcn_sched_barrier(0);   // in this order
   };
   const float unit = a.scale * kLog2e;
   float maximum = -INFINITY;
@@ -420,23 +489,18 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
   // `staged` holds tile `at` and takes the one after next
   const auto take = [&](i32x4 (&staged)[kLoads], uint32_t at) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < kLoads; ++i) {
-      const uint32_t piece = i * 256u + threadIdx.x;
-      if (piece < pieces) reinterpret_cast<i32x4*>(tile)[piece] = staged[i];
-    }
+    for (int i = 0; i < kLoads; ++i)
+      reinterpret_cast<i32x4*>(tile)[i * 256u + threadIdx.x] = staged[i];
     __syncthreads();
-    if (at + 2u * gridDim.x < end) fetch(staged, at + 2u * gridDim.x);
+    fetch(staged, at + 2u * gridDim.x);
     f32x4 s[2] = {};
 #pragma unroll
-    for (int i = 0; i < kQuery; ++i) {
-      const uint32_t c = wave + 4u * i;
-      if (c >= chunks) continue;
+    for (int i = 0; i < kQuery; ++i)
 #pragma unroll
       for (int half = 0; half < 2; ++half)
         s[half] = mfma_bf16(
-            reinterpret_cast<const i32x4*>(tile)[(half * chunks + c) * kWave + lane], q[i],
+            reinterpret_cast<const i32x4*>(tile)[half * chunks * kWave + key_at[i]], q[i],
             s[half]);
-    }
     parts[wave][0][lane] = s[0];
     parts[wave][1][lane] = s[1];
     __syncthreads();
@@ -473,8 +537,7 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
     const uint32_t token = 4u * quarter + lane % 16u / 4u;
 #pragma unroll
     for (int j = 0; j < R; ++j) {
-      const uint32_t t = wave + 4u * j;      // sixteen latent values
-      if (t >= latent_chunks * 2u) continue;
+      const uint32_t t = min(wave + 4u * j, latent_chunks * 2u - 1u);   // sixteen values
       const uint32_t column = t % 2u * 16u + lane % 4u * 4u;
       const uint16_t* fragment = tile + t / 2u * kFragment + in_fragment(token, column);
       const i32x2 left = read_transposed(fragment);
@@ -486,8 +549,8 @@ __global__ __launch_bounds__(256) void latent_split_kernel(AttentionArgs args) {
   };
   i32x4 even[kLoads], odd[kLoads];
   uint32_t next = begin + blockIdx.x;
-  if (next < end) fetch(even, next);
-  if (next + gridDim.x < end) fetch(odd, next + gridDim.x);
+  fetch(even, next);
+  fetch(odd, next + gridDim.x);
   while (next < end) {
     take(even, next);
     next += gridDim.x;
@@ -568,11 +631,28 @@ __global__ __launch_bounds__(kValueThreads) void latent_value_kernel(AttentionAr
 
   if (wave < rows) {
     const uint32_t item = (row0 + wave) * a.heads + head;
-    const float* pair = args.maxima + (size_t{min(lane, args.splits - 1u)} * items + item) * 2u;
-    const float m = lane < args.splits ? pair[0] : -INFINITY;
-    const float t = lane < args.splits ? pair[1] : 0.0f;
-    const float factor = __builtin_amdgcn_exp2f(m - wave_max(m));
-    share[wave][lane] = factor / wave_sum(factor * t);
+    constexpr uint32_t kEach = kMaximumSplits / kWave;
+    float m[kEach], t[kEach];
+    float top = -INFINITY;
+#pragma unroll
+    for (uint32_t i = 0; i < kEach; ++i) {
+      const uint32_t split = i * kWave + lane;
+      const float* pair =
+          args.maxima + (size_t{min(split, args.splits - 1u)} * items + item) * 2u;
+      m[i] = split < args.splits ? pair[0] : -INFINITY;
+      t[i] = split < args.splits ? pair[1] : 0.0f;
+      top = fmaxf(top, m[i]);
+    }
+    top = wave_max(top);
+    float total = 0.0f;
+#pragma unroll
+    for (uint32_t i = 0; i < kEach; ++i) {
+      m[i] = __builtin_amdgcn_exp2f(m[i] - top);
+      total = fmaf(m[i], t[i], total);
+    }
+    total = wave_sum(total);
+#pragma unroll
+    for (uint32_t i = 0; i < kEach; ++i) share[wave][i * kWave + lane] = m[i] / total;
   }
   __syncthreads();
   // a row's parts over as many groups as there are; every group a row if not
@@ -632,14 +712,10 @@ __global__ __launch_bounds__(kValueThreads) void latent_value_kernel(AttentionAr
     __syncthreads();
     if (unit < units && unit % 2u == 0u && column < rows) {
       sum += added[(wave + 1u) * kWave + lane];
-      const uint32_t row = row0 + column;
-      for (uint32_t i = 0; i < 4u; ++i) {
-        const uint32_t n = unit / 2u * 16u + 4u * quarter + i;
-        if (n >= a.vdim) break;
-        const uint32_t at = head * a.vdim + n;
-        store_element(static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride + at,
-                      sum[i] * gate_of(run, row, at));
-      }
+      const uint32_t n = unit / 2u * 16u + 4u * quarter;
+      f32x4 gate[1];
+      take_gates(gate, a, run, row0 + column, head, n);
+      store_four(a, run, row0 + column, head, n, sum * gate[0]);
     }
     __syncthreads();
   }
@@ -677,11 +753,11 @@ __device__ __forceinline__ void expand_unit(const AttentionArgs& args, uint32_t 
     weights[i] = static_cast<const i32x4*>(VALUES ? a.value_up : a.key_up) +
                  size_t{min(first_weight + i, weight_tiles - 1u)} * chunks * kWave + lane;
   // a wave fetches two of the eight token blocks
-  const i32x4* latents[2];
+  global_piece* latents[2];
 #pragma unroll
   for (uint32_t i = 0; i < 2u; ++i)
     latents[i] =
-        reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(
+        as_global(cache_block<const uint16_t>(
             a, args.tile0 * kTile + min(first_block + wave * 2u + i, blocks - 1u) * 16u)) +
         lane;
   f32x4 sum[WT][MB] = {};
@@ -771,11 +847,12 @@ template <int NK, int NV>
 __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs args) {
   constexpr int MT = 2;                                   // sixteen rows each, per wave
   constexpr int kFragments = 2 * NK + NV;
-  constexpr int kLoads = (kFragments + 3) / 4;            // fragments per wave and tile
+  constexpr int kLoads = kFragments / 4;                  // fragments per wave and tile
+  static_assert(kFragments % 4 == 0);
   __shared__ i32x4 staged[2][kFragments * kWave];
   const Latent& a = args.attention;
   const auto& run = args.launch;
-  const uint32_t wave = threadIdx.x / kWave;
+  const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
   const uint32_t lane = threadIdx.x % kWave;
   const uint32_t column = lane % 16u;
   const uint32_t quarter = lane / 16u;
@@ -800,8 +877,10 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
   const uint32_t begin = first_tile(a, first + block0);
   const uint32_t end = (first + last_row) / kTile + 1u;
 
-  for (uint32_t i = threadIdx.x; i < 2u * kFragments * kWave; i += blockDim.x)
-    staged[0][i] = i32x4{};
+  // No load depends on a condition - places past the end are clamped to one that
+  // exists - so that a wait for one tile's loads leaves the next one's in flight.
+  // Key chunks past the last one meet zeros of the query; value tiles past the last
+  // one end in sums that nobody reads.
   i32x4 q[MT][NK];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
@@ -811,49 +890,53 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
             32u +
         8u * quarter;
 #pragma unroll
-    for (int c = 0; c < NK; ++c)
-      q[m][c] = static_cast<uint32_t>(c) < key_chunks
-                    ? *reinterpret_cast<const i32x4*>(query + c * 32u)
-                    : i32x4{};
-  }
-  __syncthreads();   // what no load reaches is zero
-
-  // fragment f of a tile: half, key chunk; then value tiles
-  void* const* const pages = pages_of(a);
-  const auto fetch = [&](i32x4 (&loads)[kLoads], uint32_t tile) __attribute__((always_inline)) {
-    const size_t place = size_t{head} * args.tiles + (tile - args.tile0);
-    const i32x4* keys =
-        reinterpret_cast<const i32x4*>(args.keys + place * 2u * dim_chunks * kFragment);
-    const i32x4* values =
-        reinterpret_cast<const i32x4*>(args.values + place * tiles_v * kFragment);
-    const i32x4* cached =
-        rot_chunks
-            ? reinterpret_cast<const i32x4*>(cache_block<const uint16_t>(a, pages, tile * kTile))
-            : nullptr;
-#pragma unroll
-    for (int i = 0; i < kLoads; ++i) {
-      const uint32_t f = wave + 4u * i;
-      const uint32_t half = f / NK;
-      const uint32_t c = f % NK;
-      if (f < 2u * NK) {
-        if (c < dim_chunks)
-          loads[i] = keys[(half * dim_chunks + c) * kWave + lane];
-        else if (c < key_chunks)
-          loads[i] = cached[(half * (latent_chunks + rot_chunks) + latent_chunks + c -
-                             dim_chunks) * kWave + lane];
-      } else if (f - 2u * NK < tiles_v) {
-        loads[i] = values[(f - 2u * NK) * kWave + lane];
-      }
+    for (int c = 0; c < NK; ++c) {
+      const i32x4 stored = *reinterpret_cast<const i32x4*>(
+          query + min(static_cast<uint32_t>(c), key_chunks - 1u) * 32u);
+      q[m][c] = static_cast<uint32_t>(c) < key_chunks ? stored : i32x4{};
     }
+  }
+
+  // fragment f of a tile: half, key chunk; then value tiles.  A wave fetches every
+  // fourth: where it lies for the first tile (or in a tile's cache rows) and how far
+  // the next tile's is.
+  global_piece* source[kLoads];
+  uint32_t stride[kLoads];
+  uint32_t in_cache[kLoads];
+#pragma unroll
+  for (int i = 0; i < kLoads; ++i) {
+    const uint32_t f = wave + 4u * i;
+    const bool key = f < 2u * NK;
+    const uint32_t half = f / NK;
+    const uint32_t c = key ? min(f % NK, key_chunks - 1u) : 0u;
+    const uint32_t v = key ? 0u : min(f - 2u * NK, tiles_v - 1u);
+    const bool cached = key && c >= dim_chunks;
+    stride[i] = key ? 2u * dim_chunks * kWave : tiles_v * kWave;
+    const uint16_t* base = key ? args.keys : args.values;
+    source[i] = as_global(base) + size_t{head} * args.tiles * stride[i] +
+                (key ? (half * dim_chunks + (cached ? 0u : c)) * kWave : v * kWave) + lane;
+    in_cache[i] = cached ? (half * (latent_chunks + rot_chunks) + latent_chunks + c -
+                            dim_chunks) * kWave + lane
+                         : ~0u;
+  }
+  void* const* const pages = pages_of(a);
+  const auto page_for = [&](uint32_t tile) {
+    return as_global(cache_block<const uint16_t>(a, pages, min(tile, end - 1u) * kTile));
+  };
+  global_piece* ahead = page_for(begin);     // of the next fetch
+  const auto fetch = [&](i32x4 (&loads)[kLoads], uint32_t tile) __attribute__((always_inline)) {
+    global_piece* const rows = ahead;
+    ahead = page_for(tile + 1u);
+    const size_t ordinal = min(tile, end - 1u) - args.tile0;
+#pragma unroll
+    for (int i = 0; i < kLoads; ++i)
+      loads[i] = *(in_cache[i] == ~0u ? source[i] + ordinal * stride[i] : rows + in_cache[i]);
+    __builtin_amdgcn_sched_barrier(0);   // in this order
   };
   const auto publish = [&](const i32x4 (&loads)[kLoads], uint32_t slot)
       __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < kLoads; ++i) {
-      const uint32_t f = wave + 4u * i;
-      if (f < 2u * NK ? f % NK < key_chunks : f - 2u * NK < tiles_v)
-        staged[slot][f * kWave + lane] = loads[i];
-    }
+    for (int i = 0; i < kLoads; ++i) staged[slot][(wave + 4u * i) * kWave + lane] = loads[i];
   };
   const float unit = a.scale * kLog2e;
   // weights are taken relative to `base`, a maximum that may be out of date by
@@ -943,14 +1026,14 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
   // a tile is fetched two iterations and published one before its turn
   i32x4 even[kLoads], odd[kLoads];
   fetch(even, begin);
-  if (begin + 1u < end) fetch(odd, begin + 1u);
+  fetch(odd, begin + 1u);
   publish(even, 0u);
-  if (begin + 2u < end) fetch(even, begin + 2u);
+  fetch(even, begin + 2u);
   __syncthreads();
   const auto turn = [&](i32x4 (&loads)[kLoads], uint32_t tile) __attribute__((always_inline)) {
     compute(tile);
-    if (tile + 1u < end) publish(loads, (tile + 1u - begin) & 1u);
-    if (tile + 3u < end) fetch(loads, tile + 3u);
+    publish(loads, (tile + 1u - begin) & 1u);
+    fetch(loads, tile + 3u);
     __syncthreads();
   };
   for (uint32_t tile = begin; tile < end; tile += 2u) {
@@ -965,16 +1048,11 @@ __global__ __launch_bounds__(256, 2) void latent_prompt_kernel(AttentionArgs arg
     total[m] += __shfl_xor(total[m], 32, kWave);
     if (row >= run.rows) continue;
     const float inverse = 1.0f / total[m];
-    uint16_t* output =
-        static_cast<uint16_t*>(run.output) + size_t{row} * run.output_stride + head * a.vdim;
+    f32x4 gate[NV];
+    take_gates(gate, a, run, row, head, 4u * quarter);
 #pragma unroll
     for (int t = 0; t < NV; ++t)
-      for (uint32_t i = 0; i < 4u; ++i) {
-        const uint32_t n = t * 16u + 4u * quarter + i;
-        if (n < a.vdim)
-          store_element(output + n,
-                        out[m][t][i] * inverse * gate_of(run, row, head * a.vdim + n));
-      }
+      store_four(a, run, row, head, t * 16u + 4u * quarter, out[m][t] * inverse * gate[t]);
   }
 }
 
@@ -1009,7 +1087,9 @@ uint32_t splits_for(const Latent& a, uint32_t rows, uint32_t maximum_position) {
   const uint32_t most = 256u / item_tiles(a, rows);
   const uint32_t bound = most < 1u ? 1u : most < kMaximumSplits ? most : kMaximumSplits;
   const uint32_t tiles = maximum_tiles(a, rows, maximum_position);
-  return tiles < bound ? tiles : bound;
+  const uint32_t wanted =
+      tiles <= kSplitsFirst ? tiles : tiles / 4u > kSplitsFirst ? tiles / 4u : kSplitsFirst;
+  return wanted < bound ? wanted : bound;
 }
 
 size_t align16(size_t bytes) { return (bytes + 15u) / 16u * 16u; }

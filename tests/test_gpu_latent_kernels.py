@@ -310,6 +310,36 @@ def test_scores_that_grow_and_shrink_along_the_context(device, element):
                   factor=4.0 if element == F32 else 12.0)
 
 
+@pytest.mark.parametrize("rows", [1, 3, 40])
+def test_contexts_of_many_tiles(device, rows):
+    """More tiles than workgroups take one each; a key at the far end stands out."""
+    total = 9000 + rows
+    layer = Latent(device, BF16, 2, 32, 16, 16, 24, 64, 0, page_tokens=256, context=9216,
+                   scale=0.2)
+    rng = np.random.default_rng(1)
+    inputs = layer.inputs(rng, total)
+    c, shared = layer.cached(inputs[0])
+    for head, far in ((0, 5), (1, 7777)):
+        key = layer.keys(c, head)[far]
+        place = inputs[1][-1].reshape(2, 48)[head]
+        place[:] = 0.0
+        place[:32] = mm.bf16(16.0 * key / np.linalg.norm(key))
+    layer.run([a[:9000] for a in inputs], 0)
+    got = layer.run([a[9000:] for a in inputs], 9000)
+    for row in range(9000, total):
+        q = inputs[1][row].reshape(2, 48).astype(np.float64)
+        # the rotation of this row's position alone
+        turned = lo.rotate_halves(q[None, :, 32:], [row], layer.rot)[0]
+        want = []
+        for head in range(2):
+            v = c[:row + 1] @ layer.value_up[head * 24:(head + 1) * 24].T.astype(np.float64)
+            keys = np.concatenate([layer.keys(c[:row + 1], head), shared[:row + 1]], axis=1)
+            want.append(lo.attend(np.concatenate([q[head, :32], turned[head]])[None], keys, v,
+                                  layer.scale, np.ones((1, row + 1), dtype=bool))[0])
+        want = np.concatenate(want) * lo.logistic(inputs[2][row].astype(np.float64))
+        close(got[row - 9000], want, BF16, str(row), factor=2.0)
+
+
 def test_pages_and_slots_used_again(device):
     rng = np.random.default_rng(5)
     layer = Latent(device, BF16, 4, 32, 16, 16, 32, 80, 32, context=128, slots=2)
