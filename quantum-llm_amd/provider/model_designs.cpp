@@ -271,7 +271,7 @@ er::ModelDescriptor describe_zatupel(const json::Object& config,
 }
 
 // ---- Nametar -----------------------------------------------------------------
-// Layers with a norm before and after each sublayer: a mixer (latent attention
+// Sandwich layers, a norm on either side of a sublayer: a mixer (latent attention
 // without positions and with an output gate, windowed latent attention with a
 // query latent and a rotated shared key part, or gated linear attention), then a
 // gated feed-forward or none.

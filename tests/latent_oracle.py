@@ -1,7 +1,6 @@
 """A plain, slow statement of the latent-attention decoder in float64 NumPy:
 latent attention (with and without a query latent, rotated keys, a window, an
-output gate), gated linear attention, layers with a norm before and after each
-sublayer.
+output gate), gated linear attention, sublayers between two norms.
 
 One function per mechanism, each written from its equation and free of any code
 of the product path.
